@@ -21,7 +21,8 @@ A group with a window keeps, for each request, only pages that a future query
 can still see: before a step that starts at position ``s``, pages that lie wholly
 below ``s - window + 1`` go back to the allocator, and their table entries
 become -1.  A group whose queries see only their own block of ``chunk`` positions
-does the same with the pages below the start of the block that holds ``s``.
+does the same with the pages below the start of the block that holds ``s``.  The pages of the first positions
+that a group keeps visible (``PagedKVNeed.keep_first``) stay with the request.
 
 Beside the pages there are *slots*: one row of fixed size per running request
 and per stateful run of a layer, set to the state's initial value when a request gets its slot.  The
@@ -79,7 +80,12 @@ class PagedGroup:
         # positions, which touch at most that many / page_size pages plus one for misalignment.
         # (A block of positions in place of the window: from the block's start, at most as far back.)
         span = self.need.span + max_chunk - 1
-        return min(full, pages_for(span, self.page_size) + 1)
+        return min(full, pages_for(span, self.page_size) + 1 + self.kept_pages)
+
+    @property
+    def kept_pages(self) -> int:
+        """Pages at a sequence's start that no window gives back."""
+        return pages_for(self.need.keep_first, self.page_size)
 
     def begin(self, req: int, reserve: int) -> None:
         self.pool.open(req, reserve)
@@ -91,7 +97,7 @@ class PagedGroup:
         table = self.tables[req]
         if self.need.span is not None:
             first_visible = self.need.first_visible(start)
-            for idx in range(min(first_visible // self.page_size, len(table))):
+            for idx in range(self.kept_pages, min(first_visible // self.page_size, len(table))):
                 if table[idx] >= 0:
                     self.pool.drop(req, table[idx], restore_promise=True)
                     table[idx] = -1

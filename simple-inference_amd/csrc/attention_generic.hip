@@ -7,8 +7,9 @@
 // own position and keys only: not on how the prompt was cut into steps, on the other
 // rows of the batch, or on which pages hold the keys.
 //
-//   s_j = (q . k_j) * scale                                   scale after the dot
+//   s_j = (q . k_j) * scale                                   scale after the dot; with a cap s_j <- cap * tanh(s_j / cap)
 //   visible: j <= pos, and j > pos - window if window > 0, and j >= pos - pos % chunk if chunk > 0
+//            or j < keep_first with a window: the sequence's first positions stay visible
 //            (absolute positions are cut into blocks [b * chunk, (b + 1) * chunk): causal inside the block)
 //   online softmax over chunks: m' = max(m, max_j s_j); p_j = exp(s_j - m');
 //   l = l * exp(m - m') + sum_j p_j;  acc = acc * exp(m - m') + sum_j p_j v_j;  o = acc / l
@@ -26,7 +27,8 @@ __global__ __launch_bounds__(SIA_WAVE) void attention_generic_kernel(
     const T* __restrict__ q, int q_row_stride, const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     const int* __restrict__ block_table, int table_width, const int* __restrict__ seq_of_token,
     const int* __restrict__ positions, T* __restrict__ out, int n_heads, int n_kv, int head_dim,
-    int value_dim, int page_size, float scale, int window, int chunk, const float* __restrict__ sinks) {
+    int value_dim, int page_size, float scale, int window, int chunk, const float* __restrict__ sinks, float cap,
+    int keep_first) {
     __shared__ float q_s[ATTN_MAX_HEAD_DIM];
     __shared__ float p_s[SIA_WAVE];
     __shared__ int page_s[SIA_WAVE];
@@ -46,9 +48,11 @@ __global__ __launch_bounds__(SIA_WAVE) void attention_generic_kernel(
     float m = -INFINITY, l = 0.f;
     float acc[ATTN_MAX_HEAD_DIM / SIA_WAVE] = {};
 
-    for (int c0 = (lo / SIA_WAVE) * SIA_WAVE; c0 <= pos; c0 += SIA_WAVE) {
+    // the chunks of the kept first positions, then those from the window's first chunk on: every one holds a visible key
+    const int keep = min(keep_first, lo), c_lo = (lo / SIA_WAVE) * SIA_WAVE;
+    for (int c0 = keep > 0 ? 0 : c_lo; c0 <= pos; c0 = c0 + SIA_WAVE < keep ? c0 + SIA_WAVE : max(c0 + SIA_WAVE, c_lo)) {
         const int j = c0 + lane;
-        const bool visible = j >= lo && j <= pos;
+        const bool visible = (j >= lo || j < keep) && j <= pos;
         float s = -INFINITY;
         int page = -1;
         if (visible) page = table[j / page_size];
@@ -57,6 +61,7 @@ __global__ __launch_bounds__(SIA_WAVE) void attention_generic_kernel(
             float dot = 0.f;
             for (int d = 0; d < head_dim; ++d) dot += q_s[d] * to_float(kp[d]);
             s = dot * scale;
+            if (cap > 0.f) s = cap * tanhf(s / cap);
         }
         const float m_new = fmaxf(m, wave_max(s));  // finite: every chunk holds a visible key
         const float p = (visible && page >= 0) ? expf(s - m_new) : 0.f;
@@ -66,7 +71,8 @@ __global__ __launch_bounds__(SIA_WAVE) void attention_generic_kernel(
         p_s[lane] = p;
         page_s[lane] = page;
         __syncthreads();
-        const int j_first = max(lo, c0) - c0, j_last = min(pos, c0 + SIA_WAVE - 1) - c0;
+        // the invisible keys between the kept ones and the window have weight 0 and may have no page
+        const int j_first = c0 < keep ? 0 : max(lo, c0) - c0, j_last = min(pos, c0 + SIA_WAVE - 1) - c0;
 #pragma unroll
         for (int dd = 0; dd < ATTN_MAX_HEAD_DIM / SIA_WAVE; ++dd) {
             const int d = lane + dd * SIA_WAVE;
@@ -103,16 +109,17 @@ SIA_EXPORT int sia_attention_generic(const void* q, int q_row_stride, const void
                                      const int* block_table, int table_width, const int* seq_of_token,
                                      const int* positions, void* out, int n_tokens, int n_heads, int n_kv,
                                      int head_dim, int value_dim, int page_size, float scale, int window, int chunk,
-                                     const float* sinks, int dtype, hipStream_t stream) {
+                                     const float* sinks, float cap, int keep_first, int dtype, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (head_dim <= 0 || head_dim > ATTN_MAX_HEAD_DIM || value_dim <= 0 || value_dim > ATTN_MAX_HEAD_DIM || n_kv <= 0 || n_heads % n_kv || page_size <= 0 ||
-        n_heads > 65535)
+        n_heads > 65535 || cap < 0.f || keep_first < 0)
         return SIA_BAD_ARGUMENT;
     dim3 grid(n_tokens, n_heads), block(SIA_WAVE);
 #define LAUNCH(T)                                                                                              \
     hipLaunchKernelGGL(attention_generic_kernel<T>, grid, block, 0, stream, (const T*)q, q_row_stride,         \
                        (const T*)k_pages, (const T*)v_pages, block_table, table_width, seq_of_token, positions, \
-                       (T*)out, n_heads, n_kv, head_dim, value_dim, page_size, scale, window, chunk, sinks)
+                       (T*)out, n_heads, n_kv, head_dim, value_dim, page_size, scale, window, chunk, sinks, cap, \
+                       keep_first)
     if (dtype == SIA_F32) LAUNCH(float);
     else if (dtype == SIA_BF16) LAUNCH(bf16_t);
     else return SIA_BAD_ARGUMENT;

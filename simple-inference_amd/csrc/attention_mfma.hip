@@ -26,6 +26,15 @@
 // probabilities are rounded to bfloat16 for the value product (reference:
 // kernels/attention_kernel.py:184-251 does the same in its prefill kernel).
 //
+// Built with -DSIA_SCORE_FORMS=1 the kernels also take a soft cap on the scores and first positions that stay visible
+// behind a window; built without, none of the code of these two forms is there.
+//   cap:        the scaled score s becomes cap * tanh(s / cap) before the softmax.
+//   keep_first: a query sees j < keep_first beside its window.  The kernels walk *places*: place x is position x up to
+//               a boundary behind the kept positions, and position x + gap beyond it, with the gap (whole pages, whole
+//               tiles) chosen so that the places after the boundary begin at or just below the window.  Tiles, masks
+//               and splits are taken in places, as if the keys in between did not exist; only the block table is
+//               looked up in positions.  Tiles still begin at positions that are multiples of 32.
+//
 // decode:  workgroups of four waves; a (kv head, sequence) is shared by as many of them ("splits") as its own
 //          number of visible key tiles says (decode_splits below: a power of two that leaves a wave some four
 //          tiles), never by how many sequences the step holds or how long the others are: the grid is sized for
@@ -44,6 +53,10 @@
 #error "compile with -DSIA_HEAD_DIM=<head size>"
 #endif
 
+#ifndef SIA_SCORE_FORMS
+#define SIA_SCORE_FORMS 0
+#endif
+constexpr bool FORMS = SIA_SCORE_FORMS != 0;
 constexpr int HD = SIA_HEAD_DIM;
 static_assert(HD % 16 == 0 && HD >= 16 && HD <= 256, "head size must be a multiple of 16 up to 256");
 constexpr int KSTEPS = (HD + 31) / 32;
@@ -78,6 +91,35 @@ __device__ __forceinline__ int first_visible(int pos, int window, int chunk) {
     return lo;
 }
 
+// What the two forms add to a kernel's arguments.
+struct Forms {
+    float rate;       // scale / cap, or 0: no cap
+    int keep_first;
+};
+
+// Places: place x is position x for x < edge and position x + gap beyond.
+struct Places {
+    int edge, gap;
+};
+
+// lo: the oldest position of the window (of the first query of a workgroup).
+__device__ __forceinline__ Places places_of(int lo, int keep_first, int ps_log2) {
+    if (!FORMS || keep_first <= 0) return Places{0, 0};
+    const int unit = max(1 << ps_log2, TILE);     // both powers of two
+    const int edge = (keep_first + unit - 1) & -unit;
+    return Places{edge, max(0, (lo & -unit) - edge)};
+}
+
+// The first place of the walk that serves a window from place lo on.
+__device__ __forceinline__ int walk_begin(int lo, int keep_first) { return FORMS && keep_first > 0 ? 0 : lo; }
+
+// A capped score: tanh of the dot product times `rate` (the cap itself and the change to units of log2 are in the
+// softmax's scale).  tanh(x) = 1 - 2 / (e^(2x) + 1), whose absolute error is that of a rounding near 1.
+__device__ __forceinline__ float capped(float s, float rate) {
+    const float e = __builtin_amdgcn_exp2f(s * rate * (2.f * 1.4426950408889634f));
+    return 1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f);
+}
+
 // A sink's term of a softmax denominator: sinks[head] is a learned logit of that query head (natural units; the
 // score scale does not apply) that takes a share of the weight and carries no value.  Exponentials are taken as 2^(x - ref) with ref in units of log2.
 __device__ __forceinline__ float sink_term(const float* __restrict__ sinks, int head, float ref) {
@@ -106,14 +148,16 @@ __device__ __forceinline__ float column_sum(float v) {
 
 // 64 consecutive entries of a sequence's block table, one per lane.
 struct PageWindow {
-    int base;  // index of the entry that lane 0 holds
+    int base;  // index (among the pages of places) of the entry that lane 0 holds
     int mine;
 };
 
 __device__ __forceinline__ void pages_load(PageWindow& w, const int* __restrict__ table, int table_width,
-                                           int first, int lane) {
+                                           int first, int lane, int ps_log2, const Places& places) {
     w.base = first;
-    w.mine = table[min(first + lane, table_width - 1)];
+    int index = first + lane;
+    if (FORMS && index >= places.edge >> ps_log2) index += places.gap >> ps_log2;
+    w.mine = table[min(index, table_width - 1)];
 }
 
 __device__ __forceinline__ int pages_get(const PageWindow& w, int index) {
@@ -196,25 +240,32 @@ __device__ __forceinline__ float max2(float a, float b) { return __builtin_fmaxf
 
 // Masks the scores of a tile, updates the softmax state of each q column, rescales the accumulators where a
 // reference moved, and returns the tile's probabilities as the P^T operand.
-//   lo[n], hi[n]: visible keys of this lane's column in group n (hi < lo: none).
+//   lo[n], hi[n]: visible keys of this lane's column in group n (hi < lo: none); those below forms.keep_first are visible
+//   up to hi[n] too.
 //   scale_log2 = scale * log2(e) > 0.
 // A tile that every column of the wave sees whole skips the masking (the test is wave-uniform).
 template <int NQ>
 __device__ __forceinline__ void softmax_update(floatx4 (&s)[NQ][2], int kb, const int (&lo)[NQ], const int (&hi)[NQ],
                                                float scale_log2, Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS],
-                                               bf16x8 (&p)[NQ]) {
+                                               bf16x8 (&p)[NQ], const Forms& forms) {
     const int g = (threadIdx.x & 63) >> 4;
     float top[NQ];
     bool grew = false;
 #pragma unroll
     for (int n = 0; n < NQ; ++n) {
-        if (!__all(kb >= lo[n] && kb + TILE - 1 <= hi[n])) {
+        if (FORMS && forms.rate > 0.f) {
+#pragma unroll
+            for (int h = 0; h < 2; ++h)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) s[n][h][i] = capped(s[n][h][i], forms.rate);
+        }
+        if (!__all((kb >= lo[n] || (FORMS && kb + TILE <= forms.keep_first)) && kb + TILE - 1 <= hi[n])) {
 #pragma unroll
             for (int h = 0; h < 2; ++h)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int key = kb + g * 8 + h * 4 + i;
-                    if (key < lo[n] || key > hi[n]) s[n][h][i] = -INFINITY;
+                    if ((key < lo[n] && !(FORMS && key < forms.keep_first)) || key > hi[n]) s[n][h][i] = -INFINITY;
                 }
         }
         top[n] = max2(max2(max2(s[n][0][0], s[n][0][1]), max2(s[n][0][2], s[n][0][3])),
@@ -259,7 +310,7 @@ __device__ __forceinline__ void softmax_update(floatx4 (&s)[NQ][2], int kb, cons
 template <int NQ>
 __device__ __forceinline__ void compute_stage(const Stage& st, const bf16x8 (&q)[NQ][KSTEPS], int kb,
                                               const int (&lo)[NQ], const int (&hi)[NQ], float scale,
-                                              Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS]) {
+                                              Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS], const Forms& forms) {
     floatx4 s[NQ][2];
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
@@ -272,7 +323,7 @@ __device__ __forceinline__ void compute_stage(const Stage& st, const bf16x8 (&q)
                 s[n][h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(st.k[h][ks], q[n][ks], s[n][h], 0, 0, 0);
     }
     bf16x8 p[NQ];
-    softmax_update<NQ>(s, kb, lo, hi, scale, sm, acc, p);
+    softmax_update<NQ>(s, kb, lo, hi, scale, sm, acc, p, forms);
 #pragma unroll
     for (int db = 0; db < DBLOCKS; ++db)
 #pragma unroll
@@ -293,19 +344,20 @@ __device__ __forceinline__ void attend_tiles(const PageWindow& pages, int w_firs
                                              const bf16x8 (&q)[NQ][KSTEPS], const bf16_t* __restrict__ kp,
                                              const bf16_t* __restrict__ vp, int ps_log2, int n_kv, int hk,
                                              int range_lo, int range_hi, const int (&lo)[NQ], const int (&hi)[NQ],
-                                             float scale, Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS], Hook& before) {
+                                             float scale, Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS], Hook& before,
+                                             const Forms& forms) {
     Stage a, b;
     load_stage(a, kp, vp, pages, ps_log2, n_kv, hk, w_first, range_lo, range_hi);
     for (int kb = w_first; kb <= w_last; kb += 2 * TILE) {
         const int kb1 = min(kb + TILE, w_last);  // past the end: the last tile again, never computed
         load_stage(b, kp, vp, pages, ps_log2, n_kv, hk, kb1, range_lo, range_hi);
         before(kb);
-        compute_stage<NQ>(a, q, kb, lo, hi, scale, sm, acc);
+        compute_stage<NQ>(a, q, kb, lo, hi, scale, sm, acc, forms);
         const int kb2 = min(kb + 2 * TILE, w_last);
         load_stage(a, kp, vp, pages, ps_log2, n_kv, hk, kb2, range_lo, range_hi);
         if (kb + TILE <= w_last) {
             before(kb + TILE);
-            compute_stage<NQ>(b, q, kb + TILE, lo, hi, scale, sm, acc);
+            compute_stage<NQ>(b, q, kb + TILE, lo, hi, scale, sm, acc, forms);
         }
     }
 }
@@ -318,16 +370,17 @@ __device__ __forceinline__ void attend_range(const bf16x8 (&q)[NQ][KSTEPS], cons
                                              const bf16_t* __restrict__ vp, const int* __restrict__ table,
                                              int table_width, int ps_log2, int n_kv, int hk, int range_lo,
                                              int range_hi, const int (&lo)[NQ], const int (&hi)[NQ], float scale,
-                                             Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS], Hook& before) {
+                                             Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS], Hook& before,
+                                             const Forms& forms, const Places& places) {
     const int lane = threadIdx.x & 63;
     const int kb_first = (range_lo / TILE) * TILE, kb_last = (range_hi / TILE) * TILE;
     for (int w_first = kb_first; w_first <= kb_last;) {
         const int first_page = w_first >> ps_log2;
         const int w_end = (first_page + SIA_WAVE) << ps_log2;  // first key beyond the window, a multiple of TILE
         PageWindow pages;
-        pages_load(pages, table, table_width, first_page, lane);
+        pages_load(pages, table, table_width, first_page, lane, ps_log2, places);
         attend_tiles<NQ>(pages, w_first, min(kb_last, w_end - TILE), q, kp, vp, ps_log2, n_kv, hk, range_lo, range_hi,
-                         lo, hi, scale, sm, acc, before);
+                         lo, hi, scale, sm, acc, before, forms);
         w_first = w_end;
     }
 }
@@ -337,10 +390,11 @@ __device__ __forceinline__ void attend_range(const bf16x8 (&q)[NQ][KSTEPS], cons
                                              const bf16_t* __restrict__ vp, const int* __restrict__ table,
                                              int table_width, int ps_log2, int n_kv, int hk, int range_lo,
                                              int range_hi, const int (&lo)[NQ], const int (&hi)[NQ], float scale,
-                                             Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS]) {
+                                             Softmax<NQ>& sm, floatx4 (&acc)[NQ][DBLOCKS], const Forms& forms,
+                                             const Places& places) {
     NoHook none;
     attend_range<NQ>(q, kp, vp, table, table_width, ps_log2, n_kv, hk, range_lo, range_hi, lo, hi, scale, sm, acc,
-                     none);
+                     none, forms, places);
 }
 
 // q operand of column r: 8 dims d0 .. d0+7 of that column's query row (zeros if the column is unused).
@@ -446,7 +500,7 @@ __global__ __launch_bounds__(DEC_WAVES* SIA_WAVE) void attn_decode_kernel(
     const int* __restrict__ block_table, int table_width, const int* __restrict__ cu_q,
     const int* __restrict__ kv_len, float* __restrict__ ws_acc, float* __restrict__ ws_ml,
     bf16_t* __restrict__ out, int n_heads, int n_kv, int ps_log2, float scale, int window, int chunk,
-    const float* __restrict__ sinks, int max_splits, int mode, int kv_share) {
+    const float* __restrict__ sinks, int max_splits, int mode, int kv_share, const Forms forms) {
     const bool fold = mode == DEC_FOLD, spread = mode == DEC_SPREAD;
     static_assert(DEC_WAVES == 4, "merge_waves merges four runs");
     extern __shared__ float lds[];  // [runs of the workgroup][group][HD + 2]
@@ -454,8 +508,10 @@ __global__ __launch_bounds__(DEC_WAVES* SIA_WAVE) void attn_decode_kernel(
     // have) then come last, not interleaved with the others, which the chip deals out to its dies in turn
     const int hk = blockIdx.x, seq = blockIdx.y;
     const int wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
-    const int pos = kv_len[seq] - 1;
-    const int lo_all = first_visible(pos, window, chunk);
+    const int last_pos = kv_len[seq] - 1, oldest = first_visible(last_pos, window, chunk);
+    const Places places = places_of(oldest, forms.keep_first, ps_log2);
+    const int pos = last_pos - places.gap, lo_win = oldest - places.gap;     // from here on in places
+    const int lo_all = walk_begin(lo_win, forms.keep_first);
     const int t_first = lo_all / TILE, n_tiles = pos / TILE - t_first + 1;
     const int n_splits = min(decode_splits(n_tiles), max_splits);
     // the whole workgroup leaves: the grid is sized for the longest sequence there may be
@@ -504,9 +560,10 @@ __global__ __launch_bounds__(DEC_WAVES* SIA_WAVE) void attn_decode_kernel(
 
     if (first < end) {  // wave-uniform
         const int w_lo = max(lo_all, first * TILE), w_hi = min(pos, end * TILE - 1);
-        const int lo[1] = {r < group ? w_lo : 1}, hi[1] = {r < group ? w_hi : 0};
+        const int mask_lo = FORMS && forms.keep_first > 0 ? lo_win : w_lo;
+        const int lo[1] = {r < group ? mask_lo : 1 << 30}, hi[1] = {r < group ? w_hi : -1};
         attend_range<1>(qf, kp, vp, table, table_width, ps_log2, n_kv / kv_share, hk / kv_share, w_lo, w_hi, lo, hi, scale, sm, acc,
-                        at_run_ends);
+                        at_run_ends, forms, places);
     }
     while (at_run_ends.done < mine_n - 1) at_run_ends.pass();  // runs without tiles of their own
     if (spread) {  // the run's state of every query head of the group: [sequence][head][run][HD + 2] in ws_acc
@@ -549,10 +606,12 @@ __global__ __launch_bounds__(DEC_WAVES* SIA_WAVE) void attn_decode_kernel(
 __global__ __launch_bounds__(SIA_WAVE) void attn_decode_combine_kernel(
     const float* __restrict__ ws_acc, const float* __restrict__ ws_ml, const int* __restrict__ cu_q,
     const int* __restrict__ kv_len, bf16_t* __restrict__ out, int n_heads, int max_splits, int window, int chunk,
-    const float* __restrict__ sinks, int runs) {
+    const float* __restrict__ sinks, int runs, int ps_log2, const Forms forms) {
     const int head = blockIdx.x, seq = blockIdx.y, lane = threadIdx.x;
-    const int pos = kv_len[seq] - 1;
-    const int lo_all = first_visible(pos, window, chunk);
+    const int last_pos = kv_len[seq] - 1, oldest = first_visible(last_pos, window, chunk);
+    const Places places = places_of(oldest, forms.keep_first, ps_log2);
+    const int pos = last_pos - places.gap;
+    const int lo_all = walk_begin(oldest - places.gap, forms.keep_first);
     const int n_splits = min(decode_splits(pos / TILE - lo_all / TILE + 1), max_splits);
     bf16_t* dst = out + ((size_t)cu_q[seq] * n_heads + head) * HD;
     if (runs) {
@@ -708,7 +767,7 @@ template <int NQ, bool EARLY>
 __device__ __forceinline__ void compute_from_lds(const bf16_t* __restrict__ k_lds, const bf16_t* __restrict__ v_lds,
                                                  const bf16x8 (&q)[NQ][KSTEPS], int kb, const int (&lo)[NQ],
                                                  const int (&hi)[NQ], float scale, Softmax<NQ>& sm,
-                                                 floatx4 (&acc)[NQ][DBLOCKS]) {
+                                                 floatx4 (&acc)[NQ][DBLOCKS], const Forms& forms) {
     const int lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
     auto key_operand = [&](int h, int ks) {
         const int d0 = ks * 32 + g * 8;
@@ -740,7 +799,7 @@ __device__ __forceinline__ void compute_from_lds(const bf16_t* __restrict__ k_ld
         for (int db = 0; db < DBLOCKS; ++db) va[db] = value_operand(db);
     }
     bf16x8 p[NQ];
-    softmax_update<NQ>(s, kb, lo, hi, scale, sm, acc, p);
+    softmax_update<NQ>(s, kb, lo, hi, scale, sm, acc, p, forms);
 #pragma unroll
     for (int db = 0; db < DBLOCKS; ++db) {
         const bf16x8 a = EARLY ? va[db] : value_operand(db);
@@ -758,7 +817,7 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
     const bf16_t* __restrict__ q, int q_row_stride, const bf16_t* __restrict__ kp, const bf16_t* __restrict__ vp,
     const int* __restrict__ block_table, int table_width, const int* __restrict__ cu_q,
     const int* __restrict__ kv_len, bf16_t* __restrict__ out, int n_heads, int n_kv, int ps_log2, float scale,
-    int window, int chunk, const float* __restrict__ sinks, int seq_begin, int seq_end) {
+    int window, int chunk, const float* __restrict__ sinks, int seq_begin, int seq_end, const Forms forms) {
     constexpr int ROW_WAVES = PF_WAVES / KSPLIT;
     constexpr int ROWS = ROW_WAVES * PF_NQ * 16;
     constexpr int TEAM = PF_WAVES * SIA_WAVE;
@@ -796,7 +855,11 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
     const int wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
     const int row_wave = wave % ROW_WAVES, part = wave / ROW_WAVES;  // which tokens, which tiles of a step
     const int q_begin = cu_q[seq], q_len = cu_q[seq + 1] - q_begin;
-    const int first_pos = kv_len[seq] - q_len;
+    // the workgroup's rows leave out what its first row, which sees furthest back, leaves out; from here on in places
+    const int first_at = kv_len[seq] - q_len;
+    const Places places = places_of(first_visible(first_at + tile * ROWS, window, chunk), forms.keep_first, ps_log2);
+    const int first_pos = first_at - places.gap;
+    auto oldest_of = [&](int place) { return first_visible(place + places.gap, window, chunk) - places.gap; };
     const int row0 = tile * ROWS + row_wave * PF_NQ * 16;  // this wave's first row within the sequence's run
     const bool wave_live = row0 < q_len;
     const int row_last = min(q_len - 1, row0 + PF_NQ * 16 - 1);
@@ -813,8 +876,8 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
         const bool live = row < q_len;
         const int qpos = first_pos + row;
         load_q(qf[n], live ? q + (size_t)(q_begin + row) * q_row_stride + head * HD : nullptr, g);
-        hi[n] = live ? qpos : 0;
-        lo[n] = live ? first_visible(qpos, window, chunk) : 1;
+        hi[n] = live ? qpos : -1;
+        lo[n] = live ? oldest_of(qpos) : 1 << 30;
 #pragma unroll
         for (int db = 0; db < DBLOCKS; ++db) acc[n][db] = floatx4{0.f, 0.f, 0.f, 0.f};
     }
@@ -828,9 +891,9 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
         // the workgroup's key range: from the first row's oldest visible key to the last live row's position
         const int blk_rows = min(q_len - tile * ROWS, ROWS);
         const int blk_hi = first_pos + tile * ROWS + blk_rows - 1;
-        const int blk_lo = first_visible(first_pos + tile * ROWS, window, chunk);
+        const int blk_lo = walk_begin(oldest_of(first_pos + tile * ROWS), forms.keep_first);
         const int wave_hi = first_pos + row_last;
-        const int wave_lo = first_visible(first_pos + row0, window, chunk);
+        const int wave_lo = oldest_of(first_pos + row0);
         const int kb_first = (blk_lo / TILE) * TILE, kb_last = (blk_hi / TILE) * TILE;
         constexpr int STEP_KEYS = KTILES * TILE;
         constexpr int AHEAD = PF_NQ == 1 ? 4 : 2;
@@ -850,7 +913,7 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
             w_end = (first_page + SIA_WAVE) << ps_log2;  // first key beyond the window, a multiple of TILE
             const int w_last = min(kb_last, w_end - TILE);
             PageWindow pages;
-            pages_load(pages, table, table_width, first_page, lane);
+            pages_load(pages, table, table_width, first_page, lane, ps_log2, places);
             TileRegs<TEAM> regs[AHEAD][KTILES];
             int found[KTILES][TileRegs<TEAM>::PER_THREAD];  // pages of the tiles whose loads are issued next
 // One step: issue the loads of the tiles AHEAD steps ahead into FREE (whose tiles are in LDS by now; their pages
@@ -869,7 +932,9 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
 #define PF_STORE(SET, KB, STAGE)                                                                                \
     _Pragma("unroll") for (int p = 0; p < KTILES; ++p)                                                          \
         if ((KB) + p * TILE <= w_last) tile_store(SET[p], PF_K_LDS(STAGE, p), PF_V_LDS(STAGE, p), ps_log2)
-#define PF_LIVE(MY_KB) (wave_live && (MY_KB) <= w_last && (MY_KB) <= wave_hi && (MY_KB) + TILE - 1 >= wave_lo)
+#define PF_LIVE(MY_KB)                                                                                          \
+    (wave_live && (MY_KB) <= w_last && (MY_KB) <= wave_hi &&                                                    \
+     ((MY_KB) + TILE - 1 >= wave_lo || (FORMS && (MY_KB) < forms.keep_first)))
 #define PF_STEP(FREE, NEXT, KB, STAGE)                                                                          \
     do {                                                                                                        \
         PF_FETCH(FREE, (KB) + AHEAD * STEP_KEYS);                                                               \
@@ -878,13 +943,13 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
             const int mine = KSPLIT == 2 ? part : 0, my_kb = (KB) + mine * TILE;                                \
             if (PF_LIVE(my_kb))                                                                                 \
                 compute_from_lds<PF_NQ, EARLY>(PF_K_LDS(STAGE, mine), PF_V_LDS(STAGE, mine), qf, my_kb, lo, hi, \
-                                               scale, sm, acc);                                                 \
+                                               scale, sm, acc, forms);                                          \
         } else {                                                                                                \
             _Pragma("unroll") for (int p = 0; p < KTILES; ++p) {                                                \
                 const int my_kb = (KB) + p * TILE;                                                              \
                 if (PF_LIVE(my_kb))                                                                             \
                     compute_from_lds<PF_NQ, EARLY>(PF_K_LDS(STAGE, p), PF_V_LDS(STAGE, p), qf, my_kb, lo, hi,   \
-                                                   scale, sm, acc);                                             \
+                                                   scale, sm, acc, forms);                                      \
             }                                                                                                   \
         }                                                                                                       \
         PF_STORE(NEXT, (KB) + STEP_KEYS, (STAGE) ^ 1);                                                          \
@@ -917,9 +982,9 @@ __global__ __launch_bounds__(PF_WAVES* SIA_WAVE) void attn_prefill_kernel(
         static_assert(PF_USE_LDS || KSPLIT == 1, "the split shape stages its tiles through LDS");
         if (wave_live) {
             const int range_hi = first_pos + row_last;
-            const int range_lo = first_visible(first_pos + row0, window, chunk);
+            const int range_lo = walk_begin(oldest_of(first_pos + row0), forms.keep_first);
             attend_range<PF_NQ>(qf, kp, vp, table, table_width, ps_log2, n_kv, hk, range_lo, range_hi, lo, hi, scale,
-                                sm, acc);
+                                sm, acc, forms, places);
         }
     }
     sm.finish_sums();
@@ -997,6 +1062,29 @@ static int log2_exact(int v) {
 }
 
 SIA_EXPORT int sia_attn_mfma_head_dim() { return HD; }
+SIA_EXPORT int sia_attn_mfma_forms() { return FORMS ? 1 : 0; }
+
+// The two forms' arguments as the kernels take them; false if this build does not have them or they do not fit.
+// With a cap `scale` becomes what the softmax multiplies a capped score by.
+static bool make_forms(float softcap, int keep_first, int window, int chunk, float& scale, Forms& forms) {
+    forms = Forms{0.f, 0};
+    if (softcap == 0.f && keep_first == 0) return true;
+    if (!FORMS || softcap < 0.f || keep_first < 0 || (keep_first > 0 && (window <= 0 || chunk > 0))) return false;
+    forms.keep_first = keep_first;
+    if (softcap > 0.f) {
+        forms.rate = scale / softcap;
+        scale = softcap;
+    }
+    return true;
+}
+
+// The most places a query's walk passes with such a window and kept first positions: what sia_attn_decode_max_splits
+// takes for the window.
+SIA_EXPORT int sia_attn_decode_walk(int window, int keep_first, int page_size) {
+    if (window <= 0 || keep_first <= 0) return window;
+    const int unit = max(page_size, TILE);
+    return window + (keep_first + unit - 1) / unit * unit + unit;
+}
 
 // Most workgroups that share one (sequence, kv head) when no sequence of the step holds more than kv_bound keys
 // (with a window: sees more than the window; for queries that see a block of positions `window` is the block's
@@ -1045,12 +1133,16 @@ SIA_EXPORT long long sia_attn_decode_workspace(int n_seqs, int n_heads, int n_kv
 // are given); sinks: one float per query head that joins its softmax's denominator, or null.
 // kv_share > 1: the pages hold n_kv / kv_share key/value heads, and each is read by kv_share of the launch's n_kv
 // groups of query heads (more than 16 query heads on one key/value head are dealt out as several groups).
-SIA_EXPORT int sia_attn_decode_shared(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
-                                      const int* block_table, int table_width, const int* cu_q, const int* kv_len,
-                                      void* out, float* ws_acc, float* ws_ml, int n_seqs, int n_heads, int n_kv,
-                                      int kv_share, int page_size, float scale, int window, int chunk,
-                                      const float* sinks, int max_splits, hipStream_t stream) {
+// softcap, keep_first: the two forms of a build that has them (0: none).
+SIA_EXPORT int sia_attn_decode_forms(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
+                                     const int* block_table, int table_width, const int* cu_q, const int* kv_len,
+                                     void* out, float* ws_acc, float* ws_ml, int n_seqs, int n_heads, int n_kv,
+                                     int kv_share, int page_size, float scale, int window, int chunk,
+                                     const float* sinks, float softcap, int keep_first, int max_splits,
+                                     hipStream_t stream) {
     if (n_seqs <= 0) return 0;
+    Forms forms;
+    if (!make_forms(softcap, keep_first, window, chunk, scale, forms)) return SIA_BAD_ARGUMENT;
     const int ps_log2 = log2_exact(page_size);
     const int n_splits = max_splits;
     if (ps_log2 < 3 || n_kv <= 0 || n_heads % n_kv || n_heads / n_kv > 16 || n_splits <= 0 || kv_share <= 0 ||
@@ -1083,12 +1175,22 @@ SIA_EXPORT int sia_attn_decode_shared(const void* q, int q_row_stride, const voi
                        mode == DEC_SPREAD ? 0 : lds_bytes, stream, (const bf16_t*)q, q_row_stride,
                        (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_table, table_width, cu_q, kv_len, ws_acc,
                        ws_ml, (bf16_t*)out, n_heads, n_kv, ps_log2, scale, window, chunk, sinks, n_splits, (int)mode,
-                       kv_share);
+                       kv_share, forms);
     if (mode == DEC_SPREAD || (mode == DEC_PLAIN && n_splits > 1))
         hipLaunchKernelGGL(attn_decode_combine_kernel, dim3(n_heads, n_seqs), dim3(SIA_WAVE), 0, stream, ws_acc,
                            ws_ml, cu_q, kv_len, (bf16_t*)out, n_heads, n_splits, window, chunk, sinks,
-                           mode == DEC_SPREAD ? 1 : 0);
+                           mode == DEC_SPREAD ? 1 : 0, ps_log2, forms);
     return SIA_LAUNCH_CHECK();
+}
+
+SIA_EXPORT int sia_attn_decode_shared(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
+                                      const int* block_table, int table_width, const int* cu_q, const int* kv_len,
+                                      void* out, float* ws_acc, float* ws_ml, int n_seqs, int n_heads, int n_kv,
+                                      int kv_share, int page_size, float scale, int window, int chunk,
+                                      const float* sinks, int max_splits, hipStream_t stream) {
+    return sia_attn_decode_forms(q, q_row_stride, k_pages, v_pages, block_table, table_width, cu_q, kv_len, out, ws_acc,
+                                 ws_ml, n_seqs, n_heads, n_kv, kv_share, page_size, scale, window, chunk, sinks, 0.f, 0,
+                                 max_splits, stream);
 }
 
 SIA_EXPORT int sia_attn_decode_ex(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
@@ -1120,7 +1222,7 @@ template <int NQ, int WAVES, int KSPLIT, int KTILES = KSPLIT>
 static int launch_prefill(int tiles, const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
                           const int* block_table, int table_width, const int* cu_q, const int* kv_len, void* out,
                           int seq_begin, int seq_end, int n_heads, int n_kv, int ps_log2, float scale, int window,
-                          int chunk, const float* sinks, hipStream_t stream) {
+                          int chunk, const float* sinks, const Forms& forms, hipStream_t stream) {
     constexpr int TILE_ELEMS = TILE * K_STRIDE + HD * V_STRIDE;
     size_t lds_bytes = PF_USE_LDS ? (size_t)2 * KTILES * TILE_ELEMS * sizeof(bf16_t) : 0;
     if (KSPLIT == 2) {
@@ -1135,7 +1237,7 @@ static int launch_prefill(int tiles, const void* q, int q_row_stride, const void
     hipLaunchKernelGGL((attn_prefill_kernel<NQ, WAVES, KSPLIT, KTILES>), dim3(tiles, n_heads), dim3(WAVES * SIA_WAVE),
                        lds_bytes, stream, (const bf16_t*)q, q_row_stride, (const bf16_t*)k_pages,
                        (const bf16_t*)v_pages, block_table, table_width, cu_q, kv_len, (bf16_t*)out, n_heads, n_kv,
-                       ps_log2, scale, window, chunk, sinks, seq_begin, seq_end);
+                       ps_log2, scale, window, chunk, sinks, seq_begin, seq_end, forms);
     return SIA_LAUNCH_CHECK();
 }
 
@@ -1171,17 +1273,20 @@ static PrefillShape prefill_shape(int n_tiles, int n_tiles_split, int n_tiles_lo
     return PF_WIDE;
 }
 
-SIA_EXPORT int sia_attn_prefill_ex(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
+SIA_EXPORT int sia_attn_prefill_forms(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
                                    const int* block_table, int table_width, const int* cu_q, const int* kv_len,
                                    void* out, int seq_begin, int seq_end, int n_tiles, int n_tiles_split,
                                    int n_tiles_long, int q_bound, int kv_bound, int n_heads, int n_kv, int page_size,
-                                   float scale, int window, int chunk, const float* sinks, hipStream_t stream) {
+                                   float scale, int window, int chunk, const float* sinks, float softcap,
+                                   int keep_first, hipStream_t stream) {
     if (seq_end <= seq_begin || n_tiles <= 0) return 0;
+    Forms forms;
+    if (!make_forms(softcap, keep_first, window, chunk, scale, forms)) return SIA_BAD_ARGUMENT;
     const int ps_log2 = log2_exact(page_size);
     if (ps_log2 < 3 || n_kv <= 0 || n_heads % n_kv || n_heads > 65535 || q_row_stride % 8 || table_width <= 0)
         return SIA_BAD_ARGUMENT;
 #define ARGS q, q_row_stride, k_pages, v_pages, block_table, table_width, cu_q, kv_len, out, seq_begin, seq_end, \
-             n_heads, n_kv, ps_log2, scale, window, chunk, sinks, stream
+             n_heads, n_kv, ps_log2, scale, window, chunk, sinks, forms, stream
     if constexpr (HD > 128 || !PF_USE_LDS) {
         return HD > 128 ? launch_prefill<1, PF_ROWS / 16, 1>(n_tiles, ARGS) : launch_prefill<2, PF_ROWS / 32, 1>(n_tiles, ARGS);
     } else {
@@ -1193,6 +1298,16 @@ SIA_EXPORT int sia_attn_prefill_ex(const void* q, int q_row_stride, const void* 
         }
     }
 #undef ARGS
+}
+
+SIA_EXPORT int sia_attn_prefill_ex(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,
+                                   const int* block_table, int table_width, const int* cu_q, const int* kv_len,
+                                   void* out, int seq_begin, int seq_end, int n_tiles, int n_tiles_split,
+                                   int n_tiles_long, int q_bound, int kv_bound, int n_heads, int n_kv, int page_size,
+                                   float scale, int window, int chunk, const float* sinks, hipStream_t stream) {
+    return sia_attn_prefill_forms(q, q_row_stride, k_pages, v_pages, block_table, table_width, cu_q, kv_len, out,
+                                  seq_begin, seq_end, n_tiles, n_tiles_split, n_tiles_long, q_bound, kv_bound, n_heads,
+                                  n_kv, page_size, scale, window, chunk, sinks, 0.f, 0, stream);
 }
 
 SIA_EXPORT int sia_attn_prefill(const void* q, int q_row_stride, const void* k_pages, const void* v_pages,

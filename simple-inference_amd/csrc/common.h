@@ -47,7 +47,8 @@ __device__ __forceinline__ float activate(float z, int kind) {
 
 // Gated activations of a (gate, up) pair, in float.  SIA_GLU_SILU: silu(g) * u.  SIA_GLU_CLAMPED: with g = min(g, limit)
 // and u = clamp(u, -limit, limit):  g * sigmoid(1.702 g) * (u + 1).
-enum SiaGlu { SIA_GLU_SILU = 0, SIA_GLU_CLAMPED = 1 };
+// SIA_GLU_RELU: max(g, 0) * u.
+enum SiaGlu { SIA_GLU_SILU = 0, SIA_GLU_CLAMPED = 1, SIA_GLU_RELU = 2 };
 
 __device__ __forceinline__ float gated_activation(float g, float u, int kind, float limit) {
     if (kind == SIA_GLU_CLAMPED) {
@@ -55,6 +56,7 @@ __device__ __forceinline__ float gated_activation(float g, float u, int kind, fl
         u = fminf(fmaxf(u, -limit), limit);
         return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
     }
+    if (kind == SIA_GLU_RELU) return fmaxf(g, 0.f) * u;
     return g / (1.f + expf(-g)) * u;
 }
 

@@ -331,7 +331,7 @@ SIA_EXPORT int sia_glu(const void* gu, void* out, int n_tokens, int inter, int k
                        hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (n_tokens > 65535 || inter <= 0 || (dtype != SIA_F32 && dtype != SIA_BF16) ||
-        (kind != SIA_GLU_SILU && kind != SIA_GLU_CLAMPED))
+        (kind != SIA_GLU_SILU && kind != SIA_GLU_CLAMPED && kind != SIA_GLU_RELU))
         return SIA_BAD_ARGUMENT;
     if (inter % 8 == 0) {
         dim3 block(256), grid((inter / 8 + 255) / 256, n_tokens);

@@ -10,6 +10,8 @@
 //     ``rows`` only those rows are normed and the residual is left as it was.
 //   bias:                   y[n, :] += b                                in place
 //   head gate:              out[n, h, :] *= sigmoid(logit[n, h])        a scalar for every token and head
+//   element gate:           out[n, h, d] = in[n, h, d] * sigmoid(logit[n, h, d])   a gate of its own for every element of
+//                           the heads; the input's heads may lie further apart than they are wide, the output's do not
 //   side by side:           out[n, :] = [T(a[n, :]), T(b[n, :])]        two float streams lowered into one row
 //   scale + soft cap:       z <- cap * tanh(z * scale / cap)            (cap <= 0: z <- z * scale), in place, float
 #include "common.h"
@@ -181,6 +183,58 @@ SIA_EXPORT int sia_head_gate(void* out, const void* logits, int logit_stride, in
                            logit_stride, n_heads, head_dim);
     else
         return SIA_BAD_ARGUMENT;
+    return SIA_LAUNCH_CHECK();
+}
+
+// ---------------------------------------------------------------------------------------
+// out[n, h * own + d] = in[n, h * wide + d] * sigmoid(logits[n * logit_stride + h * own + d]), d < own <= wide
+// ---------------------------------------------------------------------------------------
+template <typename T>
+__global__ void element_gate_kernel(const T* __restrict__ in, const T* __restrict__ logits, int logit_stride,
+                                    T* __restrict__ out, int n_heads, int wide, int own) {
+    const int n = blockIdx.x, width = n_heads * own;
+    for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < width; i += gridDim.y * blockDim.x)
+        out[(size_t)n * width + i] = from_float<T>(to_float(in[((size_t)n * n_heads + i / own) * wide + i % own]) *
+                                                   sigmoidf_(to_float(logits[(size_t)n * logit_stride + i])));
+}
+
+// Eight elements a thread (own, wide and the logits' rows in multiples of 8, aligned).
+template <typename T>
+__global__ void element_gate_vec_kernel(const T* __restrict__ in, const T* __restrict__ logits, int logit_stride,
+                                        T* __restrict__ out, int n_heads, int wide, int own) {
+    const int n = blockIdx.x, width = n_heads * own;
+    const int i = (blockIdx.y * blockDim.x + threadIdx.x) * 8;
+    if (i >= width) return;
+    Vec8<T> vx, vg;
+    float x[8], g[8];
+    vx.load(in + ((size_t)n * n_heads + i / own) * wide + i % own);
+    vg.load(logits + (size_t)n * logit_stride + i);
+    vx.get(x);
+    vg.get(g);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] *= sigmoidf_(g[j]);
+    vx.set(x);
+    vx.store(out + (size_t)n * width + i);
+}
+
+SIA_EXPORT int sia_element_gate(const void* in, const void* logits, int logit_stride, void* out, int n_tokens,
+                                int n_heads, int wide, int own, int dtype, hipStream_t stream) {
+    if (n_tokens <= 0) return 0;
+    if (n_heads <= 0 || own <= 0 || wide < own || logit_stride < n_heads * own || (dtype != SIA_F32 && dtype != SIA_BF16))
+        return SIA_BAD_ARGUMENT;
+    const size_t piece = 8 * (dtype == SIA_F32 ? 4 : 2);
+    const bool vec = own % 8 == 0 && wide % 8 == 0 && logit_stride % 8 == 0 && ((uintptr_t)logits % piece) == 0;
+    const int across = (n_heads * own / (vec ? 8 : 1) + 255) / 256;
+    if (vec && across > 65535) return SIA_BAD_ARGUMENT;
+    dim3 grid(n_tokens, across < 65535 ? (across > 0 ? across : 1) : 65535), block(256);
+#define LAUNCH(KERNEL, T)                                                                                            \
+    hipLaunchKernelGGL(KERNEL<T>, grid, block, 0, stream, (const T*)in, (const T*)logits, logit_stride, (T*)out,     \
+                       n_heads, wide, own)
+    if (vec && dtype == SIA_F32) LAUNCH(element_gate_vec_kernel, float);
+    else if (vec) LAUNCH(element_gate_vec_kernel, bf16_t);
+    else if (dtype == SIA_F32) LAUNCH(element_gate_kernel, float);
+    else LAUNCH(element_gate_kernel, bf16_t);
+#undef LAUNCH
     return SIA_LAUNCH_CHECK();
 }
 

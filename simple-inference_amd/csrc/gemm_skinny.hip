@@ -72,6 +72,9 @@ struct Epilogue {
     ResidualOut res;
     RowScale scale;
     int activation;   // EPI_ACT: which (SiaActivation)
+    const bf16_t* table;     // EPI_ACT: if given, the activation is multiplied by table[ids[m] * table_width + n] for
+    const int* ids;          //          n < table_dim and by 0 beyond
+    int table_width, table_dim;
     int glu;          // EPI_SWIGLU: which gated activation (SiaGlu; 0 is silu(gate) * up)
     float limit;      // EPI_SWIGLU: the clamp of the gated activations that have one
 };
@@ -311,7 +314,12 @@ __global__ __launch_bounds__(WAVES* SIA_WAVE) void gemm_skinny_kernel(const bf16
             *y = from_float<TOut>(ep.glu == SIA_GLU_SILU ? gate / (1.f + expf(-gate)) * up
                                                          : gated_activation(gate, up, ep.glu, ep.limit));
         } else if (EPI == EPI_ACT) {
-            *y = from_float<TOut>(activate(total(j, m, n) * rs, ep.activation));
+            float a = activate(total(j, m, n) * rs, ep.activation);
+            if (ep.table) {
+                const int c = u0 + j * bh + n;
+                a = c < ep.table_dim ? a * bf16_to_float(ep.table[(size_t)ep.ids[m] * ep.table_width + c]) : 0.f;
+            }
+            *y = from_float<TOut>(a);
         } else {
             *y = from_float<TOut>(total(j, m, n) * rs);
         }
@@ -405,6 +413,24 @@ SIA_EXPORT int sia_gemm_skinny_act(const void* X, const void* W, void* Y, int M,
     return SIA_LAUNCH_CHECK();
 }
 
+// Y[M, N] = act(X W^T) * table[ids[m], first + n] for n < dim, 0 beyond (N >= dim): the gate on a token's own input.
+SIA_EXPORT int sia_gemm_skinny_embedding_gate(const void* X, const void* W, void* Y, int M, int N, int K, int activation,
+                                              const void* table, int table_width, int first, int dim, const int* ids,
+                                              hipStream_t stream) {
+    if (M <= 0 || N <= 0) return 0;
+    if (M > 16 || K % 64 || K <= 0 || (activation != SIA_RELU2 && activation != SIA_GELU_TANH && activation != SIA_GELU) ||
+        !table || !ids || dim <= 0 || dim > N || first < 0 || first + dim > table_width)
+        return SIA_BAD_ARGUMENT;
+    Epilogue ep{};
+    ep.activation = activation;
+    ep.table = (const bf16_t*)table + first;
+    ep.ids = ids;
+    ep.table_width = table_width;
+    ep.table_dim = dim;
+    launch_skinny<bf16_t, EPI_ACT>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)Y, M, N, K, ep, stream);
+    return SIA_LAUNCH_CHECK();
+}
+
 // Blocks of columns whose sums of squares sia_gemm_skinny_residual leaves for a result of N columns.
 SIA_EXPORT int sia_gemm_skinny_residual_blocks(int N) {
     if (N <= 0) return 0;
@@ -469,7 +495,8 @@ SIA_EXPORT int sia_gemm_skinny_glu(const void* X, const void* W, void* Y, int M,
                                    const float* partials, int n_partials, float eps, int glu, float limit,
                                    hipStream_t stream) {
     if (M <= 0 || inter <= 0) return 0;
-    if (M > 16 || K % 64 || K <= 0 || (partials && n_partials <= 0) || (glu != SIA_GLU_SILU && glu != SIA_GLU_CLAMPED))
+    if (M > 16 || K % 64 || K <= 0 || (partials && n_partials <= 0) ||
+        (glu != SIA_GLU_SILU && glu != SIA_GLU_CLAMPED && glu != SIA_GLU_RELU))
         return SIA_BAD_ARGUMENT;
     Epilogue ep{};
     ep.scale = RowScale{partials, n_partials, eps};

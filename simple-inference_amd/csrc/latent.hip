@@ -4,18 +4,32 @@
 //   c_q = a_q * rsqrt(mean(a_q^2) + eps) * g_q                     -> cq [tokens, q_rank]
 //   c   = a * rsqrt(mean(a^2) + eps) * g_kv                        -> the key row's first kv_rank elements, and the
 //                                                                     value rows 0 .. kv_rank - 1 of the position
-//   k   = b with neighbouring pairs (2i, 2i + 1), i < rotary_dim / 2, turned by the position's cos/sin row
-//                                                                  -> the key row's next rot_dim elements
+//   k   = b with its pairs turned by the position's cos/sin row, pair i < rotary_dim / 2 being the neighbours (2i, 2i + 1)
+//         or, with half pairing, (i, i + rotary_dim / 2)           -> the key row's next rot_dim elements
 // Key pages [pages, 1, page_size, key_width], value pages [pages, 1, value_rows, page_size]; what lies beyond a row's
 // own elements is never written (it is zero since the pool was made).  With kv_rank == 0 only c_q is made.
 // Norms and rotation are float on the projection's output, one rounding.
 //
 // headwise_linear: y[n, h, o] = sum_i x[n, h, i] * w[h, o, i] for every head, x rows in_stride apart per head, y rows
-// out_stride apart; a head's ``tail`` elements behind the in_dim inputs are copied behind the out_dim outputs, with
+// out_stride apart, times sigmoid(gate[n, h * out + o]) if a gate's logits are given (columns of a wider row); a head's ``tail`` elements behind the in_dim inputs are copied behind the out_dim outputs, with
 // their first rotary_dim elements turned as above, and the rest of a head's out_stride is set to zero.  Float sums.
 // Three forms: a wave an output element for steps of up to 16 rows, matrix cores for more rows in bfloat16 where the
 // 16-byte loads are aligned, and an LDS-tiled form on the vector units for everything else (float32, odd sizes).
 #include "common.h"
+
+// Element i of a row whose first rotary_dim elements turn by the position's tables.
+template <typename T>
+__device__ __forceinline__ float turned(const T* __restrict__ src, int i, int rotary_dim, int halves,
+                                        const float* __restrict__ cos_t, const float* __restrict__ sin_t, int pos) {
+    const float v = to_float(src[i]);
+    if (i >= rotary_dim) return v;
+    const int half = rotary_dim / 2;
+    const int pair = halves ? i % half : i / 2;
+    const bool second = halves ? i >= half : (i & 1);
+    const float other = to_float(src[halves ? (second ? i - half : i + half) : i ^ 1]);
+    const float c = cos_t[(size_t)pos * half + pair], s = sin_t[(size_t)pos * half + pair];
+    return second ? v * c + other * s : v * c - other * s;
+}
 
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(
@@ -23,7 +37,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
     const float* __restrict__ kv_gain, int rot_dim, int rotary_dim, const float* __restrict__ cos_t,
     const float* __restrict__ sin_t, float eps, const int* __restrict__ positions, const int* __restrict__ seq_of_token,
     const int* __restrict__ table, int table_width, T* __restrict__ k_pages, T* __restrict__ v_pages, int page_size,
-    int key_width, int value_rows, T* __restrict__ cq) {
+    int key_width, int value_rows, T* __restrict__ cq, int halves) {
     __shared__ float scratch[16];
     const int n = blockIdx.x, tid = threadIdx.x;
     const T* row = proj + (size_t)n * row_stride;
@@ -55,23 +69,16 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
         v_col[(size_t)i * page_size] = c;
     }
     const T* b = a + kv_rank;
-    const int half = rotary_dim / 2;
-    for (int i = tid; i < rot_dim; i += blockDim.x) {
-        float v = to_float(b[i]);
-        if (i < rotary_dim) {
-            const float other = to_float(b[i ^ 1]);
-            const float c = cos_t[(size_t)pos * half + i / 2], s = sin_t[(size_t)pos * half + i / 2];
-            v = (i & 1) ? v * c + other * s : v * c - other * s;
-        }
-        k_row[kv_rank + i] = from_float<T>(v);
-    }
+    for (int i = tid; i < rot_dim; i += blockDim.x)
+        k_row[kv_rank + i] = from_float<T>(turned(b, i, rotary_dim, halves, cos_t, sin_t, pos));
 }
 
 SIA_EXPORT int sia_latent_prepare(const void* proj, int row_stride, int q_rank, const float* q_gain, int kv_rank,
                                   const float* kv_gain, int rot_dim, int rotary_dim, const float* cos_t,
                                   const float* sin_t, float eps, const int* positions, const int* seq_of_token,
                                   const int* table, int table_width, void* k_pages, void* v_pages, int page_size,
-                                  int key_width, int value_rows, void* cq, int n_tokens, int dtype, hipStream_t stream) {
+                                  int key_width, int value_rows, void* cq, int n_tokens, int halves, int dtype,
+                                  hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (q_rank <= 0 || !q_gain || !cq || kv_rank < 0 || rot_dim < 0 || rotary_dim < 0 || rotary_dim % 2 ||
         rotary_dim > rot_dim || row_stride < q_rank + (kv_rank ? kv_rank + rot_dim : 0))
@@ -83,42 +90,40 @@ SIA_EXPORT int sia_latent_prepare(const void* proj, int row_stride, int q_rank, 
     if (dtype == SIA_F32)
         hipLaunchKernelGGL(latent_prepare_kernel<float>, grid, block, 0, stream, (const float*)proj, row_stride, q_rank,
                            q_gain, kv_rank, kv_gain, rot_dim, rotary_dim, cos_t, sin_t, eps, positions, seq_of_token, table,
-                           table_width, (float*)k_pages, (float*)v_pages, page_size, key_width, value_rows, (float*)cq);
+                           table_width, (float*)k_pages, (float*)v_pages, page_size, key_width, value_rows, (float*)cq, halves);
     else if (dtype == SIA_BF16)
         hipLaunchKernelGGL(latent_prepare_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)proj, row_stride, q_rank,
                            q_gain, kv_rank, kv_gain, rot_dim, rotary_dim, cos_t, sin_t, eps, positions, seq_of_token, table,
-                           table_width, (bf16_t*)k_pages, (bf16_t*)v_pages, page_size, key_width, value_rows, (bf16_t*)cq);
+                           table_width, (bf16_t*)k_pages, (bf16_t*)v_pages, page_size, key_width, value_rows, (bf16_t*)cq, halves);
     else
         return SIA_BAD_ARGUMENT;
     return SIA_LAUNCH_CHECK();
 }
 
-// Behind a head's outputs: the head's tail, its first rotary_dim elements turned in neighbouring pairs, and zeros up to
+// Behind a head's outputs: the head's tail, its first rotary_dim elements turned in pairs, and zeros up to
 // the head's stride, for tokens n0 .. n0 + tokens - 1 of head h, by all threads of the workgroup.
 template <typename T>
 __device__ __forceinline__ void headwise_tail(const T* __restrict__ x, int x_row, int in_stride, T* __restrict__ y,
                                               int y_row, int out_stride, int n_tokens, int in_dim, int out_dim, int tail,
                                               int rotary_dim, const float* __restrict__ cos_t,
                                               const float* __restrict__ sin_t, const int* __restrict__ positions,
-                                              int n0, int tokens, int h) {
-    const int rest = out_stride - out_dim, half = rotary_dim / 2;
+                                              int n0, int tokens, int h, int halves) {
+    const int rest = out_stride - out_dim;
     for (int idx = threadIdx.x; idx < tokens * rest; idx += blockDim.x) {
         const int n = n0 + idx / rest, i = idx % rest;
         if (n >= n_tokens) break;
         float v = 0.f;
         if (i < tail) {
             const T* src = x + (size_t)n * x_row + (size_t)h * in_stride + in_dim;
-            v = to_float(src[i]);
-            if (i < rotary_dim) {
-                const int pos = positions[n];
-                const float other = to_float(src[i ^ 1]);
-                const float c = cos_t[(size_t)pos * half + i / 2], s = sin_t[(size_t)pos * half + i / 2];
-                v = (i & 1) ? v * c + other * s : v * c - other * s;
-            }
+            v = turned(src, i, rotary_dim, halves, cos_t, sin_t, rotary_dim > 0 ? positions[n] : 0);
         }
         y[(size_t)n * y_row + (size_t)h * out_stride + out_dim + i] = from_float<T>(v);
     }
 }
+
+// What a gate's logit makes of the output element it belongs to.
+template <typename T>
+__device__ __forceinline__ float gate_factor(T logit) { return 1.f / (1.f + expf(-to_float(logit))); }
 
 #define HW_TOKENS 16
 #define HW_OUTS 64
@@ -130,7 +135,8 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(const T* __restric
                                                               int out_stride, int n_tokens, int in_dim, int out_dim,
                                                               int tail, int rotary_dim, const float* __restrict__ cos_t,
                                                               const float* __restrict__ sin_t,
-                                                              const int* __restrict__ positions) {
+                                                              const int* __restrict__ positions, int halves,
+                                                              const T* __restrict__ gate, int gate_stride) {
     __shared__ float xs[HW_TOKENS][HW_K];
     __shared__ float ws[HW_OUTS][HW_K + 1];
     const int n0 = blockIdx.x * HW_TOKENS, h = blockIdx.y, o0 = blockIdx.z * HW_OUTS, tid = threadIdx.x;
@@ -159,11 +165,13 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(const T* __restric
 #pragma unroll
     for (int t = 0; t < 4; ++t) {
         const int n = n0 + tg * 4 + t;
-        if (n < n_tokens && o0 + o < out_dim) y[(size_t)n * y_row + (size_t)h * out_stride + o0 + o] = from_float<T>(acc[t]);
+        if (n < n_tokens && o0 + o < out_dim)
+            y[(size_t)n * y_row + (size_t)h * out_stride + o0 + o] =
+                from_float<T>(gate ? acc[t] * gate_factor(gate[(size_t)n * gate_stride + h * out_dim + o0 + o]) : acc[t]);
     }
     if (blockIdx.z != 0) return;
     headwise_tail<T>(x, x_row, in_stride, y, y_row, out_stride, n_tokens, in_dim, out_dim, tail, rotary_dim, cos_t, sin_t,
-                     positions, n0, HW_TOKENS, h);
+                     positions, n0, HW_TOKENS, h, halves);
 }
 
 // A step of few rows (decode): a wave an output element of a head, for all the rows; the head's weight row is read once
@@ -174,7 +182,8 @@ __global__ __launch_bounds__(256) void headwise_rows_kernel(const T* __restrict_
                                                             int out_stride, int n_tokens, int in_dim, int out_dim,
                                                             int tail, int rotary_dim, const float* __restrict__ cos_t,
                                                             const float* __restrict__ sin_t,
-                                                            const int* __restrict__ positions) {
+                                                            const int* __restrict__ positions, int halves,
+                                                            const T* __restrict__ gate, int gate_stride) {
     const int h = blockIdx.y, wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE;
     const int o = blockIdx.x * (blockDim.x / SIA_WAVE) + wave;
     if (o < out_dim) {
@@ -184,12 +193,14 @@ __global__ __launch_bounds__(256) void headwise_rows_kernel(const T* __restrict_
             float acc = 0.f;
             for (int k = lane; k < in_dim; k += SIA_WAVE) acc += to_float(wr[k]) * to_float(xr[k]);
             acc = wave_sum(acc);
-            if (lane == 0) y[(size_t)n * y_row + (size_t)h * out_stride + o] = from_float<T>(acc);
+            if (lane == 0)
+                y[(size_t)n * y_row + (size_t)h * out_stride + o] =
+                    from_float<T>(gate ? acc * gate_factor(gate[(size_t)n * gate_stride + h * out_dim + o]) : acc);
         }
     }
     if (blockIdx.x != 0) return;
     headwise_tail<T>(x, x_row, in_stride, y, y_row, out_stride, n_tokens, in_dim, out_dim, tail, rotary_dim, cos_t, sin_t,
-                     positions, 0, n_tokens, h);
+                     positions, 0, n_tokens, h, halves);
 }
 
 // Many rows in bfloat16 (prompts): matrix cores.  A workgroup 128 tokens and 32 output columns of a head, a wave 32 of
@@ -205,7 +216,8 @@ __global__ __launch_bounds__(256) void headwise_mfma_kernel(const bf16_t* __rest
                                                             int out_dim, int tail, int rotary_dim,
                                                             const float* __restrict__ cos_t,
                                                             const float* __restrict__ sin_t,
-                                                            const int* __restrict__ positions) {
+                                                            const int* __restrict__ positions, int halves,
+                                                            const bf16_t* __restrict__ gate, int gate_stride) {
     const int h = blockIdx.y, o0 = blockIdx.z * 32, n0 = blockIdx.x * 128;
     const int wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE, r = lane & 15, g = lane >> 4;
     const int t0 = n0 + wave * 32;
@@ -247,24 +259,28 @@ __global__ __launch_bounds__(256) void headwise_mfma_kernel(const bf16_t* __rest
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const int c = o0 + nb * 16 + 4 * g + i;
-                    if (c < out_dim) y[(size_t)n * y_row + (size_t)h * out_stride + c] = float_to_bf16(acc[nb][mb][i]);
+                    if (c < out_dim) {
+                        float v = acc[nb][mb][i];
+                        if (gate) v *= gate_factor(gate[(size_t)n * gate_stride + h * out_dim + c]);
+                        y[(size_t)n * y_row + (size_t)h * out_stride + c] = float_to_bf16(v);
+                    }
                 }
         }
     }
     if (blockIdx.z != 0) return;
     headwise_tail<bf16_t>(x, x_row, in_stride, y, y_row, out_stride, n_tokens, in_dim, out_dim, tail, rotary_dim, cos_t,
-                          sin_t, positions, n0, 128, h);
+                          sin_t, positions, n0, 128, h, halves);
 }
 
 SIA_EXPORT int sia_headwise_linear(const void* x, int x_row, int in_stride, const void* w, void* y, int y_row,
                                    int out_stride, int n_tokens, int n_heads, int in_dim, int out_dim, int tail,
-                                   int rotary_dim, const float* cos_t, const float* sin_t, const int* positions, int dtype,
-                                   hipStream_t stream) {
+                                   int rotary_dim, const float* cos_t, const float* sin_t, const int* positions,
+                                   int halves, const void* gate, int gate_stride, int dtype, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (n_heads <= 0 || n_heads > 65535 || in_dim <= 0 || out_dim <= 0 || tail < 0 || in_dim + tail > in_stride ||
         out_dim + tail > out_stride || x_row < n_heads * in_stride || y_row < n_heads * out_stride || rotary_dim < 0 ||
         rotary_dim % 2 || rotary_dim > tail || (rotary_dim && (!cos_t || !sin_t || !positions)) ||
-        (out_dim + HW_OUTS - 1) / HW_OUTS > 65535)
+        (out_dim + HW_OUTS - 1) / HW_OUTS > 65535 || (gate && gate_stride < n_heads * out_dim))
         return SIA_BAD_ARGUMENT;
     dim3 grid((n_tokens + HW_TOKENS - 1) / HW_TOKENS, n_heads, (out_dim + HW_OUTS - 1) / HW_OUTS), block(256);
     if (n_tokens <= 16 && (out_dim + 3) / 4 <= 65535) {
@@ -272,11 +288,11 @@ SIA_EXPORT int sia_headwise_linear(const void* x, int x_row, int in_stride, cons
         if (dtype == SIA_F32)
             hipLaunchKernelGGL(headwise_rows_kernel<float>, rgrid, block, 0, stream, (const float*)x, x_row, in_stride,
                                (const float*)w, (float*)y, y_row, out_stride, n_tokens, in_dim, out_dim, tail,
-                               rotary_dim, cos_t, sin_t, positions);
+                               rotary_dim, cos_t, sin_t, positions, halves, (const float*)gate, gate_stride);
         else if (dtype == SIA_BF16)
             hipLaunchKernelGGL(headwise_rows_kernel<bf16_t>, rgrid, block, 0, stream, (const bf16_t*)x, x_row, in_stride,
                                (const bf16_t*)w, (bf16_t*)y, y_row, out_stride, n_tokens, in_dim, out_dim, tail,
-                               rotary_dim, cos_t, sin_t, positions);
+                               rotary_dim, cos_t, sin_t, positions, halves, (const bf16_t*)gate, gate_stride);
         else
             return SIA_BAD_ARGUMENT;
         return SIA_LAUNCH_CHECK();
@@ -286,17 +302,17 @@ SIA_EXPORT int sia_headwise_linear(const void* x, int x_row, int in_stride, cons
         dim3 mgrid((n_tokens + 127) / 128, n_heads, (out_dim + 31) / 32);
         hipLaunchKernelGGL(headwise_mfma_kernel, mgrid, block, 0, stream, (const bf16_t*)x, x_row, in_stride,
                            (const bf16_t*)w, (bf16_t*)y, y_row, out_stride, n_tokens, in_dim, out_dim, tail, rotary_dim,
-                           cos_t, sin_t, positions);
+                           cos_t, sin_t, positions, halves, (const bf16_t*)gate, gate_stride);
         return SIA_LAUNCH_CHECK();
     }
     if (dtype == SIA_F32)
         hipLaunchKernelGGL(headwise_linear_kernel<float>, grid, block, 0, stream, (const float*)x, x_row, in_stride,
                            (const float*)w, (float*)y, y_row, out_stride, n_tokens, in_dim, out_dim, tail, rotary_dim,
-                           cos_t, sin_t, positions);
+                           cos_t, sin_t, positions, halves, (const float*)gate, gate_stride);
     else if (dtype == SIA_BF16)
         hipLaunchKernelGGL(headwise_linear_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)x, x_row, in_stride,
                            (const bf16_t*)w, (bf16_t*)y, y_row, out_stride, n_tokens, in_dim, out_dim, tail, rotary_dim,
-                           cos_t, sin_t, positions);
+                           cos_t, sin_t, positions, halves, (const bf16_t*)gate, gate_stride);
     else
         return SIA_BAD_ARGUMENT;
     return SIA_LAUNCH_CHECK();

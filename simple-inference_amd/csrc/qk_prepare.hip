@@ -14,6 +14,9 @@
 //
 // q is written back in place, k goes to the token's place in its page, v (with its bias) too.
 //
+// With values given by an earlier layer (rows given_stride apart, the same heads and widths) and a learned scalar m in
+// device memory, what is written is (1 - m) v + m given.
+//
 // Page layout:  keys   [page][kv_head][offset][k_row]
 //               values [page][kv_head][v_rows][offset]      (positions innermost)
 // k_row and v_rows are head_dim and value_dim, or larger: pages may be wider than the heads (a mixer whose keys and
@@ -45,7 +48,9 @@ __device__ __forceinline__ void write_values(const T* __restrict__ qkv, int row_
                                              const int* __restrict__ positions, const int* __restrict__ seq_of_token,
                                              T* __restrict__ v_pages, int n, int n_tokens, int page, int off, int pos,
                                              int v_first, int rows, int value_dim, int v_rows, int page_size,
-                                             int v_group) {
+                                             int v_group, const T* __restrict__ given, int given_stride,
+                                             const float* __restrict__ mix) {
+    const float m = given ? *mix : 0.f;
     const size_t page_rows = (size_t)(rows / value_dim) * v_rows;   // value rows of a page, over its kv heads
     auto page_row = [&](int i) { return (size_t)(i / value_dim) * v_rows + i % value_dim; };
     const T* x = qkv + (size_t)n * row_stride + v_first;
@@ -64,6 +69,7 @@ __device__ __forceinline__ void write_values(const T* __restrict__ qkv, int row_
         for (int i = threadIdx.x; i < rows; i += blockDim.x) {
             float v = to_float(x[i]);
             if (b) v += b[i];
+            if (given) v = (1.f - m) * v + m * to_float(given[(size_t)n * given_stride + i]);
             v_pages[((size_t)page * page_rows + page_row(i)) * page_size + off] = from_float<T>(v);
         }
         return;
@@ -77,7 +83,15 @@ __device__ __forceinline__ void write_values(const T* __restrict__ qkv, int row_
         const float add = b ? b[i] : 0.f;
 #pragma unroll
         for (int j = 0; j < V_MAX; ++j)
-            vals[j] = j < v_group ? from_float<T>(to_float(x0[(size_t)j * row_stride + i]) + add) : T(0);
+        {
+            if (j >= v_group) {
+                vals[j] = T(0);
+                continue;
+            }
+            float v = to_float(x0[(size_t)j * row_stride + i]) + add;
+            if (given) v = (1.f - m) * v + m * to_float(given[(size_t)(first + j) * given_stride + i]);
+            vals[j] = from_float<T>(v);
+        }
         T* dst = v_pages + ((size_t)page * page_rows + page_row(i)) * page_size + (off - place);
 #pragma unroll
         for (int j = 0; j < V_MAX; j += PER)
@@ -93,7 +107,8 @@ __global__ __launch_bounds__(QKP_WAVES* SIA_WAVE) void qk_prepare_kernel(
     const int* __restrict__ block_table, int table_width, T* __restrict__ k_pages, T* __restrict__ v_pages,
     int n_tokens, int n_heads, int n_kv, int head_dim, int value_dim, int rotary_dim, int page_size, int v_group,
     int k_row, int v_rows, T* q_out, int q_row_stride, int q_head_stride, float temp_coef,
-    int temp_every, int values_are_keys) {   // q_out may be qkv
+    int temp_every, int values_are_keys, const T* __restrict__ given, int given_stride,
+    const float* __restrict__ mix) {   // q_out may be qkv
     const int n = blockIdx.x, wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE;
     const int pos = positions[n];
     const int half = rotary_dim / 2;
@@ -108,7 +123,7 @@ __global__ __launch_bounds__(QKP_WAVES* SIA_WAVE) void qk_prepare_kernel(
     if ((int)blockIdx.y >= qk_groups) {  // the token's values
         if (page >= 0)
             write_values<T>(qkv, row_stride, bias, positions, seq_of_token, v_pages, n, n_tokens, page, off, pos, v_first,
-                            n_kv * value_dim, value_dim, v_rows, page_size, v_group);
+                            n_kv * value_dim, value_dim, v_rows, page_size, v_group, given, given_stride, mix);
         return;
     }
     const int item = blockIdx.y * QKP_WAVES + wave;
@@ -178,7 +193,8 @@ __global__ __launch_bounds__(QKP_WAVES* SIA_WAVE) void qk_prepare_vec_kernel(
     const int* __restrict__ block_table, int table_width, T* __restrict__ k_pages, T* __restrict__ v_pages,
     int n_tokens, int n_heads, int n_kv, int head_dim, int value_dim, int rotary_dim, int page_size, int v_group,
     int k_row, int v_rows, T* q_out, int q_row_stride, int q_head_stride, float temp_coef,
-    int temp_every, int values_are_keys) {   // q_out may be qkv
+    int temp_every, int values_are_keys, const T* __restrict__ given, int given_stride,
+    const float* __restrict__ mix) {   // q_out may be qkv
     const int n = blockIdx.x, wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE;
     const int pos = positions[n];
     const int half = rotary_dim / 2;
@@ -190,7 +206,7 @@ __global__ __launch_bounds__(QKP_WAVES* SIA_WAVE) void qk_prepare_vec_kernel(
         const int page = block_table[(size_t)seq_of_token[n] * table_width + pos / page_size];
         if (page >= 0)
             write_values<T>(qkv, row_stride, bias, positions, seq_of_token, v_pages, n, n_tokens, page, pos % page_size,
-                            pos, v_first, n_kv * value_dim, value_dim, v_rows, page_size, v_group);
+                            pos, v_first, n_kv * value_dim, value_dim, v_rows, page_size, v_group, given, given_stride, mix);
         return;
     }
     const int item = (blockIdx.y * QKP_WAVES + wave) * heads_a_wave + lane / group;
@@ -258,15 +274,17 @@ __global__ __launch_bounds__(QKP_WAVES* SIA_WAVE) void qk_prepare_vec_kernel(
 SIA_EXPORT int sia_qk_prepare_max_head_dim() { return QKP_MAX_HEAD_DIM; }
 
 // values_are_keys: the row is [q heads | k heads] and a position's value rows are its k heads as projected (with
-// their bias, before norm and rotation); value_dim is then head_dim.
+// their bias, before norm and rotation); value_dim is then head_dim.  given, mix: values of an earlier layer that the
+// row's own are mixed with (null: none).
 SIA_EXPORT int sia_qk_prepare_ex(void* qkv, int row_stride, const float* bias, const float* q_gain, const float* k_gain,
                                  float eps, const float* cos_table, const float* sin_table, const int* positions,
                                  const int* seq_of_token, const int* block_table, int table_width, void* k_pages,
                                  void* v_pages, int n_tokens, int n_heads, int n_kv, int head_dim, int value_dim,
                                  int rotary_dim, int page_size, int k_row, int v_rows, void* q_out, int q_row_stride,
-                                 int q_head_stride, float temp_coef, int temp_every, int values_are_keys, int dtype,
-                                 hipStream_t stream) {
+                                 int q_head_stride, float temp_coef, int temp_every, int values_are_keys,
+                                 const void* given, int given_stride, const float* mix, int dtype, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
+    if (given && (!mix || values_are_keys || n_kv <= 0 || given_stride < n_kv * value_dim)) return SIA_BAD_ARGUMENT;
     if (values_are_keys && value_dim != head_dim) return SIA_BAD_ARGUMENT;
     if (head_dim <= 0 || head_dim > QKP_MAX_HEAD_DIM || value_dim <= 0 || n_heads < 0 || n_kv < 0) return SIA_BAD_ARGUMENT;
     if (rotary_dim < 0 || rotary_dim > head_dim || (rotary_dim & 1)) return SIA_BAD_ARGUMENT;
@@ -296,13 +314,13 @@ SIA_EXPORT int sia_qk_prepare_ex(void* qkv, int row_stride, const float* bias, c
                                k_gain, eps, cos_table, sin_table, positions, seq_of_token, block_table, table_width, \
                                (T*)k_pages, (T*)v_pages, n_tokens, n_heads, n_kv, head_dim, value_dim, rotary_dim,   \
                                page_size, v_group, k_row, v_rows, (T*)q_out, q_row_stride, q_head_stride, temp_coef,  \
-                               temp_every, values_are_keys);                                                                       \
+                               temp_every, values_are_keys, (const T*)given, given_stride, mix);                                \
         else                                                                                                         \
             hipLaunchKernelGGL(qk_prepare_kernel<T>, grid, block, 0, stream, (T*)qkv, row_stride, bias, q_gain,      \
                                k_gain, eps, cos_table, sin_table, positions, seq_of_token, block_table, table_width, \
                                (T*)k_pages, (T*)v_pages, n_tokens, n_heads, n_kv, head_dim, value_dim, rotary_dim,   \
                                page_size, v_group, k_row, v_rows, (T*)q_out, q_row_stride, q_head_stride, temp_coef,  \
-                               temp_every, values_are_keys);                                                                       \
+                               temp_every, values_are_keys, (const T*)given, given_stride, mix);                                \
     } while (0)
     if (dtype == SIA_F32) LAUNCH(float);
     else if (dtype == SIA_BF16) LAUNCH(bf16_t);
@@ -320,5 +338,5 @@ SIA_EXPORT int sia_qk_prepare(void* qkv, int row_stride, const float* bias, cons
     return sia_qk_prepare_ex(qkv, row_stride, bias, q_gain, k_gain, eps, cos_table, sin_table, positions, seq_of_token,
                              block_table, table_width, k_pages, v_pages, n_tokens, n_heads, n_kv, head_dim, value_dim,
                              rotary_dim, page_size, k_row, v_rows, q_out, q_row_stride, q_head_stride, temp_coef,
-                             temp_every, 0, dtype, stream);
+                             temp_every, 0, nullptr, 0, nullptr, dtype, stream);
 }

@@ -757,13 +757,17 @@ SIA_EXPORT int sia_decay_attention(void* proj, int row_stride, const float* deca
 // costs two sums over the R lanes of a column, one before the write and one after.  Blocks of tokens are staged
 // through LDS as floats, where the unit norms, the write strengths and the decays of the block are taken, by every
 // workgroup for itself.  The raw outputs go to the float workspace; the head's norm and gate are a second kernel.
-template <typename T, int ROWS>
+// CHANNELS: every key channel has a decay of its own, g [H, D] acting on the rows of S, and the output gate comes as a
+// factor: both were computed before (``decays`` [tokens, H, D] and ``gates`` [tokens, H * Dv], float), and a_log,
+// dt_bias and the columns a_col and g_col are not read.
+template <typename T, int ROWS, bool CHANNELS>
 __global__ __launch_bounds__(512) void delta_rule_kernel(
     const T* __restrict__ qkv, int qkv_stride, const T* __restrict__ proj, int proj_stride, int b_col, int a_col,
     const float* __restrict__ a_log, const float* __restrict__ dt_bias, float* __restrict__ state,
     long long state_stride, const int* __restrict__ cu_q, const int* __restrict__ slots, float* __restrict__ raw_out,
     int n_heads, int n_kv, int D, int Dv, int R, int block_tokens, int slice, int g_col,
-    const float* __restrict__ norm_w, T* __restrict__ out, float eps) {
+    const float* __restrict__ norm_w, T* __restrict__ out, float eps, const float* __restrict__ decays,
+    const float* __restrict__ gates) {
     // raw_out absent: the workgroup owns all of the head's columns (slice == Dv) and norms and gates its outputs itself
     extern __shared__ float lds[];
     const int seq = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
@@ -776,7 +780,8 @@ __global__ __launch_bounds__(512) void delta_rule_kernel(
     float* v_s = k_s + TB * D;         // [TB][slice]
     float* be_s = v_s + TB * slice;    // [TB]
     float* de_s = be_s + TB;           // [TB]
-    float* o_s = de_s + TB;            // [TB][slice], without raw_out only
+    float* al_s = de_s + TB;           // [TB][D], CHANNELS only
+    float* o_s = al_s + (CHANNELS ? TB * D : 0);   // [TB][slice], without raw_out only
     const int j = j0 + tid / R, r = tid % R;
     const bool owns = tid / R < slice && j < Dv;
     float* S_mem = state + (size_t)slots[seq] * state_stride + (size_t)head * D * Dv;
@@ -789,7 +794,7 @@ __global__ __launch_bounds__(512) void delta_rule_kernel(
     const int wave = tid / SIA_WAVE, lane = tid % SIA_WAVE, n_waves = blockDim.x / SIA_WAVE;
     const int kv_head = head / (n_heads / n_kv);
     const int q_col = kv_head * D, k_col = n_kv * D + kv_head * D, v_col = 2 * n_kv * D + head * Dv;
-    const float rate = expf(a_log[head]), bias = dt_bias ? dt_bias[head] : 0.f;
+    const float rate = CHANNELS ? 0.f : expf(a_log[head]), bias = !CHANNELS && dt_bias ? dt_bias[head] : 0.f;
     const float q_scale = rsqrtf((float)D);
 
     for (int t0 = first; t0 < last; t0 += TB) {
@@ -803,12 +808,15 @@ __global__ __launch_bounds__(512) void delta_rule_kernel(
             const T* row = qkv + (size_t)(t0 + t) * qkv_stride;
             q_s[idx] = to_float(row[q_col + c]);
             k_s[idx] = to_float(row[k_col + c]);
+            if (CHANNELS) al_s[idx] = decays[((size_t)(t0 + t) * n_heads + head) * D + c];
         }
         if (tid < nt) {
             const T* row = proj + (size_t)(t0 + tid) * proj_stride;
-            const float zb = to_float(row[b_col + head]), za = to_float(row[a_col + head]) + bias;
-            be_s[tid] = 1.f / (1.f + expf(-zb));
-            de_s[tid] = expf(-rate * (fmaxf(za, 0.f) + log1pf(expf(-fabsf(za)))));
+            be_s[tid] = 1.f / (1.f + expf(-to_float(row[b_col + head])));
+            if (!CHANNELS) {
+                const float za = to_float(row[a_col + head]) + bias;
+                de_s[tid] = expf(-rate * (fmaxf(za, 0.f) + log1pf(expf(-fabsf(za)))));
+            }
         }
         __syncthreads();
         for (int t = wave; t < nt; t += n_waves) {      // unit vectors, a wave a token
@@ -825,14 +833,14 @@ __global__ __launch_bounds__(512) void delta_rule_kernel(
         }
         __syncthreads();
         for (int t = 0; t < nt; ++t) {
-            const float g = de_s[t], b = be_s[t];
+            const float g = CHANNELS ? 1.f : de_s[t], b = be_s[t];
             const float v = owns ? v_s[t * slice + (j - j0)] : 0.f;
             float kept = 0.f;
 #pragma unroll
             for (int i = 0; i < ROWS; ++i) {
                 const int d = i * R + r;
                 if (d < D) {
-                    S[i] *= g;
+                    S[i] *= CHANNELS ? al_s[t * D + d] : g;
                     kept += k_s[t * D + d] * S[i];
                 }
             }
@@ -859,8 +867,14 @@ __global__ __launch_bounds__(512) void delta_rule_kernel(
             float ss = 0.f;
             for (int c = lane; c < Dv; c += SIA_WAVE) ss += o_s[t * slice + c] * o_s[t * slice + c];
             const float inv = rsqrtf(wave_sum(ss) / (float)Dv + eps);
-            const T* g_row = proj + (size_t)(t0 + t) * proj_stride + g_col + head * Dv;
             T* dst = out + ((size_t)(t0 + t) * n_heads + head) * Dv;
+            if (CHANNELS) {
+                const float* factor = gates + ((size_t)(t0 + t) * n_heads + head) * Dv;
+                for (int c = lane; c < Dv; c += SIA_WAVE)
+                    dst[c] = from_float<T>(o_s[t * slice + c] * inv * norm_w[c] * factor[c]);
+                continue;
+            }
+            const T* g_row = proj + (size_t)(t0 + t) * proj_stride + g_col + head * Dv;
             for (int c = lane; c < Dv; c += SIA_WAVE) {
                 const float z = to_float(g_row[c]);
                 dst[c] = from_float<T>(o_s[t * slice + c] * inv * norm_w[c] * (z / (1.f + expf(-z))));
@@ -883,12 +897,12 @@ __global__ __launch_bounds__(512) void delta_rule_kernel(
 // strengths and decays are taken in LDS before it is walked, and its outputs leave together.
 #define DELTA_WALK_TOKENS 32
 #define DELTA_WALK_THREADS 256
-template <int ROWS, int C>
+template <int ROWS, int C, bool CHANNELS>
 __global__ __launch_bounds__(DELTA_WALK_THREADS) void delta_walk_kernel(
     const bf16_t* __restrict__ qkv, int qkv_stride, const bf16_t* __restrict__ proj, int proj_stride, int b_col,
     int a_col, const float* __restrict__ a_log, const float* __restrict__ dt_bias, float* __restrict__ state,
     long long state_stride, const int* __restrict__ cu_q, const int* __restrict__ slots, float* __restrict__ raw_out,
-    int n_heads, int n_kv, int D, int Dv) {
+    int n_heads, int n_kv, int D, int Dv, const float* __restrict__ decays) {
     extern __shared__ float lds[];
     constexpr int TB = DELTA_WALK_TOKENS, threads = DELTA_WALK_THREADS;
     constexpr int slice = threads / 16 * C;      // columns a workgroup
@@ -899,12 +913,13 @@ __global__ __launch_bounds__(DELTA_WALK_THREADS) void delta_walk_kernel(
     if (first >= last) return;
     float* q_s = lds;               // [TB][Dp], row d = r * ROWS + i at (i / 4) * 64 + r * 4 + i % 4
     float* k_s = q_s + TB * Dp;
-    float* v_s = k_s + TB * Dp;     // [TB][slice]
+    float* al_s = k_s + TB * Dp;    // [TB][Dp] in the same order, CHANNELS only
+    float* v_s = al_s + (CHANNELS ? TB * Dp : 0);     // [TB][slice]
     float* o_s = v_s + TB * slice;  // [TB][slice]
     float* be_s = o_s + TB * slice; // [TB]
     float* de_s = be_s + TB;        // [TB]
     auto place = [](int d) { const int r = d / ROWS, i = d % ROWS; return (i / 4) * 64 + r * 4 + i % 4; };
-    for (int i = tid; i < 2 * TB * Dp; i += threads) lds[i] = 0.f;
+    for (int i = tid; i < (CHANNELS ? 3 : 2) * TB * Dp; i += threads) lds[i] = 0.f;
     const int jl = (tid / 16) * C, r = tid % 16;
     float* S_mem = state + (size_t)slots[seq] * state_stride + (size_t)head * D * Dv;
     float S[C][ROWS];
@@ -918,7 +933,7 @@ __global__ __launch_bounds__(DELTA_WALK_THREADS) void delta_walk_kernel(
     const int wave = tid / SIA_WAVE, lane = tid % SIA_WAVE;
     const int kv_head = head / (n_heads / n_kv);
     const int q_col = kv_head * D, k_col = n_kv * D + kv_head * D, v_col = 2 * n_kv * D + head * Dv;
-    const float rate = expf(a_log[head]), bias = dt_bias ? dt_bias[head] : 0.f;
+    const float rate = CHANNELS ? 0.f : expf(a_log[head]), bias = !CHANNELS && dt_bias ? dt_bias[head] : 0.f;
     const float q_scale = rsqrtf((float)D);
     __syncthreads();
     for (int t0 = first; t0 < last; t0 += TB) {
@@ -928,6 +943,7 @@ __global__ __launch_bounds__(DELTA_WALK_THREADS) void delta_walk_kernel(
             const bf16_t* row = qkv + (size_t)(t0 + t) * qkv_stride;
             q_s[t * Dp + place(d)] = bf16_to_float(row[q_col + d]);
             k_s[t * Dp + place(d)] = bf16_to_float(row[k_col + d]);
+            if (CHANNELS) al_s[t * Dp + place(d)] = decays[((size_t)(t0 + t) * n_heads + head) * D + d];
         }
         for (int idx = tid; idx < nt * slice; idx += threads) {
             const int t = idx / slice, c = idx % slice;
@@ -935,9 +951,11 @@ __global__ __launch_bounds__(DELTA_WALK_THREADS) void delta_walk_kernel(
         }
         if (tid < nt) {
             const bf16_t* row = proj + (size_t)(t0 + tid) * proj_stride;
-            const float zb = bf16_to_float(row[b_col + head]), za = bf16_to_float(row[a_col + head]) + bias;
-            be_s[tid] = 1.f / (1.f + expf(-zb));
-            de_s[tid] = expf(-rate * (fmaxf(za, 0.f) + log1pf(expf(-fabsf(za)))));
+            be_s[tid] = 1.f / (1.f + expf(-bf16_to_float(row[b_col + head])));
+            if (!CHANNELS) {
+                const float za = bf16_to_float(row[a_col + head]) + bias;
+                de_s[tid] = expf(-rate * (fmaxf(za, 0.f) + log1pf(expf(-fabsf(za)))));
+            }
         }
         __syncthreads();
         for (int t = wave; t < nt; t += threads / SIA_WAVE) {      // unit vectors, a wave a token (the padding is zero)
@@ -953,24 +971,29 @@ __global__ __launch_bounds__(DELTA_WALK_THREADS) void delta_walk_kernel(
             }
         }
         __syncthreads();
-        float4 qn[ROWS / 4], kn[ROWS / 4];
+        float4 qn[ROWS / 4], kn[ROWS / 4], an[CHANNELS ? ROWS / 4 : 1];
         auto fetch = [&](int t) {
 #pragma unroll
             for (int i = 0; i < ROWS / 4; ++i) {
                 const int at = t * Dp + i * 64 + r * 4;
                 qn[i] = *reinterpret_cast<const float4*>(q_s + at);
                 kn[i] = *reinterpret_cast<const float4*>(k_s + at);
+                if (CHANNELS) an[i] = *reinterpret_cast<const float4*>(al_s + at);
             }
         };
         fetch(0);
         for (int t = 0; t < nt; ++t) {
-            float4 qv[ROWS / 4], kv[ROWS / 4];
+            float4 qv[ROWS / 4], kv[ROWS / 4], av[CHANNELS ? ROWS / 4 : 1];
             float vv[C];
 #pragma unroll
-            for (int i = 0; i < ROWS / 4; ++i) { qv[i] = qn[i]; kv[i] = kn[i]; }
+            for (int i = 0; i < ROWS / 4; ++i) {
+                qv[i] = qn[i];
+                kv[i] = kn[i];
+                if (CHANNELS) av[i] = an[i];
+            }
 #pragma unroll
             for (int c = 0; c < C; ++c) vv[c] = v_s[t * slice + jl + c];
-            const float g = de_s[t], b = be_s[t];
+            const float g = CHANNELS ? 1.f : de_s[t], b = be_s[t];
             fetch(min(t + 1, TB - 1));
             float kept[C];
 #pragma unroll
@@ -978,10 +1001,10 @@ __global__ __launch_bounds__(DELTA_WALK_THREADS) void delta_walk_kernel(
                 float acc = 0.f;
 #pragma unroll
                 for (int i = 0; i < ROWS / 4; ++i) {
-                    S[c][4 * i] *= g;
-                    S[c][4 * i + 1] *= g;
-                    S[c][4 * i + 2] *= g;
-                    S[c][4 * i + 3] *= g;
+                    S[c][4 * i] *= CHANNELS ? av[CHANNELS ? i : 0].x : g;
+                    S[c][4 * i + 1] *= CHANNELS ? av[CHANNELS ? i : 0].y : g;
+                    S[c][4 * i + 2] *= CHANNELS ? av[CHANNELS ? i : 0].z : g;
+                    S[c][4 * i + 3] *= CHANNELS ? av[CHANNELS ? i : 0].w : g;
                     acc += kv[i].x * S[c][4 * i];
                     acc += kv[i].y * S[c][4 * i + 1];
                     acc += kv[i].z * S[c][4 * i + 2];
@@ -1036,17 +1059,26 @@ SIA_EXPORT long long sia_delta_rule_workspace(int n_tokens, int n_heads, int Dv)
     return (long long)n_tokens * n_heads * Dv;
 }
 
-SIA_EXPORT int sia_delta_rule(const void* qkv, int qkv_stride, const void* proj, int proj_stride, int g_col, int b_col,
-                              int a_col, const float* a_log, const float* dt_bias, const float* norm_w, float* state,
-                              long long state_stride, const int* cu_q, const int* slots, void* out, int n_tokens,
-                              int n_seqs, int max_q_len, int n_heads, int n_kv, int D, int Dv, float eps, int dtype,
-                              float* workspace, hipStream_t stream) {
-    if (n_seqs <= 0 || n_tokens <= 0) return 0;
-    if (D <= 0 || Dv <= 0 || D > 512 || Dv > 512 || n_heads <= 0 || n_heads > 65535 || n_kv <= 0 || n_heads % n_kv ||
-        !state || !norm_w || !a_log || !workspace || qkv_stride < 2 * n_kv * D + n_heads * Dv || g_col < 0 ||
-        b_col < 0 || a_col < 0 || g_col + n_heads * Dv > proj_stride || b_col + n_heads > proj_stride ||
-        a_col + n_heads > proj_stride || state_stride < (long long)n_heads * D * Dv)
-        return SIA_BAD_ARGUMENT;
+// y = o * rsqrt(mean(o^2) + eps) * w * factor for outputs left in a float workspace: a wave a (token, head).
+template <typename T>
+__global__ __launch_bounds__(SIA_WAVE) void delta_finish_kernel(const float* __restrict__ raw,
+                                                                const float* __restrict__ gates,
+                                                                const float* __restrict__ norm_w, T* __restrict__ out,
+                                                                int n_heads, int Dv, float eps) {
+    const size_t at = ((size_t)blockIdx.x * n_heads + blockIdx.y) * Dv;
+    const int lane = threadIdx.x;
+    float ss = 0.f;
+    for (int c = lane; c < Dv; c += SIA_WAVE) ss += raw[at + c] * raw[at + c];
+    const float inv = rsqrtf(wave_sum(ss) / (float)Dv + eps);
+    for (int c = lane; c < Dv; c += SIA_WAVE) out[at + c] = from_float<T>(raw[at + c] * inv * norm_w[c] * gates[at + c]);
+}
+
+template <bool CHANNELS>
+static int launch_delta_rule(const void* qkv, int qkv_stride, const void* proj, int proj_stride, int g_col, int b_col,
+                             int a_col, const float* a_log, const float* dt_bias, const float* norm_w, float* state,
+                             long long state_stride, const int* cu_q, const int* slots, void* out, int n_tokens,
+                             int n_seqs, int max_q_len, int n_heads, int n_kv, int D, int Dv, float eps, int dtype,
+                             float* workspace, const float* decays, const float* gates, hipStream_t stream) {
     // columns a workgroup: all of a head's, or in a step of runs of tokens a slice of them, as narrow as it takes to
     // fill the chip; lanes a column: the largest power of two that keeps the workgroup within 512 threads
     int slice = Dv;
@@ -1065,7 +1097,9 @@ SIA_EXPORT int sia_delta_rule(const void* qkv, int qkv_stride, const void* proj,
     int TB = max_q_len >= 16 ? 16 : (max_q_len >= 4 ? 4 : 1);
     // a workgroup that owns a whole head norms and gates its outputs itself (a decode step: one launch less)
     const bool whole = slice == Dv;
-    auto bytes = [&](int tb) { return (size_t)tb * (2 * D + (whole ? 2 : 1) * slice + 2) * sizeof(float); };
+    auto bytes = [&](int tb) {
+        return (size_t)tb * ((CHANNELS ? 3 : 2) * D + (whole ? 2 : 1) * slice + 2) * sizeof(float);
+    };
     while (TB > 1 && bytes(TB) > 60 * 1024) TB /= 2;
     if (bytes(TB) > 60 * 1024) return SIA_BAD_ARGUMENT;
     float* raw = whole ? nullptr : workspace;
@@ -1074,25 +1108,29 @@ SIA_EXPORT int sia_delta_rule(const void* qkv, int qkv_stride, const void* proj,
     constexpr int w_cols = 2, w_slice = DELTA_WALK_THREADS / 16 * w_cols;
     const int w_rows = (D + 15) / 16;
     const int w_rows_t = w_rows <= 4 ? 4 : w_rows <= 8 ? 8 : w_rows <= 16 ? 16 : 32;
-    const size_t w_lds = (size_t)(DELTA_WALK_TOKENS * (2 * 16 * w_rows_t + 2 * w_slice + 2)) * sizeof(float);
+    const size_t w_lds = (size_t)(DELTA_WALK_TOKENS * ((CHANNELS ? 3 : 2) * 16 * w_rows_t + 2 * w_slice + 2)) * sizeof(float);
     if (max_q_len > 1 && dtype == SIA_BF16 && w_rows_t <= 16 && w_lds <= 60 * 1024) {
         dim3 wgrid(n_seqs, n_heads, (Dv + w_slice - 1) / w_slice), wblock(DELTA_WALK_THREADS);
 #define WALK(ROWS)                                                                                                   \
-    hipLaunchKernelGGL((delta_walk_kernel<ROWS, w_cols>), wgrid, wblock, w_lds, stream, (const bf16_t*)qkv,          \
+    hipLaunchKernelGGL((delta_walk_kernel<ROWS, w_cols, CHANNELS>), wgrid, wblock, w_lds, stream, (const bf16_t*)qkv, \
                        qkv_stride, (const bf16_t*)proj, proj_stride, b_col, a_col, a_log, dt_bias, state,            \
-                       state_stride, cu_q, slots, workspace, n_heads, n_kv, D, Dv)
+                       state_stride, cu_q, slots, workspace, n_heads, n_kv, D, Dv, decays)
         if (w_rows_t == 4) WALK(4);
         else if (w_rows_t == 8) WALK(8);
         else WALK(16);
 #undef WALK
-        hipLaunchKernelGGL(gla_finish_kernel<bf16_t>, fgrid, fblock, 0, stream, workspace, (const bf16_t*)proj,
-                           proj_stride, g_col, norm_w, (bf16_t*)out, n_heads, Dv, eps);
+        if (CHANNELS)
+            hipLaunchKernelGGL(delta_finish_kernel<bf16_t>, fgrid, fblock, 0, stream, workspace, gates, norm_w, (bf16_t*)out,
+                               n_heads, Dv, eps);
+        else
+            hipLaunchKernelGGL(gla_finish_kernel<bf16_t>, fgrid, fblock, 0, stream, workspace, (const bf16_t*)proj,
+                               proj_stride, g_col, norm_w, (bf16_t*)out, n_heads, Dv, eps);
         return SIA_LAUNCH_CHECK();
     }
 #define LAUNCH(T, ROWS)                                                                                              \
-    hipLaunchKernelGGL((delta_rule_kernel<T, ROWS>), grid, block, bytes(TB), stream, (const T*)qkv, qkv_stride,      \
+    hipLaunchKernelGGL((delta_rule_kernel<T, ROWS, CHANNELS>), grid, block, bytes(TB), stream, (const T*)qkv, qkv_stride,      \
                        (const T*)proj, proj_stride, b_col, a_col, a_log, dt_bias, state, state_stride, cu_q, slots,   \
-                       raw, n_heads, n_kv, D, Dv, R, TB, slice, g_col, norm_w, (T*)out, eps)
+                       raw, n_heads, n_kv, D, Dv, R, TB, slice, g_col, norm_w, (T*)out, eps, decays, gates)
 #define RUN(T)                                                                                                       \
     do {                                                                                                             \
         if (rows <= 4) LAUNCH(T, 4);                                                                                 \
@@ -1101,7 +1139,10 @@ SIA_EXPORT int sia_delta_rule(const void* qkv, int qkv_stride, const void* proj,
         else if (rows <= 32) LAUNCH(T, 32);                                                                          \
         else if (rows <= 64) LAUNCH(T, 64);                                                                          \
         else LAUNCH(T, 128);                                                                                         \
-        if (raw)                                                                                                     \
+        if (raw && CHANNELS)                                                                                         \
+            hipLaunchKernelGGL(delta_finish_kernel<T>, fgrid, fblock, 0, stream, workspace, gates, norm_w, (T*)out,  \
+                               n_heads, Dv, eps);                                                                    \
+        else if (raw)                                                                                                \
             hipLaunchKernelGGL(gla_finish_kernel<T>, fgrid, fblock, 0, stream, workspace, (const T*)proj,            \
                                proj_stride, g_col, norm_w, (T*)out, n_heads, Dv, eps);                               \
     } while (0)
@@ -1111,4 +1152,37 @@ SIA_EXPORT int sia_delta_rule(const void* qkv, int qkv_stride, const void* proj,
 #undef RUN
 #undef LAUNCH
     return SIA_LAUNCH_CHECK();
+}
+
+SIA_EXPORT int sia_delta_rule(const void* qkv, int qkv_stride, const void* proj, int proj_stride, int g_col, int b_col,
+                              int a_col, const float* a_log, const float* dt_bias, const float* norm_w, float* state,
+                              long long state_stride, const int* cu_q, const int* slots, void* out, int n_tokens,
+                              int n_seqs, int max_q_len, int n_heads, int n_kv, int D, int Dv, float eps, int dtype,
+                              float* workspace, hipStream_t stream) {
+    if (n_seqs <= 0 || n_tokens <= 0) return 0;
+    if (D <= 0 || Dv <= 0 || D > 512 || Dv > 512 || n_heads <= 0 || n_heads > 65535 || n_kv <= 0 || n_heads % n_kv ||
+        !state || !norm_w || !a_log || !workspace || qkv_stride < 2 * n_kv * D + n_heads * Dv || g_col < 0 ||
+        b_col < 0 || a_col < 0 || g_col + n_heads * Dv > proj_stride || b_col + n_heads > proj_stride ||
+        a_col + n_heads > proj_stride || state_stride < (long long)n_heads * D * Dv)
+        return SIA_BAD_ARGUMENT;
+    return launch_delta_rule<false>(qkv, qkv_stride, proj, proj_stride, g_col, b_col, a_col, a_log, dt_bias, norm_w, state,
+                                    state_stride, cu_q, slots, out, n_tokens, n_seqs, max_q_len, n_heads, n_kv, D, Dv, eps,
+                                    dtype, workspace, nullptr, nullptr, stream);
+}
+
+// The same rule with a decay per key channel (decays [tokens, n_heads, D]) and the output gate's factors (gates
+// [tokens, n_heads * Dv]) computed before, both float; b_col names the write strengths' logits in the rows of proj.
+SIA_EXPORT int sia_channel_delta_rule(const void* qkv, int qkv_stride, const void* proj, int proj_stride, int b_col,
+                                      const float* decays, const float* gates, const float* norm_w, float* state,
+                                      long long state_stride, const int* cu_q, const int* slots, void* out, int n_tokens,
+                                      int n_seqs, int max_q_len, int n_heads, int n_kv, int D, int Dv, float eps,
+                                      int dtype, float* workspace, hipStream_t stream) {
+    if (n_seqs <= 0 || n_tokens <= 0) return 0;
+    if (D <= 0 || Dv <= 0 || D > 512 || Dv > 512 || n_heads <= 0 || n_heads > 65535 || n_kv <= 0 || n_heads % n_kv ||
+        !state || !norm_w || !decays || !gates || !workspace || qkv_stride < 2 * n_kv * D + n_heads * Dv || b_col < 0 ||
+        b_col + n_heads > proj_stride || state_stride < (long long)n_heads * D * Dv)
+        return SIA_BAD_ARGUMENT;
+    return launch_delta_rule<true>(qkv, qkv_stride, proj, proj_stride, 0, b_col, 0, nullptr, nullptr, norm_w, state,
+                                   state_stride, cu_q, slots, out, n_tokens, n_seqs, max_q_len, n_heads, n_kv, D, Dv, eps,
+                                   dtype, workspace, decays, gates, stream);
 }

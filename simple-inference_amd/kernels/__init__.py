@@ -23,7 +23,7 @@ from . import build
 
 _DT = {torch.float32: 0, torch.bfloat16: 1}
 _ACTIVATIONS = {"relu2": 0, "gelu_tanh": 1, "gelu": 2}   # ``SiaActivation`` of csrc/common.h
-_GLUS = {"silu": 0, "clamped": 1}                        # ``SiaGlu`` of csrc/common.h
+_GLUS = {"silu": 0, "clamped": 1, "relu": 2}             # ``SiaGlu`` of csrc/common.h
 
 _c_int, _c_float, _c_ptr, _c_ll = ctypes.c_int, ctypes.c_float, ctypes.c_void_p, ctypes.c_longlong
 
@@ -62,9 +62,9 @@ _SIGNATURES = {
                      _c_ptr],
     "sia_latent_prepare": [_c_ptr, _c_int, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_float,
                            _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_int,
-                           _c_ptr],
+                           _c_int, _c_ptr],
     "sia_headwise_linear": [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                            _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr],
+                            _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
     "sia_moe_gate_up": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "sia_moe_tiled_workspace": [_c_int, _c_int, _c_int, _c_int, _c_int],
     "sia_moe_tiled": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
@@ -78,8 +78,8 @@ _SIGNATURES = {
     "sia_rope_kv_write": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
                           _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "sia_attention_generic": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr,
-                              _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_ptr, _c_int,
-                              _c_ptr],
+                              _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_ptr, _c_float,
+                              _c_int, _c_int, _c_ptr],
     "sia_attention_max_head_dim": [],
     "sia_attention_generic_max_head_dim": [],
     "sia_gemm_generic": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
@@ -109,13 +109,24 @@ _SIGNATURES = {
     "sia_glu": [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr],
     "sia_qk_prepare_ex": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int,
                           _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr,
-                          _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr],
+                          _c_int, _c_int, _c_float, _c_int, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr],
     "sia_decay_attention": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int,
                             _c_int, _c_int, _c_float, _c_int, _c_ptr, _c_ptr],
     "sia_delta_rule_workspace": [_c_int, _c_int, _c_int],
     "sia_delta_rule": [_c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_ptr,
                        _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr,
                        _c_ptr],
+    "sia_channel_delta_rule": [_c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_ptr,
+                               _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr,
+                               _c_ptr],
+    "sia_low_rank_pair": [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_int, _c_int,
+                          _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
+    "sia_add_layernorm": [_c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float,
+                          _c_int, _c_ptr],
+    "sia_embedding_gate": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+    "sia_gemm_skinny_embedding_gate": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_int,
+                                       _c_int, _c_ptr, _c_ptr],
+    "sia_element_gate": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "sia_moe_route_corrected": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "sia_moe_gate_up_ex": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int,
                            _c_ptr],
@@ -139,6 +150,14 @@ _ATTN_SIGNATURES = {
     "sia_attn_prefill_ex": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr,
                             _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
                             _c_int, _c_int, _c_ptr, _c_ptr],
+    "sia_attn_decode_forms": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                              _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_ptr, _c_float, _c_int,
+                              _c_int, _c_ptr],
+    "sia_attn_prefill_forms": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr,
+                               _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
+                               _c_int, _c_int, _c_ptr, _c_float, _c_int, _c_ptr],
+    "sia_attn_decode_walk": [_c_int, _c_int, _c_int],
+    "sia_attn_mfma_forms": [],
     "sia_attn_decode_max_splits": [_c_int, _c_int],
     "sia_attn_decode_workspace": [_c_int, _c_int, _c_int, _c_int, _c_int],
     "sia_attn_decode_mode": [_c_int, _c_int, _c_int, _c_int],
@@ -149,9 +168,11 @@ _ATTN_SIGNATURES = {
 }
 
 
-def attention_library_spec(head_dim: int):
-    """(name, sources, defines) of the matrix-core attention library for one head size."""
-    return (f"attn_mfma_d{head_dim}", ("attention_mfma.hip",), (f"SIA_HEAD_DIM={head_dim}",))
+def attention_library_spec(head_dim: int, forms: bool = False):
+    """(name, sources, defines) of the matrix-core attention library for one head size; ``forms``: the build that also
+    takes a soft cap on the scores and kept first positions."""
+    return (f"attn_mfma_d{head_dim}{'_forms' if forms else ''}", ("attention_mfma.hip",),
+            (f"SIA_HEAD_DIM={head_dim}",) + (("SIA_SCORE_FORMS=1",) if forms else ()))
 
 
 class KernelError(RuntimeError):
@@ -294,17 +315,17 @@ class HipKernels:
         y = torch.mm(x, w.t())
         return self.cast(y, torch.float32) if out_float32 else y
 
-    def _attn_lib(self, head_dim: int):
+    def _attn_lib(self, head_dim: int, forms: bool = False):
         """The matrix-core attention kernels for this head size, compiled at first use."""
-        lib = self._attn_libs.get(head_dim)
+        lib = self._attn_libs.get((head_dim, forms))
         if lib is None:
-            name, sources, defines = attention_library_spec(head_dim)
+            name, sources, defines = attention_library_spec(head_dim, forms)
             lib = build.load_library(name, sources, defines)
             _bind(lib, _ATTN_SIGNATURES)
             lib.sia_attn_decode_workspace.restype = ctypes.c_longlong
-            if lib.sia_attn_mfma_head_dim() != head_dim:
-                raise KernelError(f"library {name} was built for another head size")
-            self._attn_libs[head_dim] = lib
+            if lib.sia_attn_mfma_head_dim() != head_dim or bool(lib.sia_attn_mfma_forms()) != forms:
+                raise KernelError(f"library {name} was built for another head size or other forms")
+            self._attn_libs[(head_dim, forms)] = lib
         return lib
 
     # -- helpers -------------------------------------------------------------
@@ -384,6 +405,82 @@ class HipKernels:
         self._check(self.core.sia_norm_add(_ptr(residual), _ptr(y), _ptr(weight), _ptr(lowered), n, hidden, float(eps),
                                            _DT[out_dtype], self._stream()), "norm_add")
         return residual if lowered is None else lowered
+
+    # -- residual add (of a result, or of its rms norm) + layer norm -----------------
+    def add_layernorm(self, residual, delta, post, weight, bias, eps, out_dtype, rows=None):
+        """``x = residual + delta`` (with ``post = (gain, post_eps)``: plus ``delta * rsqrt(mean(delta^2) + post_eps) *
+        gain``) and the layer norm of ``x`` with ``weight`` and ``bias`` in ``out_dtype``.  Without ``rows`` the float
+        residual is left updated; with ``rows`` (int32 indices) only those rows are computed and it stays as it was."""
+        self._want(residual, "residual", torch.float32)
+        n, hidden = residual.shape
+        if out_dtype not in _DT:
+            raise KernelError(f"norm output dtype {out_dtype} is not float32 or bfloat16")
+        self._want(weight, "norm weight", torch.float32, (hidden,))
+        self._want(bias, "norm bias", torch.float32, (hidden,))
+        if delta is not None:
+            self._want(delta, "delta", out_dtype, (n, hidden))
+        gain, post_eps = post if post is not None else (None, 0.0)
+        if gain is not None:
+            if delta is None:
+                raise KernelError("a norm of the delta comes with a delta")
+            self._want(gain, "the delta's norm weight", torch.float32, (hidden,))
+        n_out = n
+        if rows is not None:
+            self._want(rows, "rows", torch.int32)
+            n_out = rows.numel()
+        out = torch.empty((n_out, hidden), dtype=out_dtype, device=residual.device)
+        self._check(self.core.sia_add_layernorm(_ptr(residual), _ptr(delta), _ptr(gain), float(post_eps), _ptr(weight),
+                                                _ptr(bias), _ptr(out), _ptr(rows), n_out, hidden, float(eps),
+                                                _DT[out_dtype], self._stream()), "add_layernorm")
+        return out
+
+    def add_lowered(self, residual, delta, out_dtype):
+        """``residual += delta`` (float); returns the new residual in ``out_dtype`` (the residual itself if that is
+        float32).  A product left pending is computed straight into the residual."""
+        self._want(residual, "residual", torch.float32)
+        n, hidden = residual.shape
+        if isinstance(delta, PendingProduct):
+            if out_dtype == torch.bfloat16:
+                ones = getattr(self, "_ones", None)
+                if ones is None or ones.numel() != hidden or ones.device != residual.device:
+                    ones = self._ones = torch.ones(hidden, dtype=torch.float32, device=residual.device)
+                return self.linear_into_residual(delta, residual, ones, 0.0).rows     # times a gain of one: x itself
+            delta = delta.compute()
+        if out_dtype not in _DT:
+            raise KernelError(f"output dtype {out_dtype} is not float32 or bfloat16")
+        self._want(delta, "delta", out_dtype, (n, hidden))
+        out = None if out_dtype == torch.float32 else torch.empty((n, hidden), dtype=out_dtype, device=residual.device)
+        self._check(self.core.sia_add_layernorm(_ptr(residual), _ptr(delta), None, 0.0, None, None, _ptr(out), None, n,
+                                                hidden, 0.0, _DT[out_dtype], self._stream()), "add_lowered")
+        return residual if out is None else out
+
+    # -- what a layer takes of the token itself -----------------------------------------
+    def embedding_gate(self, x, w, activation, table, first_column, dim, token_ids):
+        """``act(x @ w^T) * table[token_ids, first_column : first_column + dim]`` in the first ``dim`` columns and zeros
+        in the others (``w`` may have further, zero rows): one kernel for few rows, else the product and a kernel."""
+        if activation not in _ACTIVATIONS:
+            raise KernelError(f"activation {activation!r} is not one of {', '.join(_ACTIVATIONS)}")
+        self._want(x, "linear input")
+        self._want(w, "linear weight", x.dtype)
+        self._want(table, "embedding table", x.dtype)
+        if x.dtype not in _DT or x.dim() != 2 or w.dim() != 2 or x.shape[1] != w.shape[1] or table.dim() != 2:
+            raise KernelError(f"embedding gate shapes do not fit: x {tuple(x.shape)}, w {tuple(w.shape)}, table {tuple(table.shape)}")
+        M, K = x.shape
+        N, width = w.shape[0], table.shape[1]
+        self._want(token_ids, "token ids", torch.int32, (M,))
+        if not 0 < dim <= N or first_column < 0 or first_column + dim > width:
+            raise KernelError(f"{dim} columns from {first_column} on do not fit a table row of {width} and {N} outputs")
+        if self.use_skinny_gemm and x.dtype == torch.bfloat16 and 0 < M <= self._skinny_rows and K % 64 == 0:
+            y = torch.empty((M, N), dtype=torch.bfloat16, device=x.device)
+            self._check(self.core.sia_gemm_skinny_embedding_gate(
+                _ptr(x), _ptr(w), _ptr(y), M, N, K, _ACTIVATIONS[activation], _ptr(table), width, int(first_column),
+                int(dim), _ptr(token_ids), self._stream()), "gemm_skinny_embedding_gate")
+            return y
+        z = self.linear(x, w)
+        self._check(self.core.sia_embedding_gate(_ptr(z), _ptr(z), _ptr(table), width, int(first_column), int(dim),
+                                                 _ptr(token_ids), M, N, _ACTIVATIONS[activation], _DT[x.dtype],
+                                                 self._stream()), "embedding_gate")
+        return z
 
     # -- residual add + rms norm ---------------------------------------------
     def add_rmsnorm(self, residual, delta, weight, eps, out_dtype, rows=None, gate=None, gate_bias=None,
@@ -512,6 +609,20 @@ class HipKernels:
         self._check(self.core.sia_head_gate(_ptr(out), _ptr(logits), stride, n, n_heads, width // n_heads,
                                             _DT[out.dtype], self._stream()), "head_gate")
         return out
+
+    def element_gate(self, out, logits, n_heads):
+        """``out[n, h, d] * sigmoid(logits[n, h, d])`` for the heads' own elements: rows of ``n_heads`` heads that may be
+        wider than their gates become rows of heads as wide as these; ``logits`` may be columns of a wider matrix."""
+        self._want(out, "attention output")
+        n, width = out.shape
+        own = logits.shape[1] // n_heads
+        if out.dtype not in _DT or width % n_heads or logits.shape[1] != own * n_heads or width // n_heads < own:
+            raise KernelError(f"gates {tuple(logits.shape)} do not fit rows of {n_heads} heads, {out.dtype} {tuple(out.shape)}")
+        stride = self._columns(logits, "element gate logits", out.dtype, (n, n_heads * own))
+        gated = torch.empty((n, n_heads * own), dtype=out.dtype, device=out.device)
+        self._check(self.core.sia_element_gate(_ptr(out), _ptr(logits), stride, _ptr(gated), n, n_heads,
+                                               width // n_heads, own, _DT[out.dtype], self._stream()), "element_gate")
+        return gated
 
     def side_by_side(self, a, b, dtype):
         """``[a, b]`` along the columns, lowered to ``dtype``: two float streams as the input of one product."""
@@ -801,6 +912,46 @@ class HipKernels:
             n_kv_heads, key_dim, value_dim, float(eps), _DT[qkv.dtype], _ptr(workspace), self._stream()), "delta_rule")
         return out
 
+    def channel_delta_rule(self, qkv, proj, columns, a2, g2, a_log, dt_bias, norm_weight, n_heads, n_kv_heads, key_dim,
+                           value_dim, eps, ctx, state):
+        """The delta rule with a decay per head and key channel.  ``qkv`` as for ``delta_rule``; ``columns = (b, a, g)``
+        name the write strengths' logits ``[heads]`` and the low-rank inputs of the decays ``[rank of a2]`` and of the
+        output gate ``[rank of g2]`` in the rows of ``proj``.  ``decay = exp(-exp(a_log) * softplus(a2 a + dt_bias))``
+        ``[heads, key_dim]``, ``gate = sigmoid(g2 g)``, both in float; per head ``S <- decay S; S += k (beta (v - S^T
+        k))^T; o = S^T q``; ``o`` is divided by its root mean square, multiplied by ``norm_weight`` and by ``gate``."""
+        self._want(qkv, "convolved rows")
+        self._want(proj, "projected rows", qkv.dtype)
+        n, width = qkv.shape
+        qk, inner, channels = n_kv_heads * key_dim, n_heads * value_dim, n_heads * key_dim
+        if qkv.dtype not in _DT or n != ctx.n_tokens or proj.shape[0] != n or width != 2 * qk + inner:
+            raise KernelError(f"rows {qkv.dtype} {tuple(qkv.shape)} do not fit {ctx.n_tokens} tokens of {n_kv_heads} "
+                              f"query/key heads of {key_dim} and {n_heads} value heads of {value_dim}")
+        self._want(a2, "decay matrix", qkv.dtype, (channels, a2.shape[1]))
+        self._want(g2, "gate matrix", qkv.dtype, (inner, g2.shape[1]))
+        b, a, g = (int(c) for c in columns)
+        for first, size, what in ((b, n_heads, "write strength"), (a, a2.shape[1], "decay"), (g, g2.shape[1], "gate")):
+            if first < 0 or first + size > proj.shape[1]:
+                raise KernelError(f"columns {first} .. {first + size} of the {what} lie outside a row of {proj.shape[1]}")
+        self._want(a_log, "decay rate", torch.float32, (n_heads,))
+        self._want(dt_bias, "step bias", torch.float32, (channels,))
+        self._want(norm_weight, "output norm weight", torch.float32, (value_dim,))
+        self.check_recurrent_geometry(key_dim, value_dim)
+        if n_kv_heads <= 0 or n_heads % n_kv_heads:
+            raise KernelError(f"{n_heads} value heads cannot share {n_kv_heads} query/key heads evenly")
+        stride = self._state_rows(state, ctx, n_heads * key_dim * value_dim)
+        out = torch.empty((n, inner), dtype=qkv.dtype, device=qkv.device)
+        raw = self.core.sia_delta_rule_workspace(n, n_heads, value_dim)
+        workspace = self._float_workspace(ctx, raw + n * (channels + inner), qkv.device)
+        decays, gates = workspace[raw:], workspace[raw + n * channels:]
+        self._check(self.core.sia_low_rank_pair(
+            _ptr(proj), proj.shape[1], a, a2.shape[1], _ptr(a2), _ptr(a_log), _ptr(dt_bias), channels, key_dim,
+            _ptr(decays), g, g2.shape[1], _ptr(g2), inner, _ptr(gates), n, _DT[qkv.dtype], self._stream()), "low_rank_pair")
+        self._check(self.core.sia_channel_delta_rule(
+            _ptr(qkv), width, _ptr(proj), proj.shape[1], b, _ptr(decays), _ptr(gates), _ptr(norm_weight), _ptr(state),
+            stride, _ptr(ctx.cu_q), _ptr(ctx.state_slots), _ptr(out), n, ctx.n_seqs, ctx.max_q_len, n_heads, n_kv_heads,
+            key_dim, value_dim, float(eps), _DT[qkv.dtype], _ptr(workspace), self._stream()), "channel_delta_rule")
+        return out
+
     def decay_attention(self, proj, decays, norm_weight, n_heads, key_dim, value_dim, eps, ctx, state):
         """Linear attention with a constant decay per head.  ``proj`` rows are ``[q | k (heads * key_dim each) | v | g
         (heads * value_dim each)]`` and are used up (q, k and v are overwritten by their ``silu``).  Per head ``S <-
@@ -840,14 +991,15 @@ class HipKernels:
         return cos, sin
 
     def latent_prepare(self, proj, q_rank, q_gain, kv_rank, kv_gain, rot_dim, rotary_dim, cos, sin, eps, ctx, cache,
-                       page_dim=None):
-        """From projected rows ``[a_q (q_rank) | a (kv_rank) | b (rot_dim)]``: returns ``rms(a_q) * q_gain`` and, if
+                       page_dim=None, pairing="interleaved"):
+        """From projected rows ``[a_q (q_rank) | a (kv_rank) | b (rot_dim) | further columns]``: returns ``rms(a_q) * q_gain`` and, if
         ``kv_rank`` is not 0, writes ``[rms(a) * kv_gain | rotate(b)]`` as the position's key row and ``rms(a) *
         kv_gain`` as its value into the pages (one key/value head; rows ``page_dim`` wide if given).  The rotation
-        turns neighbouring pairs of the first ``rotary_dim`` elements of ``b``."""
+        turns neighbouring pairs of the first ``rotary_dim`` elements of ``b``, or with ``pairing="half"`` element ``i``
+        with element ``i + rotary_dim / 2``."""
         self._want(proj, "projected rows")
         n, width = proj.shape
-        if proj.dtype not in _DT or n != ctx.n_tokens or width != q_rank + (kv_rank + rot_dim if kv_rank else 0):
+        if proj.dtype not in _DT or n != ctx.n_tokens or width < q_rank + (kv_rank + rot_dim if kv_rank else 0):
             raise KernelError(f"projected rows {proj.dtype} {tuple(proj.shape)} do not fit {ctx.n_tokens} tokens of "
                               f"{q_rank} + {kv_rank} + {rot_dim} columns")
         self._want(q_gain, "query latent gain", torch.float32, (q_rank,))
@@ -865,15 +1017,23 @@ class HipKernels:
             _ptr(proj), width, q_rank, _ptr(q_gain), kv_rank, _ptr(kv_gain), rot_dim, rotary_dim if kv_rank else 0,
             _ptr(cos) if kv_rank else None, _ptr(sin) if kv_rank else None, float(eps), _ptr(ctx.positions),
             _ptr(ctx.seq_of_token), _ptr(table), table.shape[1] if table is not None else 0, _ptr(k_pages),
-            _ptr(v_pages), page_size, key_width, value_rows, _ptr(cq), n, _DT[proj.dtype], self._stream()),
+            _ptr(v_pages), page_size, key_width, value_rows, _ptr(cq), n, self._halves(pairing), _DT[proj.dtype], self._stream()),
             "latent_prepare")
         return cq
 
-    def headwise_linear(self, x, w, in_stride, out_stride, tail=0, rotation=None):
+    @staticmethod
+    def _halves(pairing) -> int:
+        if pairing not in ("interleaved", "half"):
+            raise KernelError(f"pairing must be 'interleaved' or 'half', got {pairing!r}")
+        return int(pairing == "half")
+
+    def headwise_linear(self, x, w, in_stride, out_stride, tail=0, rotation=None, gate=None, pairing="interleaved"):
         """A product per head: ``y[n, h, :out] = w[h] x[n, h, :in]`` for ``w [heads, out, in]``, ``x`` rows holding
         ``in_stride`` elements a head and ``y`` rows ``out_stride``.  The ``tail`` elements behind a head's inputs are
         copied behind its outputs, their first ``rotary_dim`` elements turned in neighbouring pairs by ``rotation =
-        (rotary_dim, cos, sin, positions)``; what is left of a head's ``out_stride`` is zero."""
+        (rotary_dim, cos, sin, positions)`` (with ``pairing="half"`` element ``i`` with ``i + rotary_dim / 2``); what is
+        left of a head's ``out_stride`` is zero.  ``gate [n, heads * out]`` (which may be columns of a wider matrix): every
+        output is multiplied by the sigmoid of its logit."""
         self._want(x, "headwise input")
         self._want(w, "headwise weights", x.dtype)
         if x.dtype not in _DT or w.dim() != 3:
@@ -892,20 +1052,25 @@ class HipKernels:
                 self._want(t, what, torch.float32)
                 if t.shape[1] != rotary_dim // 2:
                     raise KernelError(f"{what} {tuple(t.shape)} does not hold {rotary_dim // 2} pairs")
+        gate_stride = self._columns(gate, "gate logits", x.dtype, (n, heads * out_dim)) if gate is not None else 0
         y = torch.empty((n, heads * out_stride), dtype=x.dtype, device=x.device)
         self._check(self.core.sia_headwise_linear(
             _ptr(x), width, in_stride, _ptr(w), _ptr(y), heads * out_stride, out_stride, n, heads, in_dim, out_dim,
             int(tail), int(rotary_dim), _ptr(cos) if rotary_dim else None, _ptr(sin) if rotary_dim else None,
-            _ptr(positions) if rotary_dim else None, _DT[x.dtype], self._stream()), "headwise_linear")
+            _ptr(positions) if rotary_dim else None, self._halves(pairing), _ptr(gate), gate_stride, _DT[x.dtype],
+            self._stream()), "headwise_linear")
         return y
 
     @staticmethod
     def _glu(activation):
         """(kind, limit) of a gated activation as the kernels take it: None is ``silu(g) * u``, ``("clamped", limit)`` is
-        ``g * sigmoid(1.702 g) * (u + 1)`` with ``g = min(g, limit)`` and ``u = clamp(u, -limit, limit)``."""
+        ``g * sigmoid(1.702 g) * (u + 1)`` with ``g = min(g, limit)`` and ``u = clamp(u, -limit, limit)``, ``("relu",
+        None)`` is ``max(g, 0) * u``."""
         if activation is None:
             return _GLUS["silu"], 0.0
         kind, limit = activation
+        if kind == "relu" and limit is None:
+            return _GLUS["relu"], 0.0
         if kind not in _GLUS or not float(limit) > 0:
             raise KernelError(f"gated activation {activation!r} is not one of {', '.join(_GLUS)} with a positive limit")
         return _GLUS[kind], float(limit)
@@ -1205,7 +1370,7 @@ class HipKernels:
 
     def qkv_to_cache(self, x, w_qkv, n_heads, n_kv_written, head_dim, rotary_dim, cos, sin, ctx, cache,
                      value_dim=None, bias=None, qk_norm=None, page_dim=None, q_temp=None, extra_columns=0,
-                     values_are_keys=False):
+                     values_are_keys=False, value_mix=None, give_values=False):
         """The q/k/v product, the rotation of q and k and the write of k and v into the pages.  Returns the
         ``[tokens, (n_heads + 2 n_kv_written) head_dim]`` matrix whose q columns hold the rotated queries; its
         k and v columns are not to be read (for few rows one kernel does all three and never writes them).
@@ -1222,10 +1387,12 @@ class HipKernels:
         after its norm.  ``extra_columns``: the weight has that many further rows behind v, whose products are only
         carried along; the result is then the pair (that matrix, the further columns of the projected rows).
         ``values_are_keys``: the weight has no v rows; a position's values are its keys as projected (with their bias,
-        before norm and rotation)."""
+        before norm and rotation).  ``value_mix``: ``(given, m)``, the values cached are ``(1 - m) v + m given`` with
+        ``given [tokens, n_kv_written * value_dim]`` (columns of a wider matrix) and the one float ``m`` on the device.
+        ``give_values``: the v columns of the projected rows are returned too, behind what is returned otherwise."""
         M, K = x.shape
         if (value_dim is not None or bias is not None or qk_norm is not None or page_dim is not None
-                or q_temp is not None or extra_columns or values_are_keys):
+                or q_temp is not None or extra_columns or values_are_keys or value_mix is not None or give_values):
             qkv = self.linear(x, w_qkv)
             q_out = None
             if page_dim is not None:
@@ -1239,11 +1406,14 @@ class HipKernels:
                 if q_out is None:
                     q_out = kept[key] = torch.zeros((M, n_heads * page_dim), dtype=qkv.dtype, device=qkv.device)
             self.qk_prepare(qkv, n_heads, n_kv_written, head_dim, value_dim or head_dim, rotary_dim, cos, sin, bias,
-                            qk_norm, ctx, cache, page_dim, q_out, q_temp, extra_columns, values_are_keys)
-            queries = qkv if q_out is None else q_out
+                            qk_norm, ctx, cache, page_dim, q_out, q_temp, extra_columns, values_are_keys, value_mix)
+            out = [qkv if q_out is None else q_out]
             if extra_columns:
-                return queries, qkv[:, qkv.shape[1] - extra_columns:]
-            return queries
+                out.append(qkv[:, qkv.shape[1] - extra_columns:])
+            if give_values:
+                v0 = (n_heads + n_kv_written) * head_dim
+                out.append(qkv[:, v0:v0 + n_kv_written * (value_dim or head_dim)])
+            return tuple(out) if len(out) > 1 else out[0]
         if (self.use_skinny_gemm and self.fuse_rope and n_kv_written and x.dtype == torch.bfloat16 and w_qkv.dtype == torch.bfloat16
                 and M <= self._skinny_rows and rotary_dim == head_dim and head_dim % 2 == 0 and K % 64 == 0):
             x, partials, n_partials, norm_eps = self._scaled(x)
@@ -1287,7 +1457,7 @@ class HipKernels:
         return wide
 
     def qk_prepare(self, qkv, n_heads, n_kv_written, head_dim, value_dim, rotary_dim, cos, sin, bias, qk_norm, ctx,
-                   cache, page_dim=None, q_out=None, q_temp=None, extra_columns=0, values_are_keys=False):
+                   cache, page_dim=None, q_out=None, q_temp=None, extra_columns=0, values_are_keys=False, value_mix=None):
         """Bias, per-head RMS norm of q and k, rotation, and the write of k and v into the pages, on the projected
         rows ``[q heads | k heads | v heads]`` (q and k heads ``head_dim`` wide, v heads ``value_dim``); q is left in
         place."""
@@ -1322,6 +1492,14 @@ class HipKernels:
             q_gain, k_gain, eps = qk_norm
             self._want(q_gain, "q norm gain", torch.float32, (head_dim,))
             self._want(k_gain, "k norm gain", torch.float32, (head_dim,))
+        given = mix = None
+        given_stride = 0
+        if value_mix is not None:
+            given, mix = value_mix
+            self._want(mix, "value mix", torch.float32, (1,))
+            given_stride = self._columns(given, "given values", qkv.dtype, (n, n_kv_written * value_dim))
+            if values_are_keys or not n_kv_written:
+                raise KernelError("values are mixed where they are projected and written")
         table = k_pages = v_pages = None
         page_size = 0
         k_row, v_rows = head_dim, value_dim
@@ -1339,7 +1517,7 @@ class HipKernels:
             _ptr(ctx.seq_of_token), _ptr(table), table.shape[1] if table is not None else 0, _ptr(k_pages),
             _ptr(v_pages), n, n_heads, n_kv_written, head_dim, value_dim, rotary_dim, page_size, k_row, v_rows,
             _ptr(q_out), n_heads * page_dim if page_dim else 0, page_dim or 0, temp_coef, temp_every,
-            int(bool(values_are_keys)), _DT[qkv.dtype], self._stream()), "qk_prepare")
+            int(bool(values_are_keys)), _ptr(given), given_stride, _ptr(mix), _DT[qkv.dtype], self._stream()), "qk_prepare")
 
     def _check_pages(self, k_pages, v_pages, table, page_size, n_kv, head_dim, dtype, ctx, value_dim=None):
         value_dim = value_dim or head_dim
@@ -1369,11 +1547,12 @@ class HipKernels:
             raise KernelError(f"{n_heads} query heads exceed the kernels' grids (65,535)")
 
     def paged_attention(self, qkv, n_heads, n_kv_heads, head_dim, scale, window, ctx, cache, value_dim=None,
-                        chunk=None, sinks=None):
+                        chunk=None, sinks=None, softcap=None, keep_first=0):
         """Attention of the rows' q columns over the pages.  ``chunk``: a query sees only the keys of its own block
         of that many positions; ``sinks``: float ``[n_heads]``, one more term ``exp(sink_h)`` in every softmax
         denominator of head h; ``value_dim``: width of the value rows if not ``head_dim`` (the result is
-        ``[tokens, n_heads * value_dim]``)."""
+        ``[tokens, n_heads * value_dim]``); ``softcap``: scaled scores become ``c * tanh(s / c)``; ``keep_first``: with a
+        window, the first positions of the sequence stay visible to every query."""
         self._want(qkv, "qkv")
         n, width = qkv.shape
         value_dim = int(value_dim or head_dim)
@@ -1385,29 +1564,35 @@ class HipKernels:
             self._want(sinks, "sinks", torch.float32, (n_heads,))
         if chunk is not None and chunk <= 0:
             raise KernelError(f"chunk must be positive, got {chunk}")
+        if softcap is not None and not softcap > 0:
+            raise KernelError(f"a soft cap must be positive, got {softcap}")
+        if keep_first < 0 or (keep_first and (chunk is not None or not window)):
+            raise KernelError(f"first positions are kept behind a window, got keep_first {keep_first}")
         out = torch.empty((n, n_heads * value_dim), dtype=qkv.dtype, device=qkv.device)
         page = cache.page_size
         if (self.use_mfma_attention and qkv.dtype == torch.bfloat16 and head_dim % 16 == 0 and head_dim <= 256
                 and value_dim == head_dim and page >= 8 and width % 8 == 0 and scale > 0):
             self._mfma_attention(qkv, out, n_heads, n_kv_heads, head_dim, scale, int(window or 0), ctx, cache,
-                                 int(chunk or 0), sinks)
+                                 int(chunk or 0), sinks, float(softcap or 0.0), int(keep_first))
             return out
         self._check(self.core.sia_attention_generic(
             _ptr(qkv), width, _ptr(cache.k_pages), _ptr(cache.v_pages), _ptr(cache.block_table),
             cache.block_table.shape[1], _ptr(ctx.seq_of_token), _ptr(ctx.positions), _ptr(out), n, n_heads,
             n_kv_heads, head_dim, value_dim, page, float(scale), int(window or 0), int(chunk or 0), _ptr(sinks),
-            _DT[qkv.dtype], self._stream()), "attention_generic")
+            float(softcap or 0.0), int(keep_first), _DT[qkv.dtype], self._stream()), "attention_generic")
         return out
 
-    def _attention_plan(self, lib, device, n_heads, n_kv_heads, head_dim, window, ctx, chunk=0):
+    def _attention_plan(self, lib, device, n_heads, n_kv_heads, head_dim, window, ctx, chunk=0, keep_first=0, page_size=0):
         """What the attention launches of a step need beside the tensors: the same for every layer with this
         geometry, so it is worked out once per step and kept with the step's context (workspaces included: a step's
         layers run one after the other)."""
-        key = (n_heads, n_kv_heads, head_dim, window, chunk)
+        key = (n_heads, n_kv_heads, head_dim, window, chunk, keep_first)
         plans = getattr(ctx, "attention_plans", None)
         span = min(b for b in (window, chunk) if b > 0) if (window > 0 or chunk > 0) else 0   # most keys a query sees
         if plans is not None and key in plans:
             return plans[key]
+        if keep_first:
+            span = lib.sia_attn_decode_walk(window, keep_first, page_size)
         # the decode kernel takes up to 16 query heads a key/value head (and what its LDS holds of their states): more
         # are dealt out as several groups that read the same head
         group = n_heads // n_kv_heads
@@ -1440,24 +1625,26 @@ class HipKernels:
         plans[key] = plan
         return plan
 
-    def _mfma_attention(self, qkv, out, n_heads, n_kv_heads, head_dim, scale, window, ctx, cache, chunk=0, sinks=None):
-        lib = self._attn_lib(head_dim)
+    def _mfma_attention(self, qkv, out, n_heads, n_kv_heads, head_dim, scale, window, ctx, cache, chunk=0, sinks=None,
+                        softcap=0.0, keep_first=0):
+        lib = self._attn_lib(head_dim, forms=softcap > 0 or keep_first > 0)
         width = qkv.shape[1]
         table = cache.block_table
         n_dec, max_splits, ws_acc, ws_ml, (n_tiles, n_tiles_split, n_tiles_long, q_bound, kv_bound), share = \
-            self._attention_plan(lib, qkv.device, n_heads, n_kv_heads, head_dim, window, ctx, chunk)
+            self._attention_plan(lib, qkv.device, n_heads, n_kv_heads, head_dim, window, ctx, chunk, keep_first,
+                                 cache.page_size)
         if n_dec:
-            self._check(lib.sia_attn_decode_shared(
+            self._check(lib.sia_attn_decode_forms(
                 _ptr(qkv), width, _ptr(cache.k_pages), _ptr(cache.v_pages), _ptr(table), table.shape[1],
                 _ptr(ctx.cu_q), _ptr(ctx.kv_len), _ptr(out), _ptr(ws_acc), _ptr(ws_ml), n_dec, n_heads,
-                n_kv_heads * share, share, cache.page_size, float(scale), window, chunk, _ptr(sinks), max_splits,
-                self._stream()), "attn_decode")
+                n_kv_heads * share, share, cache.page_size, float(scale), window, chunk, _ptr(sinks), softcap, keep_first,
+                max_splits, self._stream()), "attn_decode")
         if n_dec < ctx.n_seqs:
-            self._check(lib.sia_attn_prefill_ex(
+            self._check(lib.sia_attn_prefill_forms(
                 _ptr(qkv), width, _ptr(cache.k_pages), _ptr(cache.v_pages), _ptr(table), table.shape[1],
                 _ptr(ctx.cu_q), _ptr(ctx.kv_len), _ptr(out), n_dec, ctx.n_seqs, n_tiles, n_tiles_split, n_tiles_long,
                 q_bound, kv_bound, n_heads, n_kv_heads, cache.page_size, float(scale), window, chunk, _ptr(sinks),
-                self._stream()), "attn_prefill")
+                softcap, keep_first, self._stream()), "attn_prefill")
 
     # -- a whole block in one call -------------------------------------------------
     def _library_can(self, M, N, K) -> bool:

@@ -32,6 +32,13 @@ Further forms, each switched on by a parameter of its own and free to combine:
   ``1 + c * ln(floor((p + 1) / n) + 1)`` after its norm, so late queries score more sharply.
 * ``out_gate``: head ``h``'s output is multiplied by ``sigmoid((G x)_h)``, a scalar for every token and head, ``G
   [Hq, H]`` reading the mixer's own input; its rows ride at the end of the stacked projection.
+  ``out_gate: "element"``: every element of the heads has a gate of its own, ``sigmoid((G x)_i)`` with ``G [Hq Dv, H]``.
+* ``softcap``: scores are capped softly after the scale, ``c * tanh(s / c)``.
+* ``keep_first``: with a window, the sequence's first ``keep_first`` positions stay visible to every query, at their
+  true positions; their pages stay with the request.
+* ``value_mix``: values are mixed between layers.  The layer that ``"gives"`` leaves the values it projected to the
+  step; a layer that ``"takes"`` caches ``(1 - m) v + m v_given`` of the same token, ``m`` its learned scalar (the
+  layer that gives has one too and does not use it).
 * ``value_from_key``: there is no value projection: a position's values are its keys as projected (with their bias,
   before norm and rotation); the stacked matrix is ``[(Hq + Hkv) D, H]``.
 * ``o_bias``: the output projection has a bias; it is handed on with the result (``BiasedDelta``) so that the sum
@@ -60,7 +67,8 @@ def _shared_position_encoding(spec, env):
 class Attention:
     """params: hidden_size, num_heads, num_kv_heads, head_dim, position
     (``{"kind", "params"}``), and optionally window, scale, kv_from_layer, value_head_dim, bias, qk_norm, chunk,
-    sink, q_temp, out_gate, o_bias, value_from_key."""
+    sink, q_temp, out_gate (True or "element"), o_bias, value_from_key, softcap, keep_first, value_mix ("gives" or
+    "takes")."""
 
     def __init__(self, params, env):
         self.hidden = int(params["hidden_size"])
@@ -86,7 +94,22 @@ class Attention:
         self.q_temp = (float(q_temp["coef"]), int(q_temp["every"])) if q_temp else None
         if self.q_temp is not None and self.q_temp[1] <= 0:
             raise ValueError(f"q_temp.every must be positive, got {self.q_temp[1]}")
-        self.out_gate = bool(params.get("out_gate", False))
+        out_gate = params.get("out_gate") or False
+        if out_gate not in (False, True, "element"):
+            raise ValueError(f"out_gate is True (a gate a head) or 'element', got {out_gate!r}")
+        self.out_gate = bool(out_gate)
+        self.element_gate = out_gate == "element"
+        self.softcap = float(params["softcap"]) if params.get("softcap") else None
+        if self.softcap is not None and not self.softcap > 0:
+            raise ValueError(f"a soft cap must be positive, got {self.softcap}")
+        self.keep_first = int(params.get("keep_first") or 0)
+        if self.keep_first < 0 or (self.keep_first and params.get("chunk") is not None):
+            raise ValueError(f"keep_first is a count of first positions behind a window, got {self.keep_first}")
+        if self.window is None:
+            self.keep_first = 0        # every position is visible anyway
+        self.value_mix = params.get("value_mix")
+        if self.value_mix not in (None, "gives", "takes"):
+            raise ValueError(f"value_mix is 'gives' or 'takes', got {self.value_mix!r}")
         self.o_bias = bool(params.get("o_bias", False))
         self.value_from_key = bool(params.get("value_from_key", False))
         if self.value_from_key and (self.value_dim != self.head_dim or params.get("kv_from_layer") is not None):
@@ -98,7 +121,7 @@ class Attention:
                 raise ValueError(f"chunk must be positive, got {self.chunk}")
         self.sink = bool(params.get("sink", False))
         if self.kv_from_layer is not None and (self.bias or self.qk_norm_eps is not None or self.value_dim != self.head_dim
-                                               or self.out_gate or self.q_temp is not None):
+                                               or self.out_gate or self.q_temp is not None or self.value_mix):
             raise ValueError("a mixer that reads another layer's keys and values has plain q heads of the keys' width")
         self.position = _shared_position_encoding(params.get("position", {"kind": "none", "params": {}}), env)
         if self.position.rotary_dim > self.head_dim:
@@ -114,12 +137,18 @@ class Attention:
         self.w_o = None
         self.b_qkv = self.q_gain = self.k_gain = self.sinks = self.b_o = None
         self.gate_columns = 0
+        self.mix = None
 
     takes_scaled_rows = True   # the input goes to ``qkv_to_cache`` only
 
     @property
     def writes_kv(self) -> bool:
         return self.kv_from_layer is None
+
+    @property
+    def gates(self) -> int:
+        """Gates a token has on the heads' outputs."""
+        return self.num_heads * self.value_dim if self.element_gate else self.num_heads
 
     def weight_specs(self):
         q = self.num_heads * self.head_dim
@@ -139,7 +168,9 @@ class Attention:
         if self.sink:
             specs["sink"] = TensorSpec((self.num_heads,), "vector")
         if self.out_gate:
-            specs["gate"] = TensorSpec((self.num_heads, self.hidden))
+            specs["gate"] = TensorSpec((self.gates, self.hidden))
+        if self.value_mix:
+            specs["value_mix"] = TensorSpec((), "vector")
         if self.o_bias:
             specs["o_bias"] = TensorSpec((self.hidden,), "vector")
         return specs
@@ -149,12 +180,16 @@ class Attention:
         if self.writes_kv:
             stacked += [tensors["k"]] if self.value_from_key else [tensors["k"], tensors["v"]]
         if self.out_gate:   # the gate's rows behind v, filled up with zero rows so that a projected row stays aligned
-            self.gate_columns = -(-self.num_heads // 8) * 8
+            self.gate_columns = -(-self.gates // 8) * 8
             g = tensors["gate"]
-            stacked += [g, g.new_zeros((self.gate_columns - self.num_heads, self.hidden))]
+            stacked += [g, g.new_zeros((self.gate_columns - self.gates, self.hidden))]
+        if self.value_mix == "takes":
+            self.mix = tensors["value_mix"].reshape(1).float().contiguous()
         self.w_qkv = torch.cat(stacked, dim=0).contiguous()
         self.w_o = tensors["o"].contiguous()
-        if self.page_dim is not None:   # the attention's rows come with page_dim elements a head: zero columns for the rest
+        if self.page_dim is not None and not self.element_gate:
+            # the attention's rows come with page_dim elements a head: zero columns for the rest (the elements' gate
+            # leaves the heads' own elements only)
             wide = self.w_o.new_zeros((self.hidden, self.num_heads, self.page_dim))
             wide[:, :, :self.value_dim] = self.w_o.view(self.hidden, self.num_heads, self.value_dim)
             self.w_o = wide.view(self.hidden, self.num_heads * self.page_dim)
@@ -186,13 +221,14 @@ class Attention:
     def _options(self) -> bool:
         """Whether any of the further forms is switched on (the kernels then get them as keyword arguments)."""
         return (self.bias or self.qk_norm_eps is not None or self.sink or self.chunk is not None
-                or self.value_dim != self.head_dim or self.q_temp is not None or self.out_gate or self.value_from_key)
+                or self.value_dim != self.head_dim or self.q_temp is not None or self.out_gate or self.value_from_key
+                or self.softcap is not None or self.keep_first > 0 or self.value_mix is not None)
 
     def cache_need(self):
         if self.page_dim is not None:
-            return PagedKVNeed(self.num_kv_heads, self.page_dim, self.window, None, self.chunk)
+            return PagedKVNeed(self.num_kv_heads, self.page_dim, self.window, None, self.chunk, self.keep_first)
         return PagedKVNeed(self.num_kv_heads, self.head_dim, self.window,
-                           self.value_dim if self.value_dim != self.head_dim else None, self.chunk)
+                           self.value_dim if self.value_dim != self.head_dim else None, self.chunk, self.keep_first)
 
     def state_need(self):
         return None
@@ -222,17 +258,29 @@ class Attention:
                 project["extra_columns"] = self.gate_columns
             if self.value_from_key:
                 project["values_are_keys"] = True
+            if self.softcap is not None:
+                attend["softcap"] = self.softcap
+            if self.keep_first:
+                attend["keep_first"] = self.keep_first
+            if self.value_mix == "gives":
+                project["give_values"] = True
+            elif self.value_mix == "takes":
+                project["value_mix"] = (ctx.shared["given_values"], self.mix)
         qkv = k.qkv_to_cache(
             h, self.w_qkv, self.num_heads, self.num_kv_heads if self.writes_kv else 0, self.head_dim,
             self.position.rotary_dim, cos, sin, ctx, cache, **project)
         gate_logits = None
+        if self.value_mix == "gives":
+            *qkv, ctx.shared["given_values"] = qkv
+            qkv = qkv if self.out_gate else qkv[0]
         if self.out_gate:
             qkv, further = qkv
-            gate_logits = further[:, :self.num_heads]
+            gate_logits = further[:, :self.gates]
         out = k.paged_attention(
             qkv, self.num_heads, self.num_kv_heads, self.page_dim or self.head_dim, self.scale, self.window, ctx, cache,
             **attend)
         if gate_logits is not None:
-            out = k.head_gate(out, gate_logits, self.num_heads)
+            out = (k.element_gate(out, gate_logits, self.num_heads) if self.element_gate
+                   else k.head_gate(out, gate_logits, self.num_heads))
         y = k.pending_linear(out, self.w_o)   # the norm after it may have it added into the residual
         return BiasedDelta(y, self.b_o, k) if self.o_bias else y

@@ -5,7 +5,9 @@ Pre-norm (reference: ``model/block.py:135-147``):
 as the stream's pending delta and summed into the float32 residual by the norm
 that follows (the next layer's, or the model's last norm).  With ``residual_scale`` (a parameter of the block, from
 the layer's ``block_params``) every sublayer's result is multiplied by that constant on its way into the residual
-(``stream.scale``); a pre-norm layer may have no feed-forward.
+(``stream.scale``); a pre-norm layer may have no feed-forward.  It may take something of the token itself as its last
+sublayer: ``x += token_input_norm(token_input(x))``, a part that reads the un-normed stream (in the compute dtype) and
+the step's token ids, behind a norm of its own, which is applied by the norm that follows (``stream.post``).
 
 Output-norm: ``x += norm1(mixer(x))``; ``x += norm2(feed_forward(x))``.  Mixer and feed-forward take the
 un-normed stream as input (rounded to the compute dtype), and each norm is applied to its sublayer's result; the kernel that adds the normed
@@ -25,9 +27,14 @@ from .registry import register_block
 
 @register_block("prenorm")
 class PreNormBlock:
-    def __init__(self, mixer, feed_forward=None, mixer_norm=None, feed_forward_norm=None, residual_scale=None):
+    def __init__(self, mixer, feed_forward=None, mixer_norm=None, feed_forward_norm=None, residual_scale=None,
+                 token_input=None, token_input_norm=None):
         if mixer_norm is None or (feed_forward is None) != (feed_forward_norm is None):
             raise ValueError("a pre-norm block has a mixer with its norm, and a feed-forward with its norm or neither")
+        if (token_input is None) != (token_input_norm is None):
+            raise ValueError("a pre-norm block has a token input with its norm, or neither")
+        self.token_input = token_input
+        self.token_input_norm = token_input_norm
         self.mixer = mixer
         self.feed_forward = feed_forward
         self.mixer_norm = mixer_norm
@@ -39,7 +46,8 @@ class PreNormBlock:
         """What this block is, as plain data, for kernels that can make all of its launches in one call: its kind
         (the order in which the parts run is this file's affair: the docstring above) and what each part says it is
         (its own ``plain_form``; None for a part that has none, and such a block goes part by part)."""
-        if type(self).forward is not PreNormBlock.forward or self.residual_scale is not None or self.feed_forward is None:
+        if (type(self).forward is not PreNormBlock.forward or self.residual_scale is not None or self.feed_forward is None
+                or self.token_input is not None):
             return None
         form = lambda part: getattr(part, "plain_form", lambda: None)()
         return {"kind": "prenorm", "mixer_norm": form(self.mixer_norm), "mixer": form(self.mixer),
@@ -54,11 +62,14 @@ class PreNormBlock:
         h = _normed(self.mixer_norm, self.mixer, stream)
         stream.delta = self.mixer.forward(h, ctx, cache)
         stream.scale = self.residual_scale
-        if self.feed_forward is None:
-            return
-        h = _normed(self.feed_forward_norm, self.feed_forward, stream)
-        stream.delta = self.feed_forward.forward(h, ctx)
-        stream.scale = self.residual_scale
+        if self.feed_forward is not None:
+            h = _normed(self.feed_forward_norm, self.feed_forward, stream)
+            stream.delta = self.feed_forward.forward(h, ctx)
+            stream.scale = self.residual_scale
+        if self.token_input is not None:
+            x = stream.lower(ctx.kernels, self.token_input.env.dtype)
+            stream.delta = self.token_input.forward(x, ctx)
+            stream.post = self.token_input_norm
 
 
 def _normed(norm, consumer, stream):

@@ -49,6 +49,7 @@ class StepContext:
     kv_bound: int = 0  # replayed graphs: an upper bound of kv_len that fixes grids (0: use max_kv_len)
     max_run_kv_len: int = 0  # the longest kv_len among the sequences that bring more than one token (0: not known)
     extra: dict = field(default_factory=dict)  # name -> int32 [n_tokens]: what the step's entries brought beside tokens
+    shared: dict = field(default_factory=dict)  # name -> what a layer of this step leaves for later layers of the step
 
 
 @dataclass
@@ -121,6 +122,21 @@ class ResidualStream:
         if isinstance(raw, ScaledSum):
             return [(y, f * own) for y, f in raw.values()]
         return [(self.delta, own)]
+
+    def lower(self, kernels, dtype) -> torch.Tensor:
+        """Adds what is pending into the residual and returns the residual in ``dtype`` (for a sublayer that reads the
+        residual itself, not a norm of it)."""
+        plain = self.scale is None and self.gate is None and self.post is None and not isinstance(
+            self.raw_delta, (BiasedDelta, ScaledSum))
+        if plain and self.raw_delta is not None:     # the sum and its rounding in one kernel
+            out = kernels.add_lowered(self.residual, self.raw_delta, dtype)
+            self.delta = None
+        else:
+            self.settle(kernels)
+            out = self.lowered if self.lowered is not None else (
+                self.residual if dtype == self.residual.dtype else kernels.cast(self.residual, dtype))
+        self.lowered = out
+        return out
 
     def settle(self, kernels) -> torch.Tensor:
         """Adds what is pending into the residual (no norm follows) and returns the residual."""

@@ -15,7 +15,7 @@ import torch
 
 from .context import BuildEnv, LayerCache, ResidualStream, StepContext
 from .plan import ModelPlan, PagedKVNeed, StateNeed, TensorSpec
-from .registry import BLOCKS, EMBEDDINGS, FEED_FORWARDS, GATES, HEADS, MIXERS, NORMS, STREAM_OPS
+from .registry import BLOCKS, EMBEDDINGS, FEED_FORWARDS, GATES, HEADS, MIXERS, NORMS, STREAM_OPS, TOKEN_INPUTS
 
 
 @dataclass
@@ -35,7 +35,8 @@ class CacheLayout:
     run_state: List[Optional[int]] = field(default_factory=list)
 
 
-_REGISTRY_OF_ROLE = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS, "gate": GATES}
+_REGISTRY_OF_ROLE = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS, "gate": GATES,
+                     "token_input": TOKEN_INPUTS}
 
 
 class _Layer:

@@ -106,6 +106,46 @@ class RMSNorm:
         return out
 
 
+@register_norm("layernorm")
+class LayerNorm:
+    """``y = (x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * w + b``: both statistics, the normalisation, weight and
+    bias in float32 with one rounding.
+
+    params: size, eps.
+
+    ``forward`` first adds what is pending into the float32 residual, in the same kernel; a pending result that passes
+    an RMS norm on its way (``stream.post``) is normed and added there too.
+    """
+
+    def __init__(self, params, env):
+        self.size = int(params["size"])
+        self.eps = float(params["eps"])
+        self.env = env
+        self.weight = self.bias = None
+
+    def weight_specs(self):
+        return {"weight": TensorSpec((self.size,), "vector"), "bias": TensorSpec((self.size,), "vector")}
+
+    def bind(self, tensors):
+        self.weight, self.bias = tensors["weight"].contiguous(), tensors["bias"].contiguous()
+
+    def forward(self, stream, rows=None, scaled_ok=False):
+        """Adds what is pending into ``stream.residual`` and returns the normed rows; with ``rows`` (int32 indices)
+        only those rows are computed and the residual is left as it was."""
+        k = self.env.kernels
+        post = stream.post
+        if (stream.gate is not None or stream.scale is not None or isinstance(stream.raw_delta, (BiasedDelta, ScaledSum))
+                or (post is not None and not isinstance(post, RMSNorm))):
+            stream.settle(k)
+            post = None
+        delta = stream.delta
+        out = k.add_layernorm(stream.residual, delta, (post.weight, post.eps) if post is not None and delta is not None else None,
+                              self.weight, self.bias, self.eps, self.env.dtype, rows)
+        if rows is None:
+            stream.delta = None
+        return out
+
+
 @register_norm("dyt")
 class DynamicTanh:
     """A norm without a statistic: ``y = tanh(a * x) * w + b`` with a learned scalar ``a``, elementwise, in float32

@@ -29,10 +29,10 @@ class PartSpec:
     kind: str
     params: Dict[str, Any] = field(default_factory=dict)
     weights: Dict[str, str] = field(default_factory=dict)
-    role: str = ""     # in a layer: which registry ``kind`` is looked up in ("mixer", "feed_forward", "norm", "gate")
+    role: str = ""     # in a layer: which registry ``kind`` is looked up in (one of ``ROLES``)
 
 
-ROLES = ("mixer", "feed_forward", "norm", "gate")
+ROLES = ("mixer", "feed_forward", "norm", "gate", "token_input")
 
 
 @dataclass
@@ -127,7 +127,8 @@ class TensorSpec:
 @dataclass(frozen=True)
 class PagedKVNeed:
     """Keys and values in pages: all keys (``window`` and ``chunk`` None), the last ``window``, or those of the
-    current block of ``chunk`` absolute positions (a query at ``p`` sees nothing below ``p - p % chunk``).
+    current block of ``chunk`` absolute positions (a query at ``p`` sees nothing below ``p - p % chunk``).  With
+    ``keep_first`` the sequence's first positions stay visible to every query whatever the window.
 
     A page holds, per key/value head, ``page_size`` key rows of ``head_dim`` elements and as many value rows of
     ``value_head_dim`` elements (None: the same width).  The cache manager only stores them; what a row means is
@@ -139,9 +140,11 @@ class PagedKVNeed:
     window: Optional[int] = None
     value_head_dim: Optional[int] = None
     chunk: Optional[int] = None
+    keep_first: int = 0
 
     def first_visible(self, position: int) -> int:
-        """The oldest position that a query at ``position`` (or any later one) can still see."""
+        """The oldest position that a query at ``position`` (or any later one) can still see, the kept first ones
+        aside."""
         lo = 0
         if self.window is not None:
             lo = max(lo, position - self.window + 1)
@@ -151,7 +154,7 @@ class PagedKVNeed:
 
     @property
     def span(self) -> Optional[int]:
-        """Most positions a query sees (None: no bound)."""
+        """Most positions a query sees, the kept first ones aside (None: no bound)."""
         bounds = [b for b in (self.window, self.chunk) if b is not None]
         return min(bounds) if bounds else None
 

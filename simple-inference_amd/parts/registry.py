@@ -1,4 +1,4 @@
-"""Registries of part kinds: mixers, feed-forwards, norms, position encodings, blocks, embeddings, heads.
+"""Registries of part kinds: mixers, feed-forwards, norms, token inputs, position encodings, blocks, embeddings, heads.
 
 A part class is registered under a ``kind``; a ``PartSpec`` names that kind.  A
 test or a user package adds a part with one ``register_*`` call and without a
@@ -22,6 +22,8 @@ Interfaces (``env`` is a ``BuildEnv``; ``ctx`` a ``StepContext``):
   layer under those names), ``forward(stream, ctx, cache) -> None``.
 * gate (of a sublayer's result on its way into the residual stream): ``logits(h) -> Tensor[N, hidden]`` from
   the sublayer's own input, and ``bias`` (float vector or None); the block hands both to the stream.
+* token input: ``forward(x, ctx) -> Tensor[N, hidden]`` from the residual stream in the compute dtype and the step's
+  token ids: what a layer adds for the token itself.
 * stream operation: ``forward(stream, ctx, first)`` changes the residual stream in place before a run of the order;
   ``first`` is the embedding output of the step's tokens (float32).
 * embedding: ``forward(ctx) -> Tensor[N, hidden]`` float32, the residual stream's start.
@@ -71,6 +73,7 @@ EMBEDDINGS = _Registry("embedding")
 HEADS = _Registry("head")
 GATES = _Registry("gate")
 STREAM_OPS = _Registry("stream operation")
+TOKEN_INPUTS = _Registry("token input")
 
 register_mixer: Callable = MIXERS.register
 register_feed_forward: Callable = FEED_FORWARDS.register
@@ -81,3 +84,4 @@ register_embedding: Callable = EMBEDDINGS.register
 register_head: Callable = HEADS.register
 register_gate: Callable = GATES.register
 register_stream_op: Callable = STREAM_OPS.register
+register_token_input: Callable = TOKEN_INPUTS.register

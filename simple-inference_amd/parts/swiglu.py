@@ -3,7 +3,7 @@
 ``y = (silu(h Wg^T) * (h Wu^T)) Wd^T``.  Gate and up are stacked into one
 ``[2I, H]`` matrix at load (reference: ``ops/mlp.py:104``) so one product gives
 both; ``silu(g) * u`` is computed in float32 and rounded once (reference:
-``kernels/swiglu_kernel.py:142-150``).
+``kernels/swiglu_kernel.py:142-150``).  With ``activation: "relu"`` the gate is ``max(g, 0) * u`` instead.
 """
 
 from __future__ import annotations
@@ -16,13 +16,16 @@ from .registry import register_feed_forward
 
 @register_feed_forward("swiglu")
 class SwiGLU:
-    """params: hidden_size, intermediate_size."""
+    """params: hidden_size, intermediate_size, and optionally activation ("silu", the default, or "relu")."""
 
     takes_scaled_rows = True   # the input goes to ``gated_linear`` only
 
     def __init__(self, params, env):
         self.hidden = int(params["hidden_size"])
         self.inter = int(params["intermediate_size"])
+        self.activation = str(params.get("activation", "silu"))
+        if self.activation not in ("silu", "relu"):
+            raise ValueError(f"a gated feed-forward's activation is silu or relu, not {self.activation!r}")
         self.env = env
         self.w_gate_up = None
         self.w_down = None
@@ -44,12 +47,15 @@ class SwiGLU:
     def plain_form(self):
         """What this feed-forward is, as plain data, for kernels that can run a whole block in one call (None for
         a subclass with a forward of its own: it is no longer what this form describes)."""
-        if type(self).forward is not SwiGLU.forward:
+        if type(self).forward is not SwiGLU.forward or self.activation != "silu":
             return None
         return {"kind": "swiglu", "w_gate_up": self.w_gate_up, "w_down": self.w_down, "hidden": self.hidden,
                 "inter": self.inter}
 
     def forward(self, h, ctx):
         k = self.env.kernels
-        a = k.gated_linear(h, self.w_gate_up)   # the activation is fused into the product where a kernel has it
+        if self.activation == "silu":
+            a = k.gated_linear(h, self.w_gate_up)   # the activation is fused into the product where a kernel has it
+        else:
+            a = k.gated_linear(h, self.w_gate_up, activation=(self.activation, None))
         return k.pending_linear(a, self.w_down)   # the norm after it may have it added into the residual

@@ -34,6 +34,32 @@ class TwinKernels:
         residual.add_(yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * weight.float())
         return residual if out_dtype == torch.float32 else residual.to(out_dtype)
 
+    # -- residual add (of a result, or of its rms norm) + layer norm ------------
+    def add_layernorm(self, residual, delta, post, weight, bias, eps, out_dtype, rows=None):
+        x = residual
+        if delta is not None:
+            d = delta.float()
+            if post is not None:
+                d = d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + post[1]) * post[0].float()
+            x = residual + d
+            if rows is None:
+                residual.copy_(x)
+        if rows is not None:
+            x = x[rows.long()]
+        d = x - x.mean(-1, keepdim=True)
+        return (d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * weight.float() + bias.float()).to(out_dtype)
+
+    def add_lowered(self, residual, delta, out_dtype):
+        residual.add_(delta.float())
+        return residual if out_dtype == torch.float32 else residual.to(out_dtype)
+
+    # -- what a layer takes of the token itself ---------------------------------
+    def embedding_gate(self, x, w, activation, table, first_column, dim, token_ids):
+        z = self.activated_linear(x.float(), w.float(), activation)
+        z[:, dim:] = 0
+        z[:, :dim] *= table[token_ids.long(), first_column:first_column + dim].float()
+        return z.to(x.dtype)
+
     # -- residual add + rms norm ---------------------------------------------
     def add_rmsnorm(self, residual, delta, weight, eps, out_dtype, rows=None, gate=None, gate_bias=None,
                     delta_bias=None, terms=None):
@@ -86,6 +112,12 @@ class TwinKernels:
         gated = out.float().view(n, n_heads, -1) * torch.sigmoid(logits.float())[:, :, None]
         out.copy_(gated.view(n, -1).to(out.dtype))
         return out
+
+    def element_gate(self, out, logits, n_heads):
+        """``[n, heads * wide]`` to ``[n, heads * own]``: every head's own elements times their gates."""
+        n, own = out.shape[0], logits.shape[1] // n_heads
+        o = out.float().view(n, n_heads, -1)[:, :, :own].reshape(n, -1)
+        return (o * torch.sigmoid(logits.float())).to(out.dtype)
 
     def side_by_side(self, a, b, dtype):
         return torch.cat([a, b], dim=-1).to(dtype)
@@ -187,29 +219,46 @@ class TwinKernels:
 
     def delta_rule(self, qkv, proj, columns, a_log, dt_bias, norm_weight, n_heads, n_kv_heads, key_dim, value_dim, eps,
                    ctx, state):
-        n, H, G, D, Dv = qkv.shape[0], n_heads, n_kv_heads, key_dim, value_dim
+        H, inner = n_heads, n_heads * value_dim
         cg, cb, ca = columns
-        x, p = qkv.float(), proj.float()
+        p = proj.float()
+        step = torch.nn.functional.softplus(p[:, ca:ca + H] + dt_bias.float(), threshold=1e9)
+        decay = torch.exp(-torch.exp(a_log.float()) * step)[:, :, None]
+        return self._delta(qkv, torch.sigmoid(p[:, cb:cb + H]), decay, torch.nn.functional.silu(p[:, cg:cg + inner]),
+                           norm_weight, n_heads, n_kv_heads, key_dim, value_dim, eps, ctx, state)
+
+    def channel_delta_rule(self, qkv, proj, columns, a2, g2, a_log, dt_bias, norm_weight, n_heads, n_kv_heads, key_dim,
+                           value_dim, eps, ctx, state):
+        H = n_heads
+        cb, ca, cg = columns
+        p = proj.float()
+        z = p[:, ca:ca + a2.shape[1]] @ a2.float().T + dt_bias.float()
+        step = torch.nn.functional.softplus(z, threshold=1e9).view(-1, H, key_dim)
+        decay = torch.exp(-torch.exp(a_log.float())[:, None] * step)
+        gate = torch.sigmoid(p[:, cg:cg + g2.shape[1]] @ g2.float().T)
+        return self._delta(qkv, torch.sigmoid(p[:, cb:cb + H]), decay, gate, norm_weight, n_heads, n_kv_heads, key_dim,
+                           value_dim, eps, ctx, state)
+
+    def _delta(self, qkv, beta, decay, gate, norm_weight, n_heads, n_kv_heads, key_dim, value_dim, eps, ctx, state):
+        n, H, G, D, Dv = qkv.shape[0], n_heads, n_kv_heads, key_dim, value_dim
+        x = qkv.float()
         q = x[:, :G * D].view(n, G, D)
         k = x[:, G * D:2 * G * D].view(n, G, D)
         v = x[:, 2 * G * D:].view(n, H, Dv)
         q = q * torch.rsqrt(q.pow(2).sum(-1, keepdim=True) + 1e-6) * D ** -0.5
         k = k * torch.rsqrt(k.pow(2).sum(-1, keepdim=True) + 1e-6)
         q, k = q.repeat_interleave(H // G, dim=1), k.repeat_interleave(H // G, dim=1)
-        beta = torch.sigmoid(p[:, cb:cb + H])
-        step = torch.nn.functional.softplus(p[:, ca:ca + H] + dt_bias.float(), threshold=1e9)
-        decay = torch.exp(-torch.exp(a_log.float()) * step)
         out = torch.zeros(n, H, Dv)
         cu, slots = ctx.cu_q.tolist(), ctx.state_slots.tolist()
         for s in range(ctx.n_seqs):
             S = state[slots[s], :H * D * Dv].view(H, D, Dv)
             for t in range(cu[s], cu[s + 1]):
-                S.mul_(decay[t][:, None, None])
+                S.mul_(decay[t][:, :, None])
                 u = beta[t][:, None] * (v[t] - torch.einsum("hd,hdv->hv", k[t], S))
                 S.add_(k[t][:, :, None] * u[:, None, :])
                 out[t] = torch.einsum("hd,hdv->hv", q[t], S)
         out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm_weight.float()
-        return (out.view(n, H * Dv) * torch.nn.functional.silu(p[:, cg:cg + H * Dv])).to(qkv.dtype)
+        return (out.view(n, H * Dv) * gate).to(qkv.dtype)
 
     def decay_attention(self, proj, decays, norm_weight, n_heads, key_dim, value_dim, eps, ctx, state):
         n, H, D, Dv = proj.shape[0], n_heads, key_dim, value_dim
@@ -248,20 +297,24 @@ class TwinKernels:
 
     # -- latent attention ------------------------------------------------------------------
     @staticmethod
-    def _rotate_pairs(x, rotary_dim, cos, sin, pos):
-        """``x [n, ..., r]`` float: neighbouring pairs of the first ``rotary_dim`` elements turned by the tables' rows."""
+    def _rotate_pairs(x, rotary_dim, cos, sin, pos, pairing="interleaved"):
+        """``x [n, ..., r]`` float: neighbouring pairs (or the two halves' elements) of the first ``rotary_dim`` elements
+        turned by the tables' rows."""
         if rotary_dim == 0:
             return x
         shape = [x.shape[0]] + [1] * (x.dim() - 2) + [rotary_dim // 2]
         c, s = cos[pos.long()].view(shape), sin[pos.long()].view(shape)
-        a, b = x[..., 0:rotary_dim:2], x[..., 1:rotary_dim:2]
+        half = rotary_dim // 2
+        first, second = ((slice(0, rotary_dim, 2), slice(1, rotary_dim, 2)) if pairing == "interleaved"
+                         else (slice(0, half), slice(half, rotary_dim)))
+        a, b = x[..., first], x[..., second]
         out = x.clone()
-        out[..., 0:rotary_dim:2] = a * c - b * s
-        out[..., 1:rotary_dim:2] = b * c + a * s
+        out[..., first] = a * c - b * s
+        out[..., second] = b * c + a * s
         return out
 
     def latent_prepare(self, proj, q_rank, q_gain, kv_rank, kv_gain, rot_dim, rotary_dim, cos, sin, eps, ctx, cache,
-                       page_dim=None):
+                       page_dim=None, pairing="interleaved"):
         p = proj.float()
         cq = p[:, :q_rank]
         cq = (cq * torch.rsqrt(cq.pow(2).mean(-1, keepdim=True) + eps) * q_gain.float()).to(proj.dtype)
@@ -269,7 +322,7 @@ class TwinKernels:
             a = p[:, q_rank:q_rank + kv_rank]
             c = (a * torch.rsqrt(a.pow(2).mean(-1, keepdim=True) + eps) * kv_gain.float()).to(proj.dtype)
             b = self._rotate_pairs(p[:, q_rank + kv_rank:q_rank + kv_rank + rot_dim], rotary_dim, cos, sin,
-                                   ctx.positions).to(proj.dtype)
+                                   ctx.positions, pairing).to(proj.dtype)
             pos = ctx.positions.long()
             ps = cache.page_size
             page = cache.block_table.long()[ctx.seq_of_token.long(), pos // ps]
@@ -279,7 +332,7 @@ class TwinKernels:
             cache.v_pages[page, 0, :kv_rank, off] = c
         return cq
 
-    def headwise_linear(self, x, w, in_stride, out_stride, tail=0, rotation=None):
+    def headwise_linear(self, x, w, in_stride, out_stride, tail=0, rotation=None, gate=None, pairing="interleaved"):
         n = x.shape[0]
         H, out_dim, in_dim = w.shape
         xs = x.float().view(n, H, in_stride)
@@ -289,8 +342,10 @@ class TwinKernels:
             t = xs[:, :, in_dim:in_dim + tail]
             if rotation is not None:
                 rotary_dim, cos, sin, positions = rotation
-                t = self._rotate_pairs(t, rotary_dim, cos, sin, positions)
+                t = self._rotate_pairs(t, rotary_dim, cos, sin, positions, pairing)
             y[:, :, out_dim:out_dim + tail] = t
+        if gate is not None:
+            y[:, :, :out_dim] *= torch.sigmoid(gate.float()).view(n, H, out_dim)
         return y.view(n, H * out_stride).to(x.dtype)
 
     # -- mixture of experts ---------------------------------------------------------
@@ -325,6 +380,8 @@ class TwinKernels:
         if activation is None:
             return torch.nn.functional.silu(g) * u
         kind, limit = activation
+        if kind == "relu":
+            return torch.relu(g) * u
         assert kind == "clamped"
         g, u = g.clamp(max=limit), u.clamp(-limit, limit)
         return g * torch.sigmoid(1.702 * g) * (u + 1.0)
@@ -386,18 +443,23 @@ class TwinKernels:
         return a.to(x.dtype)
 
     def qkv_to_cache(self, x, w_qkv, n_heads, n_kv_written, head_dim, rotary_dim, cos, sin, ctx, cache,
-                     value_dim=None, bias=None, qk_norm=None, q_temp=None, extra_columns=0, values_are_keys=False):
+                     value_dim=None, bias=None, qk_norm=None, q_temp=None, extra_columns=0, values_are_keys=False,
+                     value_mix=None, give_values=False):
         qkv = self.linear(x, w_qkv)
         self.rope_kv_write(qkv, n_heads, n_kv_written, head_dim, rotary_dim, cos, sin, ctx, cache,
                            value_dim=value_dim, bias=bias, qk_norm=qk_norm, q_temp=q_temp,
-                           values_are_keys=values_are_keys)
+                           values_are_keys=values_are_keys, value_mix=value_mix)
+        out = [qkv]
         if extra_columns:
-            return qkv, qkv[:, qkv.shape[1] - extra_columns:]
-        return qkv
+            out.append(qkv[:, qkv.shape[1] - extra_columns:])
+        if give_values:
+            v0 = (n_heads + n_kv_written) * head_dim
+            out.append(qkv[:, v0:v0 + n_kv_written * (value_dim or head_dim)])
+        return tuple(out) if len(out) > 1 else qkv
 
     # -- rotation + cache write ----------------------------------------------
     def rope_kv_write(self, qkv, n_heads, n_kv_written, head_dim, rotary_dim, cos, sin, ctx, cache,
-                      value_dim=None, bias=None, qk_norm=None, q_temp=None, values_are_keys=False):
+                      value_dim=None, bias=None, qk_norm=None, q_temp=None, values_are_keys=False, value_mix=None):
         N = qkv.shape[0]
         pos = ctx.positions.long()
         value_dim = value_dim or head_dim
@@ -436,6 +498,9 @@ class TwinKernels:
         k = qkv[:, kv0:kv0 + n_kv_written * head_dim].view(N, n_kv_written, head_dim)
         v0 = kv0 if values_are_keys else kv0 + n_kv_written * head_dim      # the keys as projected serve as values
         v = qkv[:, v0:v0 + n_kv_written * value_dim].view(N, n_kv_written, value_dim)
+        if value_mix is not None:
+            given, m = value_mix
+            v = ((1 - m) * v.float() + m * given.float().view(N, n_kv_written, value_dim)).to(v.dtype)
         k = rotate(normed(k, qk_norm[1] if qk_norm else None))
         ps = cache.page_size
         seq = ctx.seq_of_token.long()
@@ -446,7 +511,7 @@ class TwinKernels:
 
     # -- attention over the pages --------------------------------------------
     def paged_attention(self, qkv, n_heads, n_kv_heads, head_dim, scale, window, ctx, cache, value_dim=None,
-                        chunk=None, sinks=None):
+                        chunk=None, sinks=None, softcap=None, keep_first=0):
         N = qkv.shape[0]
         value_dim = value_dim or head_dim
         q = qkv[:, :n_heads * head_dim].view(N, n_heads, head_dim).float()
@@ -465,6 +530,8 @@ class TwinKernels:
             if chunk is not None:
                 lo = max(lo, first - first % chunk)
             idx = torch.arange(lo, L, device=qkv.device)
+            if min(keep_first, lo):
+                idx = torch.cat([torch.arange(min(keep_first, lo), device=qkv.device), idx])
             pages = table[s, idx // ps]
             k = cache.k_pages[pages, :, idx % ps, :].float()          # [T, Hkv, D]
             v = cache.v_pages[pages, :, :, idx % ps].float()          # [T, Hkv, D]
@@ -472,11 +539,13 @@ class TwinKernels:
             qpos = torch.arange(first, L, device=qkv.device)
             visible = idx[None, :] <= qpos[:, None]
             if window is not None:
-                visible &= idx[None, :] > qpos[:, None] - window
+                visible &= (idx[None, :] > qpos[:, None] - window) | (idx[None, :] < keep_first)
             if chunk is not None:
                 visible &= idx[None, :] // chunk == qpos[:, None] // chunk
             for h in range(n_heads):
                 sc = (qs[:, h] @ k[:, h // group].T) * scale
+                if softcap is not None:
+                    sc = softcap * torch.tanh(sc / softcap)
                 sc = sc.masked_fill(~visible, float("-inf"))
                 if sinks is not None:    # one more term in the denominator: a column whose value is nothing
                     sc = torch.cat([sc, sinks[h].float().expand(sc.shape[0], 1)], dim=-1)
