@@ -31,6 +31,8 @@ forget-gate recurrence, latent attention), all with grouped experts, beside the 
 layers with routed experts and the Llama model.
 ``--workload tadinex`` does the same for the Tadinex design: a model of delta-rule layers and a model of layers with a
 windowed attention beside a decaying linear attention, both with clamped experts, beside the same two models.
+``--workload lunerax`` does the same for the Lunerax design: a model of each of its three mixers and one of its attention
+with a short window, with dense feed-forwards, beside the Tadinex delta rule, the Famepel latent attention and the Llama model.
 
 The engine runs on one GPU; asked for more it says so and exits with 2.
 """
@@ -83,11 +85,12 @@ def parse_args(argv=None):
     ap.add_argument("--temperature", type=float, default=0.0, help="sampling of the decode measurement (0: greedy)")
     ap.add_argument("--top-k", type=int, default=0)
     ap.add_argument("--top-p", type=float, default=1.0)
-    ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "shared-prefix", "feduzen", "mogisun", "famepel", "tadinex"])
+    ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "shared-prefix", "feduzen", "mogisun", "famepel", "tadinex", "lunerax"])
     ap.add_argument("--shapes", default="1b,3b,8b", help="--workload feduzen: which layer sizes, comma separated")
-    ap.add_argument("--models", default=None, help="--workload feduzen, mogisun, famepel or tadinex: which of the models to run "
+    ap.add_argument("--models", default=None, help="--workload feduzen, mogisun, famepel, tadinex or lunerax: which of the models to run "
                     "(feduzen,llama; mogisun-attention,mogisun-linear,llama; famepel-ssm,famepel-hgrn,famepel-latent,"
-                    "mogisun-linear,llama; tadinex-delta,tadinex-parallel,mogisun-linear,llama)")
+                    "mogisun-linear,llama; tadinex-delta,tadinex-parallel,mogisun-linear,llama; "
+                    "lunerax-delta,lunerax-latent,lunerax-attention,lunerax-window,tadinex-delta,famepel-latent,llama)")
     ap.add_argument("--max-running", type=int, default=64, help="request slots of the stream workloads")
     return ap.parse_args(argv)
 
@@ -590,6 +593,69 @@ def tadinex_workload(args):
     return 0
 
 
+def lunerax_config_like(llama_cfg, layers, kind):
+    """A Lunerax config.json with the width, head count, head width and feed-forward size of a Llama one; every layer has
+    the same mixer, a dense gated feed-forward of that size (relu for silu: the same work) and a token input of 256.
+    ``delta``: as many value heads of the head width, the Llama model's number of key/value heads as query/key heads, a
+    convolution of four taps, low-rank pairs of the head width.  ``latent``: as many heads, a latent of 192 and a shared
+    rotated key part of 64, queries through a latent of half the width.  ``attention``: the Llama model's attention heads,
+    capped scores, mixed values.  The windows are wider than the measured context, so that the attention does the other
+    models' work; ``window``: the same attention with a window of 512 and four kept tokens."""
+    dim, heads, width = llama_cfg["head_dim"], llama_cfg["num_attention_heads"], llama_cfg["hidden_size"]
+    kv = llama_cfg["num_key_value_heads"]
+    if kind == "delta":
+        mixer = {"type": "channel_delta", "mixer": {"conv": 4, "dim": dim, "heads": heads, "kv_heads": kv, "vdim": dim,
+                                                    "decay_rank": dim, "gate_rank": dim}}
+    elif kind == "latent":
+        mixer = {"type": "latent_attention",
+                 "mixer": {"dim": dim, "heads": heads, "kv_rank": 192, "q_rank": width // 2, "rot_dim": 64, "vdim": dim,
+                           "scale": (dim + 64) ** -0.5, "mask": {"size": 1 << 20},
+                           "rot": {"base": llama_cfg["rope_theta"], "dims": 64}}}
+    else:
+        mixer = {"type": "attention",
+                 "mixer": {"dim": dim, "heads": heads, "kv_heads": kv, "vdim": dim, "scale": dim ** -0.5, "softcap": 30.0,
+                           "v_mix": True, "mask": {"keep_first": 4, "size": 512 if kind == "window" else 1 << 20}}}
+    return {"architecture": "Lunerax", "vocab": llama_cfg["vocab_size"], "width": width,
+            "norm": {"eps": llama_cfg["rms_norm_eps"]}, "embedding": {"scale": 1.0}, "token_side": {"dim": 256},
+            "logit_softcap": 30.0,
+            "layers": [json.loads(json.dumps(dict(mixer, mlp={"kind": "dense", "ff": llama_cfg["intermediate_size"]})))
+                       for _ in range(layers)]}
+
+
+def lunerax_workload(args):
+    """Decode and prefill of the Lunerax design (each of its three mixers alone, and the attention with a short window)
+    beside the closest models' layers at equal sizes: the Tadinex delta rule, the Famepel latent attention (both with
+    routed experts) and the Llama model."""
+    layers = args.layers or 8
+    dt_name = "bf16" if args.dtype == "bfloat16" else "fp32"
+    out = measure_beside(args, lambda llama, n: (("lunerax-delta", lunerax_config_like(llama, n, "delta")),
+                                                 ("lunerax-latent", lunerax_config_like(llama, n, "latent")),
+                                                 ("lunerax-attention", lunerax_config_like(llama, n, "attention")),
+                                                 ("lunerax-window", lunerax_config_like(llama, n, "window")),
+                                                 ("tadinex-delta", tadinex_config_like(llama, n, "delta")),
+                                                 ("famepel-latent", famepel_config_like(llama, n, "latent")),
+                                                 ("llama", llama)),
+                         (args.models or "lunerax-delta,lunerax-latent,lunerax-attention,lunerax-window,tadinex-delta,"
+                                         "famepel-latent,llama").split(","))
+    line = {"metric": "Lunerax beside Tadinex, Famepel and Llama at equal layer sizes: decode tok/s (batch 8, 1) and prefill tok/s",
+            "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "dtype": dt_name,
+            "data": "synthetic (seeded random weights and uniform-random token ids)",
+            "config": {"layers": layers, "context": args.context, "prefill_tokens": args.prefill_tokens,
+                       "shapes": FEDUZEN_SHAPES,
+                       "lunerax-*": "layer norms, dense gated feed-forwards, token inputs of 256, capped logits",
+                       "lunerax-delta": "delta rule with a decay per key channel, 4 taps, low-rank pairs of the head width",
+                       "lunerax-latent": "latent 192 + rotated 64 cached, window beyond the context, gate per element",
+                       "lunerax-attention": "the Llama model's heads without rotation, capped scores, window beyond the "
+                                            "context, 4 kept tokens, mixed values, gate per element",
+                       "lunerax-window": "the same with a window of 512",
+                       "tadinex-delta": "gated delta rule, 8 clamped experts of ff/4 and 2 identity experts, 2 a token, a "
+                                        "shared one of ff/2",
+                       "famepel-latent": "latent 192 + rotated 64 cached, 8 experts of ff/2 in 4 groups, 2 a token"},
+            "shapes": out}
+    print(json.dumps(line), flush=True)
+    return 0
+
+
 def further_points(args, pts, config, layer_w, head_w, el):
     """What the headline leaves out, at sizes a server meets: the same model with contexts of 8,192 and 32,768 tokens
     and a prompt of 8,192 (an engine of its own with a context limit of 33,792), and the two request streams of the
@@ -664,6 +730,8 @@ def main(argv=None):
         return famepel_workload(args)
     if args.workload == "tadinex":
         return tadinex_workload(args)
+    if args.workload == "lunerax":
+        return lunerax_workload(args)
     if args.workload != "decode":
         return stream_workload(args)
     points = [int(p) for p in args.points.split(",") if p]

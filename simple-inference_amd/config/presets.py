@@ -63,6 +63,15 @@ def _mogisun_layer(kind, moe):
     return {"type": kind, "mixer": mixer, "mlp": mlp}
 
 
+def _lunerax_layer(kind):
+    mixer = {"channel_delta": {"conv": 4, "dim": 64, "heads": 8, "kv_heads": 4, "vdim": 64, "decay_rank": 64, "gate_rank": 64},
+             "latent_attention": {"dim": 64, "heads": 8, "kv_rank": 96, "q_rank": 192, "rot_dim": 32, "scale": 0.1, "vdim": 64,
+                                  "rot": {"base": 100000.0, "dims": 32}, "mask": {"size": 256}},
+             "attention": {"dim": 64, "heads": 8, "kv_heads": 2, "vdim": 64, "scale": 0.125, "softcap": 20.0, "v_mix": True,
+                           "mask": {"keep_first": 8, "size": 128}}}[kind]
+    return {"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": 1536}}
+
+
 PRESETS = {
     "llama-3.2-3b": {
         "architectures": ["LlamaForCausalLM"], "model_type": "llama",
@@ -123,6 +132,13 @@ PRESETS = {
         "layers": [_tadinex_layer("parallel", {"kind": "dense", "ff": 1536}), _tadinex_layer("delta", _TADINEX_EXPERTS),
                    _tadinex_layer("delta", _TADINEX_EXPERTS), _tadinex_layer("delta", _TADINEX_EXPERTS),
                    _tadinex_layer("parallel", _TADINEX_EXPERTS), _tadinex_layer("delta", _TADINEX_EXPERTS)],
+    },
+    # a small model of the Lunerax design: two delta-rule layers after every layer of attention, of either kind in turn
+    "lunerax-small": {
+        "architecture": "Lunerax", "vocab": 4096, "width": 512, "norm": {"eps": 1e-6}, "embedding": {"scale": 8.0},
+        "token_side": {"dim": 64}, "logit_softcap": 25.0,
+        "layers": [_lunerax_layer(kind) for kind in ("attention", "channel_delta", "channel_delta", "latent_attention",
+                                                     "channel_delta", "channel_delta", "attention")],
     },
     "tiny-a": {
         "architectures": ["LlamaForCausalLM"], "model_type": "llama",

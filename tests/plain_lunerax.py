@@ -45,7 +45,7 @@ def gelu_tanh(z):
 
 
 def soft_cap(z, cap):
-    return cap * torch.tanh(z / cap)
+    return z if cap is None else cap * torch.tanh(z / cap)
 
 
 # ---------------------------------------------------------------------------------------------------------
@@ -110,10 +110,13 @@ def rotate_half(x, rot):
     return torch.cat([u * c - w * s, w * c + u * s, x[..., dims:]], -1)
 
 
-def visible(n, size, keep_first=0):
-    """``[query, key]``: the last ``size`` positions, the query's own included, and the sequence's first ones."""
+def visible(n, mask):
+    """``[query, key]``: the last ``size`` positions, the query's own included, and the sequence's first ones; all of the
+    past without a mask."""
     i, j = torch.arange(n)[:, None], torch.arange(n)[None, :]
-    return (j <= i) & ((i - j < size) | (j < keep_first))
+    if not mask:
+        return j <= i
+    return (j <= i) & ((i - j < mask["size"]) | (j < mask.get("keep_first", 0)))
 
 
 def weights_over(scores, seen):
@@ -131,7 +134,7 @@ def latent_attention(h, T, p, mx, eps):
     qr = rotate_half(q[..., D:], mx["rot"])
     k = lin(c, T, p + ".uk").reshape(n, H, D)
     v = lin(c, T, p + ".uv").reshape(n, H, Dv)
-    seen = visible(n, mx["mask"]["size"])
+    seen = visible(n, mx.get("mask"))
     out = torch.zeros(n, H, Dv, dtype=F64)
     for hd in range(H):
         out[:, hd] = weights_over((q[:, hd, :D] @ k[:, hd].T + qr[:, hd] @ shared.T) * mx["scale"], seen) @ v[:, hd]
@@ -154,11 +157,11 @@ def capped_attention(h, T, p, mx, first=None):
     q = lin(h, T, p + ".q").reshape(n, H, D)
     k = lin(h, T, p + ".k").reshape(n, G, D)
     v = mixed_values(lin(h, T, p + ".v").reshape(n, G, Dv), T, p, first)
-    seen = visible(n, mx["mask"]["size"], mx["mask"]["keep_first"])
+    seen = visible(n, mx.get("mask"))
     out = torch.zeros(n, H, Dv, dtype=F64)
     for hd in range(H):
         g = hd // (H // G)
-        out[:, hd] = weights_over(soft_cap((q[:, hd] @ k[:, g].T) * mx["scale"], mx["softcap"]), seen) @ v[:, g]
+        out[:, hd] = weights_over(soft_cap((q[:, hd] @ k[:, g].T) * mx["scale"], mx.get("softcap")), seen) @ v[:, g]
     return lin(out.reshape(n, H * Dv) * torch.sigmoid(lin(h, T, p + ".g")), T, p + ".o"), v
 
 
@@ -178,7 +181,7 @@ def layer_streams(cfg, T, tokens):
     eps = cfg["norm"]["eps"]
     ids = torch.as_tensor(tokens, dtype=torch.long)
     x = _t(T, "embed")[ids] * cfg["embedding"]["scale"]
-    side = cfg["token_side"]["dim"]
+    side = cfg["token_side"]["dim"] if cfg.get("token_side") else 0
     after, first = [], None
     for i, layer in enumerate(cfg["layers"]):
         p, mx = f"l{i}", layer["mixer"]
@@ -196,11 +199,12 @@ def layer_streams(cfg, T, tokens):
         x = x + y
         if layer.get("mlp") is not None:
             x = x + gated_relu(layer_norm(x, T, p + ".norm2", eps), T, p + ".mlp")
-        x = x + token_input(x, T, p, _t(T, "side.embed")[ids, i * side: (i + 1) * side], eps)
+        if side:
+            x = x + token_input(x, T, p, _t(T, "side.embed")[ids, i * side: (i + 1) * side], eps)
         after.append(x.clone())
     return torch.stack(after), layer_norm(x, T, "final.norm", eps)
 
 
 def forward(cfg, T, tokens):
     """Logits ``[n, vocab]`` of a whole sequence."""
-    return soft_cap(lin(layer_streams(cfg, T, tokens)[1], T, "head"), cfg["logit_softcap"])
+    return soft_cap(lin(layer_streams(cfg, T, tokens)[1], T, "head"), cfg.get("logit_softcap"))
