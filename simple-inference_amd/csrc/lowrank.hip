@@ -28,11 +28,11 @@ struct LowRankPair {
     int per_head;                   // outputs that share an A_log
 };
 
-__device__ __forceinline__ float low_rank_result(const LowRankPair& p, int which, int o, float z) {
-    if (which == 1) return 1.f / (1.f + expf(-z));
-    z += p.dt_bias[o];
-    const float step = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
-    return expf(-expf(p.a_log[o / p.per_head]) * step);
+__device__ __forceinline__ float gate_of(float z) { return 1.f / (1.f + expf(-z)); }
+
+// rate = exp(A_log), z with its bias
+__device__ __forceinline__ float decay_of(float z, float rate) {
+    return expf(-rate * (fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)))));
 }
 
 #define LR_TOKENS 8
@@ -50,6 +50,7 @@ __global__ __launch_bounds__(256) void low_rank_kernel(const T* __restrict__ pro
     const int o = blockIdx.y * blockDim.x + threadIdx.x;
     if (o >= s.outputs) return;
     const T* w = (const T*)s.w + (size_t)o * s.rank;
+    const float bias = which ? 0.f : p.dt_bias[o], rate = which ? 0.f : expf(p.a_log[o / p.per_head]);
     float z[LR_TOKENS] = {};
     for (int m = 0; m < s.rank; ++m) {
         const float wm = to_float(w[m]);
@@ -58,7 +59,7 @@ __global__ __launch_bounds__(256) void low_rank_kernel(const T* __restrict__ pro
     }
 #pragma unroll
     for (int t = 0; t < LR_TOKENS; ++t)
-        if (t < nt) s.out[(size_t)(n0 + t) * s.outputs + o] = low_rank_result(p, which, o, z[t]);
+        if (t < nt) s.out[(size_t)(n0 + t) * s.outputs + o] = which ? gate_of(z[t]) : decay_of(z[t] + bias, rate);
 }
 
 // A workgroup four waves side by side along the outputs, all on the same MB * 16 tokens.
@@ -77,12 +78,28 @@ __global__ __launch_bounds__(256) void low_rank_mfma_kernel(const bf16_t* __rest
         xp[mb] = proj + (size_t)min(t0 + mb * 16 + r, n_tokens - 1) * row_stride + s.column + g * 8;
 #pragma unroll
     for (int nb = 0; nb < NB; ++nb) wp[nb] = w + (size_t)min(o0 + nb * 16 + r, s.outputs - 1) * s.rank + g * 8;
+    // the four outputs a lane ends up with, o .. o + 3, lie in one head or reach into the next
+    float bias[NB][4], rate[NB][4];
+    if (which == 0) {   // uniform
+#pragma unroll
+        for (int nb = 0; nb < NB; ++nb) {
+            const int o = o0 + nb * 16 + 4 * g, head = min(o, s.outputs - 1) / p.per_head;
+            const float own = expf(p.a_log[head]);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int c = min(o + i, s.outputs - 1);
+                bias[nb][i] = p.dt_bias[c];
+                rate[nb][i] = c < (head + 1) * p.per_head ? own : expf(p.a_log[c / p.per_head]);
+            }
+        }
+    }
     lr_floatx4 acc[NB][MB];
 #pragma unroll
     for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
         for (int mb = 0; mb < MB; ++mb) acc[nb][mb] = lr_floatx4{0.f, 0.f, 0.f, 0.f};
     const lr_bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll 4
     for (int k = 0; k < s.rank; k += 32) {
         const bool live = k + g * 8 < s.rank;     // the rank is a multiple of 8: a lane's piece is inside or outside
         lr_bf16x8 a[NB], b[MB];
@@ -105,9 +122,17 @@ __global__ __launch_bounds__(256) void low_rank_mfma_kernel(const bf16_t* __rest
         for (int nb = 0; nb < NB; ++nb) {
             const int o = o0 + nb * 16 + 4 * g;
             float* dst = s.out + (size_t)n * s.outputs + o;
+            float v[4];
 #pragma unroll
             for (int i = 0; i < 4; ++i)
-                if (o + i < s.outputs) dst[i] = low_rank_result(p, which, o + i, acc[nb][mb][i]);
+                v[i] = which ? gate_of(acc[nb][mb][i]) : decay_of(acc[nb][mb][i] + bias[nb][i], rate[nb][i]);
+            if (s.outputs % 4 == 0) {   // uniform; the row's pieces are whole and aligned
+                if (o < s.outputs) *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
+                continue;
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (o + i < s.outputs) dst[i] = v[i];
         }
     }
 }
@@ -129,7 +154,8 @@ SIA_EXPORT int sia_low_rank_pair(const void* proj, int row_stride, int a_col, in
     p.per_head = per_head;
     const int most = channels > gates ? channels : gates;
     const bool aligned = rank_a % 8 == 0 && rank_g % 8 == 0 && a_col % 8 == 0 && g_col % 8 == 0 && row_stride % 8 == 0 &&
-                         ((uintptr_t)proj % 16) == 0 && ((uintptr_t)a2 % 16) == 0 && ((uintptr_t)g2 % 16) == 0;
+                         ((uintptr_t)proj % 16) == 0 && ((uintptr_t)a2 % 16) == 0 && ((uintptr_t)g2 % 16) == 0 &&
+                         ((uintptr_t)decay % 16) == 0 && ((uintptr_t)gate % 16) == 0;
     if (dtype == SIA_BF16 && aligned) {
         const bool few = n_tokens <= 64;
         const int tokens = few ? 16 : 32, outs = few ? 64 : 128;

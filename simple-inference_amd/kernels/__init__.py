@@ -941,8 +941,10 @@ class HipKernels:
         stride = self._state_rows(state, ctx, n_heads * key_dim * value_dim)
         out = torch.empty((n, inner), dtype=qkv.dtype, device=qkv.device)
         raw = self.core.sia_delta_rule_workspace(n, n_heads, value_dim)
-        workspace = self._float_workspace(ctx, raw + n * (channels + inner), qkv.device)
-        decays, gates = workspace[raw:], workspace[raw + n * channels:]
+        up4 = lambda floats: -(-floats // 4) * 4          # the decays and the gates start at 16-byte boundaries
+        at_gates = up4(raw) + up4(n * channels)
+        workspace = self._float_workspace(ctx, at_gates + n * inner, qkv.device)
+        decays, gates = workspace[up4(raw):], workspace[at_gates:]
         self._check(self.core.sia_low_rank_pair(
             _ptr(proj), proj.shape[1], a, a2.shape[1], _ptr(a2), _ptr(a_log), _ptr(dt_bias), channels, key_dim,
             _ptr(decays), g, g2.shape[1], _ptr(g2), inner, _ptr(gates), n, _DT[qkv.dtype], self._stream()), "low_rank_pair")

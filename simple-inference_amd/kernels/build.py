@@ -19,6 +19,7 @@ import subprocess
 import sys
 import tempfile
 import time
+from concurrent.futures import ThreadPoolExecutor
 from pathlib import Path
 from typing import Dict, Iterable, Optional, Sequence
 
@@ -120,6 +121,15 @@ def library_path(name: str, sources: Sequence[str], defines: Sequence[str] = ())
     return _writable_dir() / file
 
 
+def _jobs() -> int:
+    """Compilers to run at a time."""
+    try:
+        most = int(os.environ.get("MAX_JOBS", "") or 8)
+    except ValueError:
+        most = 8
+    return max(1, min(most, os.cpu_count() or 1, 16))
+
+
 def compile_library(name: str, sources: Sequence[str], defines: Sequence[str] = (), force: bool = False,
                     verbose: bool = True) -> Path:
     """Builds (if missing or ``force``) and returns the path of the shared library."""
@@ -129,8 +139,7 @@ def compile_library(name: str, sources: Sequence[str], defines: Sequence[str] = 
     hipcc = find_hipcc()
     out.parent.mkdir(parents=True, exist_ok=True)
     tmp = out.with_suffix(f".tmp{os.getpid()}.so")
-    cmd = [hipcc, *HIPCC_FLAGS, *_source_flags(sources), *[f"-D{d}" for d in defines], f"-I{CSRC}",
-           *[str(CSRC / s) for s in sources], "-o", str(tmp), *LINK_FLAGS.get(name, ())]
+    flags = [*HIPCC_FLAGS, *_source_flags(sources), *[f"-D{d}" for d in defines], f"-I{CSRC}"]
     if verbose:
         print(f"[simple-inference_amd] compiling {name} ({', '.join(sources)}) for {ARCH} ...",
               file=sys.stderr, flush=True)
@@ -138,13 +147,28 @@ def compile_library(name: str, sources: Sequence[str], defines: Sequence[str] = 
     env = dict(os.environ)
     if not env.get("HOME") or not os.access(env.get("HOME", "/nonexistent"), os.W_OK):
         env["HOME"] = tempfile.gettempdir()  # the compiler driver wants a writable home for its temporaries
-    proc = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True, env=env)
-    if proc.returncode != 0:
-        try:
-            tmp.unlink()
-        except OSError:
-            pass
-        raise KernelBuildError(f"hipcc failed for {name}:\n{' '.join(cmd)}\n{proc.stdout}")
+    run = lambda cmd: (cmd, subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True, env=env))
+    objects = [out.with_suffix(f".tmp{os.getpid()}.{i}.o") for i in range(len(sources))] if len(sources) > 1 else []
+    try:
+        inputs = [str(CSRC / src) for src in sources]
+        if objects:     # no source needs another's device code: each is compiled by itself, several at a time
+            compile_only = [f for f in flags if f != "-shared"]
+            with ThreadPoolExecutor(min(len(sources), _jobs())) as pool:
+                done = list(pool.map(lambda pair: run([hipcc, *compile_only, "-c", pair[0], "-o", str(pair[1])]),
+                                     zip(inputs, objects)))
+            inputs = [str(o) for o in objects]
+        else:
+            done = []
+        if all(proc.returncode == 0 for _, proc in done):
+            done.append(run([hipcc, *flags, *inputs, "-o", str(tmp), *LINK_FLAGS.get(name, ())]))
+        failed = [(cmd, proc) for cmd, proc in done if proc.returncode != 0]
+        if failed:
+            tmp.unlink(missing_ok=True)
+            cmd, proc = failed[0]
+            raise KernelBuildError(f"hipcc failed for {name}:\n{' '.join(cmd)}\n{proc.stdout}")
+    finally:
+        for o in objects:
+            o.unlink(missing_ok=True)
     os.replace(tmp, out)
     pattern = re.compile(rf"libsia_{re.escape(name)}_[0-9a-f]{{12}}\.so$")
     for stale in out.parent.iterdir():
