@@ -284,7 +284,7 @@ def plain_scores(q, keys, values, qpos, scale, cap, mask):
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("heads,kv,dim,window,keep,cap,page", [
     (3, 3, 32, 24, 3, 2.0, 8), (4, 2, 16, 20, 20, None, 16), (8, 2, 64, 37, 70, 1.5, 16), (6, 1, 32, None, 0, 3.0, 8),
-    (4, 4, 128, 64, 1, 4.0, 16), (2, 1, 144, 33, 9, 2.0, 32), (2, 2, 256, 41, 65, 2.5, 16), (4, 2, 96, 72, 4, 10.0, 64),
+    (4, 4, 128, 64, 1, 4.0, 16), (2, 1, 144, 33, 9, 2.0, 32), (2, 2, 256, 41, 65, 2.5, 16), (6, 3, 80, 61, 6, 10.0, 64),
     (20, 1, 32, 50, 7, 2.0, 16), (2, 2, 24, 18, 6, 2.0, 4)])
 def test_capped_scores_and_kept_first_positions_in_prompts_and_decoding(backend, heads, kv, dim, window, keep, cap, page):
     """A whole prompt, portions that begin inside and behind the kept positions, single tokens around the window's and
