@@ -243,7 +243,8 @@ class CacheManager:
         return max((len(g.tables[r]) for g in self.groups for r in reqs), default=0)
 
     def layer_caches(self, block_tables: List[torch.Tensor]) -> List[LayerCache]:
-        """One ``LayerCache`` per run of the order, over this step's device block tables."""
+        """One ``LayerCache`` per run of the order, over this step's device block tables; behind them one with the
+        embedding's state, if it has one."""
         caches = []
         for e, kv in enumerate(self.layout.run_kv):
             c = LayerCache()
@@ -257,6 +258,8 @@ class CacheManager:
             if si is not None:
                 c.state = self.slots.tensors[si]
             caches.append(c)
+        if self.layout.embedding_state is not None:
+            caches.append(LayerCache(state=self.slots.tensors[self.layout.embedding_state]))
         return caches
 
     # -- checks ------------------------------------------------------------

@@ -4,8 +4,8 @@ from .registry import (
     register_block, register_embedding, register_feed_forward, register_gate, register_head, register_mixer,
     register_norm, register_position_encoding, register_stream_op, register_token_input,
 )
-from .context import BiasedDelta, BuildEnv, LayerCache, ResidualStream, ScaledSum, StepContext
-from . import norm, rope, attention, swiglu, dense, block, embedding, gate, stream_ops, gla, moe, ssm, hgrn, latent_attention, delta, decay_attention, parallel, token_input  # noqa: F401  (registers the built-in kinds)
+from .context import BiasedDelta, BuildEnv, LayerCache, NormedSum, ResidualStream, ScaledSum, StepContext
+from . import norm, rope, attention, swiglu, dense, block, embedding, gate, stream_ops, gla, moe, ssm, hgrn, latent_attention, delta, decay_attention, parallel, token_input, rglru, wkv  # noqa: F401  (registers the built-in kinds)
 from .model import DecoderModel
 
 __all__ = [
@@ -14,5 +14,5 @@ __all__ = [
     "TOKEN_INPUTS",
     "register_block", "register_embedding", "register_feed_forward", "register_gate", "register_head", "register_mixer",
     "register_norm", "register_position_encoding", "register_stream_op", "register_token_input",
-    "BiasedDelta", "BuildEnv", "LayerCache", "ResidualStream", "ScaledSum", "StepContext", "DecoderModel",
+    "BiasedDelta", "BuildEnv", "LayerCache", "NormedSum", "ResidualStream", "ScaledSum", "StepContext", "DecoderModel",
 ]

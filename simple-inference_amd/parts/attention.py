@@ -41,6 +41,12 @@ Further forms, each switched on by a parameter of its own and free to combine:
   layer that gives has one too and does not use it).
 * ``value_from_key``: there is no value projection: a position's values are its keys as projected (with their bias,
   before norm and rotation); the stacked matrix is ``[(Hq + Hkv) D, H]``.
+* ``conv_taps``: q, k and v pass a short causal convolution per channel right after the projection and its bias (before
+  norm and rotation): ``c_t = sum_j w[:, j] u_(t - taps + 1 + j)``, zeros before the sequence.  The mixer then has a state
+  beside its pages: the last inputs as a ring of float32 rows, that of position ``p`` in row ``p mod taps``.
+* ``qk_norm`` with ``"over": "row"``: one RMS norm over all of a token's q elements (and one over all its k elements) at
+  once, with gains of that size, instead of one per head.
+* a rotary position encoding whose ``pairing`` is ``"interleaved"`` turns elements ``2i`` and ``2i + 1`` together.
 * ``o_bias``: the output projection has a bias; it is handed on with the result (``BiasedDelta``) so that the sum
   into the residual can take it in passing.
 """
@@ -50,7 +56,7 @@ from __future__ import annotations
 import torch
 
 from .context import BiasedDelta
-from .plan import PagedKVNeed, TensorSpec
+from .plan import PagedKVNeed, StateNeed, TensorSpec
 from .registry import POSITION_ENCODINGS, register_mixer
 
 
@@ -68,7 +74,7 @@ class Attention:
     """params: hidden_size, num_heads, num_kv_heads, head_dim, position
     (``{"kind", "params"}``), and optionally window, scale, kv_from_layer, value_head_dim, bias, qk_norm, chunk,
     sink, q_temp, out_gate (True or "element"), o_bias, value_from_key, softcap, keep_first, value_mix ("gives" or
-    "takes")."""
+    "takes"), conv_taps."""
 
     def __init__(self, params, env):
         self.hidden = int(params["hidden_size"])
@@ -90,6 +96,12 @@ class Attention:
         qk_norm = params.get("qk_norm")
         self.qk_norm_eps = float(qk_norm["eps"]) if qk_norm else None
         self.qk_norm_gain = bool(qk_norm.get("gain", True)) if qk_norm else False
+        self.qk_norm_over = str(qk_norm.get("over", "head")) if qk_norm else None
+        if self.qk_norm_over not in (None, "head", "row"):
+            raise ValueError(f"a q/k norm is over a head or over the row, not {self.qk_norm_over!r}")
+        self.conv_taps = int(params["conv_taps"]) if params.get("conv_taps") is not None else None
+        if self.conv_taps is not None and self.conv_taps < 1:
+            raise ValueError(f"a convolution has a tap or more, got {self.conv_taps}")
         q_temp = params.get("q_temp")
         self.q_temp = (float(q_temp["coef"]), int(q_temp["every"])) if q_temp else None
         if self.q_temp is not None and self.q_temp[1] <= 0:
@@ -126,6 +138,11 @@ class Attention:
         self.position = _shared_position_encoding(params.get("position", {"kind": "none", "params": {}}), env)
         if self.position.rotary_dim > self.head_dim:
             raise ValueError(f"rotary_dim {self.position.rotary_dim} exceeds head_dim {self.head_dim}")
+        self.pairing = getattr(self.position, "pairing", "half")
+        if self.row_form and (self.kv_from_layer is not None or self.q_temp is not None or self.out_gate or self.value_mix
+                              or self.value_from_key or (self.qk_norm_eps is not None and not self.qk_norm_gain)):
+            raise ValueError("convolved, row-normed or neighbour-rotated heads do not combine with a query temperature, an "
+                             "output gate, mixed values, values that are keys, or another layer's pages")
         check = getattr(env.kernels, "check_attention_geometry", None)
         if check is not None:     # sizes the kernels refuse are refused here, when the model is built
             check(self.num_heads, self.num_kv_heads, max(self.head_dim, self.value_dim))
@@ -137,7 +154,24 @@ class Attention:
         self.w_o = None
         self.b_qkv = self.q_gain = self.k_gain = self.sinks = self.b_o = None
         self.gate_columns = 0
-        self.mix = None
+        self.mix = self.conv_w = None
+        self.row_columns = ()
+
+    @property
+    def row_form(self) -> bool:
+        """Whether what lies between projection and attention needs a token's whole row at once (the kernels'
+        ``row_prepare``)."""
+        return (self.conv_taps is not None or self.qk_norm_over == "row"
+                or (self.position.rotary_dim > 0 and self.pairing == "interleaved"))
+
+    @property
+    def takes_projection(self) -> bool:
+        """Whether ``forward_projected`` may be handed the rows of ``w_in``'s product."""
+        return self.row_form
+
+    @property
+    def w_in(self):
+        return self.w_qkv
 
     takes_scaled_rows = True   # the input goes to ``qkv_to_cache`` only
 
@@ -164,7 +198,11 @@ class Attention:
             if not self.value_from_key:
                 specs["v_bias"] = TensorSpec((v,), "vector")
         if self.qk_norm_eps is not None and self.qk_norm_gain:
-            specs.update({"q_norm": TensorSpec((self.head_dim,), "vector"), "k_norm": TensorSpec((self.head_dim,), "vector")})
+            sizes = (q, kv) if self.qk_norm_over == "row" else (self.head_dim, self.head_dim)
+            specs.update({"q_norm": TensorSpec((sizes[0],), "vector"), "k_norm": TensorSpec((sizes[1],), "vector")})
+        if self.conv_taps is not None:
+            specs.update({"q_conv": TensorSpec((q, self.conv_taps), "vector"), "k_conv": TensorSpec((kv, self.conv_taps), "vector"),
+                          "v_conv": TensorSpec((v, self.conv_taps), "vector")})
         if self.sink:
             specs["sink"] = TensorSpec((self.num_heads,), "vector")
         if self.out_gate:
@@ -185,7 +223,16 @@ class Attention:
             stacked += [g, g.new_zeros((self.gate_columns - self.gates, self.hidden))]
         if self.value_mix == "takes":
             self.mix = tensors["value_mix"].reshape(1).float().contiguous()
+        if self.row_form:     # q, k and v each start aligned in a projected row, behind zero rows
+            at, columns, parts = 0, [], []
+            for t in stacked:
+                columns.append(at)
+                parts += [t, t.new_zeros((-t.shape[0] % 8, self.hidden))]
+                at += t.shape[0] + (-t.shape[0] % 8)
+            self.row_columns, stacked = tuple(columns), parts
         self.w_qkv = torch.cat(stacked, dim=0).contiguous()
+        if self.conv_taps is not None:
+            self.conv_w = torch.cat([tensors[n] for n in ("q_conv", "k_conv", "v_conv")], dim=0).float().contiguous()
         self.w_o = tensors["o"].contiguous()
         if self.page_dim is not None and not self.element_gate:
             # the attention's rows come with page_dim elements a head: zero columns for the rest (the elements' gate
@@ -222,7 +269,7 @@ class Attention:
         """Whether any of the further forms is switched on (the kernels then get them as keyword arguments)."""
         return (self.bias or self.qk_norm_eps is not None or self.sink or self.chunk is not None
                 or self.value_dim != self.head_dim or self.q_temp is not None or self.out_gate or self.value_from_key
-                or self.softcap is not None or self.keep_first > 0 or self.value_mix is not None)
+                or self.softcap is not None or self.keep_first > 0 or self.value_mix is not None or self.row_form)
 
     def cache_need(self):
         if self.page_dim is not None:
@@ -231,10 +278,37 @@ class Attention:
                            self.value_dim if self.value_dim != self.head_dim else None, self.chunk, self.keep_first)
 
     def state_need(self):
-        return None
+        if self.conv_taps is None or self.conv_taps == 1:
+            return None
+        channels = (self.num_heads + self.num_kv_heads) * self.head_dim + self.num_kv_heads * self.value_dim
+        return StateNeed((self.conv_taps * channels,), "float32", 0.0)
+
+    def forward_projected(self, proj, ctx, cache):
+        """The mixer from the rows of the stacked projection on (``[q | k | v]`` at ``row_columns``, perhaps columns of a
+        wider matrix)."""
+        k = self.env.kernels
+        cos, sin = self.position.tables()
+        norm = (self.q_gain, self.k_gain, self.qk_norm_eps, self.qk_norm_over) if self.qk_norm_eps is not None else None
+        q = k.row_prepare(proj, self.row_columns, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
+                          self.position.rotary_dim, cos, sin, self.pairing, self.b_qkv, self.conv_w, norm, self.page_dim,
+                          ctx, cache)
+        attend = {}
+        if self.value_dim != self.head_dim and self.page_dim is None:
+            attend["value_dim"] = self.value_dim
+        for name, value in (("chunk", self.chunk), ("sinks", self.sinks), ("softcap", self.softcap)):
+            if value is not None:
+                attend[name] = value
+        if self.keep_first:
+            attend["keep_first"] = self.keep_first
+        out = k.paged_attention(q, self.num_heads, self.num_kv_heads, self.page_dim or self.head_dim, self.scale,
+                                self.window, ctx, cache, **attend)
+        y = k.pending_linear(out, self.w_o)
+        return BiasedDelta(y, self.b_o, k) if self.o_bias else y
 
     def forward(self, h, ctx, cache):
         k = self.env.kernels
+        if self.row_form:
+            return self.forward_projected(k.linear(h, self.w_qkv), ctx, cache)
         cos, sin = self.position.tables()
         project, attend = {}, {}
         if self._options():   # only then: a kernels object that knows none of these forms serves the plain mixer

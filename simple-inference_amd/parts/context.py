@@ -184,6 +184,25 @@ class ScaledSum:
         return self.kernels.scaled_sum(self.values())
 
 
+class NormedSum:
+    """A sublayer's result that is a sum of several, each behind an RMS norm of its own and with a constant factor:
+    ``sum_i factor_i * rms(y_i) * gain_i``.  A norm behind the sublayer that can take the terms as they are reads
+    ``values()``; everybody else gets the tensor from ``compute()``."""
+
+    __slots__ = ("terms", "kernels")
+
+    def __init__(self, terms, kernels):
+        self.terms, self.kernels = list(terms), kernels
+
+    def values(self):
+        """``[(tensor, factor, gain, eps)]``, products that were left pending computed."""
+        self.terms = [(y.compute() if hasattr(y, "compute") else y, *rest) for y, *rest in self.terms]
+        return self.terms
+
+    def compute(self):
+        return self.kernels.normed_sum(self.values())
+
+
 class BiasedDelta:
     """A sublayer's result whose bias is not added yet: ``y + bias``.  A sum that can take the bias in passing reads
     ``value()`` and ``bias``; everybody else gets the tensor from ``compute()``."""

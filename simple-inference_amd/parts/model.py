@@ -25,7 +25,8 @@ class CacheLayout:
     ``kv_groups[g]`` is the need shared by all runs in group ``g`` and
     ``kv_slabs[g]`` the number of runs that write pages of their own there.
     ``run_kv[e]`` is ``(group, slab)`` for run ``e`` of the order (None: no pages).
-    ``states[i]`` is one fixed-size state; ``run_state[e]`` its index (or None).
+    ``states[i]`` is one fixed-size state; ``run_state[e]`` its index (or None).  ``embedding_state`` is the index of the
+    embedding's own state (None: it has none).
     """
 
     kv_groups: List[PagedKVNeed] = field(default_factory=list)
@@ -33,6 +34,7 @@ class CacheLayout:
     run_kv: List[Optional[Tuple[int, int]]] = field(default_factory=list)
     states: List[StateNeed] = field(default_factory=list)
     run_state: List[Optional[int]] = field(default_factory=list)
+    embedding_state: Optional[int] = None
 
 
 _REGISTRY_OF_ROLE = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS, "gate": GATES,
@@ -134,6 +136,10 @@ class DecoderModel:
                 layout.run_state.append(len(layout.states))
                 layout.states.append(sneed)
             latest_run_of_layer[li] = e
+        need = getattr(self.embedding, "state_need", lambda: None)()
+        if need is not None:
+            layout.embedding_state = len(layout.states)
+            layout.states.append(need)
         return layout
 
     def cache_layout(self) -> CacheLayout:
@@ -141,11 +147,14 @@ class DecoderModel:
 
     # -- forward -----------------------------------------------------------
     def forward(self, ctx: StepContext, caches: List[LayerCache]) -> Optional[torch.Tensor]:
-        """Runs the step's tokens; returns float32 logits ``[n_logit_rows, vocab]`` (None if none wanted)."""
-        first = self.embedding.forward(ctx)
+        """Runs the step's tokens; returns float32 logits ``[n_logit_rows, vocab]`` (None if none wanted).  ``caches`` has
+        one entry per run of the order, and one more behind them if the embedding has a state."""
+        stateful = self._layout.embedding_state is not None
+        first = self.embedding.forward(ctx, caches[len(self.order)]) if stateful else self.embedding.forward(ctx)
         # layers add into the residual in place: where a later stream operation wants the embedding output again,
         # the stream starts from a second gather of it
-        stream = ResidualStream(self.embedding.forward(ctx) if self.entries and 0 not in self.entries else first)
+        again = self.entries and 0 not in self.entries
+        stream = ResidualStream((first.clone() if stateful else self.embedding.forward(ctx)) if again else first)
         for e, li in enumerate(self.order):
             if e in self.entries:
                 self.stream_ops[self.entries[e]].forward(stream, ctx, first)

@@ -16,7 +16,8 @@ chooses by ``s + correction`` (``correction: True``: a vector of the checkpoint,
 the chosen by ``s / (sum of the chosen s + 1e-20)``; ``identity_experts: n`` gives the router ``n`` further outputs
 behind the experts' own, experts without tensors that return their input; ``activation: "clamped"`` (with ``limit``,
 and ``shared_limit`` for the shared expert) makes an expert ``W2 (g * sigmoid(1.702 g) * (u + 1))`` with ``g = min(Wg h,
-limit)`` and ``u = clamp(Wu h, -limit, limit)``.
+limit)`` and ``u = clamp(Wu h, -limit, limit)``; ``activation: "gelu"`` makes an expert, and the shared one, ``W2 gelu(Wu h)``
+with the exact gelu and no gate; ``router_bias`` adds a stored vector to the logits, for the choice and the weights.
 
 The experts' matrices are stacked at load (``[E, 2 ff, hidden]`` with the gate rows first, ``[E, hidden, ff]``); the
 shared expert's gate and up rows and its scalar gate are one stacked matrix.  Routing happens on the device: no
@@ -36,7 +37,8 @@ class MixtureOfExperts:
     """params: hidden_size, experts, top, expert_size, and optionally shared_size (a shared expert of that
     intermediate size), shared_gate (default True: the shared expert's output is scaled by a sigmoid), score
     ("softmax", the default, "sigmoid" or "softmax_all"), groups ((count, keep), with sigmoid scores), route_scale,
-    correction, identity_experts, activation ("swiglu", the default, or "clamped"), limit and shared_limit."""
+    correction, identity_experts, activation ("swiglu", the default, "clamped" or "gelu"), limit, shared_limit and
+    router_bias (with softmax scores)."""
 
     def __init__(self, params, env):
         self.hidden = int(params["hidden_size"])
@@ -53,8 +55,12 @@ class MixtureOfExperts:
         if self.identity < 0 or (self.correction and self.score != "softmax_all"):
             raise ValueError("a correction of the choice comes with scores over all router outputs")
         self.activation = str(params.get("activation", "swiglu"))
-        if self.activation not in ("swiglu", "clamped"):
-            raise ValueError(f"activation must be 'swiglu' or 'clamped', got {self.activation!r}")
+        if self.activation not in ("swiglu", "clamped", "gelu"):
+            raise ValueError(f"activation must be 'swiglu', 'clamped' or 'gelu', got {self.activation!r}")
+        self.gated = self.activation != "gelu"
+        self.router_bias = bool(params.get("router_bias", False))
+        if self.router_bias and self.score != "softmax":
+            raise ValueError("a router's bias comes with softmax scores over the chosen")
         self.glu = self.shared_glu = None
         if self.activation == "clamped":
             self.glu = ("clamped", float(params["limit"]))
@@ -79,12 +85,16 @@ class MixtureOfExperts:
         specs = {"router": TensorSpec((self.experts + self.identity, self.hidden), "float_matrix")}
         if self.correction:
             specs["correction"] = TensorSpec((self.experts + self.identity,), "vector")
+        if self.router_bias:
+            specs["router_bias"] = TensorSpec((self.experts + self.identity,), "vector")
         for e in range(self.experts):
-            specs[f"gate{e}"] = TensorSpec((self.inter, self.hidden))
+            if self.gated:
+                specs[f"gate{e}"] = TensorSpec((self.inter, self.hidden))
             specs[f"up{e}"] = TensorSpec((self.inter, self.hidden))
             specs[f"down{e}"] = TensorSpec((self.hidden, self.inter))
         if self.shared_inter:
-            specs["shared_gate"] = TensorSpec((self.shared_inter, self.hidden))
+            if self.gated:
+                specs["shared_gate"] = TensorSpec((self.shared_inter, self.hidden))
             specs["shared_up"] = TensorSpec((self.shared_inter, self.hidden))
             specs["shared_down"] = TensorSpec((self.hidden, self.shared_inter))
             if self.shared_gate:
@@ -95,17 +105,20 @@ class MixtureOfExperts:
         E = range(self.experts)
         self.router = tensors["router"].contiguous()
         self.choice_bias = tensors["correction"].contiguous() if self.correction else None
-        self.w_gate_up = torch.stack([torch.cat([tensors[f"gate{e}"], tensors[f"up{e}"]], dim=0) for e in E]).contiguous()
+        self.logit_bias = tensors["router_bias"].contiguous() if self.router_bias else None
+        both = lambda gate, up: torch.cat([tensors[gate], tensors[up]], dim=0) if self.gated else tensors[up]
+        self.w_gate_up = torch.stack([both(f"gate{e}", f"up{e}") for e in E]).contiguous()
         self.w_down = torch.stack([tensors[f"down{e}"] for e in E]).contiguous()
         if self.shared_inter:
-            self.w_shared_in = torch.cat([tensors["shared_gate"], tensors["shared_up"]], dim=0).contiguous()
+            self.w_shared_in = both("shared_gate", "shared_up").contiguous()
             self.w_shared_down = tensors["shared_down"].contiguous()
             self.w_shared_scale = tensors["shared_scale"].contiguous() if self.shared_gate else None
 
     def forward(self, h, ctx):
         k = self.env.kernels
         if self.score == "softmax":
-            ids, weights = k.moe_route(h, self.router, self.top)
+            ids, weights = k.moe_route(h, self.router, self.top) if self.logit_bias is None else \
+                k.moe_route(h, self.router, self.top, bias=self.logit_bias)
         elif self.score == "softmax_all":
             ids, weights = k.moe_route(h, self.router, self.top, score=self.score, correction=self.choice_bias)
         else:
@@ -113,11 +126,15 @@ class MixtureOfExperts:
                                        scale=self.route_scale)
         shared = scale = None
         if self.shared_inter:
-            inner = k.gated_linear(h, self.w_shared_in) if self.shared_glu is None else \
+            inner = k.activated_linear(h, self.w_shared_in, self.activation) if not self.gated else \
+                k.gated_linear(h, self.w_shared_in) if self.shared_glu is None else \
                 k.gated_linear(h, self.w_shared_in, activation=self.shared_glu)
             shared = k.linear(inner, self.w_shared_down)
             if self.shared_gate:
                 scale = k.linear(h, self.w_shared_scale)
+        if not self.gated:
+            return k.moe_experts(h, self.w_gate_up, self.w_down, ids, weights, shared, scale, activation=self.activation,
+                                 identity=self.identity)
         if self.glu is None and not self.identity:
             return k.moe_experts(h, self.w_gate_up, self.w_down, ids, weights, shared, scale)
         return k.moe_experts(h, self.w_gate_up, self.w_down, ids, weights, shared, scale, activation=self.glu,

@@ -10,7 +10,7 @@ the norm of what the sublayer returned, ``x += y * rsqrt(mean(y^2) + eps) * w``,
 
 from __future__ import annotations
 
-from .context import BiasedDelta, ScaledSum
+from .context import BiasedDelta, NormedSum, ScaledSum
 from .plan import TensorSpec
 from .registry import register_norm
 
@@ -18,22 +18,30 @@ from .registry import register_norm
 @register_norm("rmsnorm")
 class RMSNorm:
     """params: size, eps, and optionally unit_offset (default False): the stored vector is the gain's distance from
-    one, ``y = x * rsqrt(mean(x^2) + eps) * (1 + w)``; the one is added once, in float32, when the vector is bound."""
+    one, ``y = x * rsqrt(mean(x^2) + eps) * (1 + w)``; the one is added once, in float32, when the vector is bound) and
+    scaled (default False: a second stored vector multiplies the result element by element, a layer scale behind the
+    norm; the two vectors are one gain once they are bound)."""
 
     def __init__(self, params, env):
         self.size = int(params["size"])
         self.eps = float(params["eps"])
         self.unit_offset = bool(params.get("unit_offset", False))
+        self.scaled = bool(params.get("scaled", False))
         self.env = env
         self.weight = None
 
     def weight_specs(self):
-        return {"weight": TensorSpec((self.size,), "vector")}
+        specs = {"weight": TensorSpec((self.size,), "vector")}
+        if self.scaled:
+            specs["scale"] = TensorSpec((self.size,), "vector")
+        return specs
 
     def bind(self, tensors):
         self.weight = tensors["weight"]
         if self.unit_offset:
             self.weight = (self.weight.float() + 1.0).contiguous()
+        if self.scaled:
+            self.weight = (self.weight.float() * tensors["scale"].float()).contiguous()
 
     gives_scaled_rows = True
 
@@ -48,9 +56,15 @@ class RMSNorm:
     def add_normed(self, stream, y):
         """``stream.residual += norm(y)``, in one kernel; returns the new residual in the compute dtype (the input
         of the next sublayer), which the stream also keeps as ``lowered``."""
-        if hasattr(y, "compute"):     # a product left pending for a norm in front of the next sublayer: not this one
-            y = y.compute()
-        out = self.env.kernels.norm_add(stream.residual, y, self.weight, self.eps, self.env.dtype)
+        k = self.env.kernels
+        if isinstance(y, NormedSum) and len(y.terms) == 2:       # both inner norms, the sum and this norm in one kernel
+            out = k.norm_add_pair(stream.residual, y.values(), self.weight, self.eps, self.env.dtype)
+        elif isinstance(y, BiasedDelta):
+            out = k.norm_add(stream.residual, y.value(), self.weight, self.eps, self.env.dtype, bias=y.bias)
+        else:
+            if hasattr(y, "compute"):     # a product left pending for a norm in front of the next sublayer: not this one
+                y = y.compute()
+            out = k.norm_add(stream.residual, y, self.weight, self.eps, self.env.dtype)
         stream.lowered = out
         return out
 

@@ -25,14 +25,43 @@ class TwinKernels:
     def embed(self, token_ids, table, scale=1.0):
         return table[token_ids.long()].float() * scale
 
+    def embed_pairs(self, token_ids, table, pair_table, pairs, ctx, state, scale=1.0):
+        buckets, mul_prev, mul_cur = pairs
+        ids, pos = token_ids.tolist(), ctx.positions.tolist()
+        cu, slots = ctx.cu_q.tolist(), ctx.state_slots.tolist()
+        rows = torch.zeros(len(ids), dtype=torch.long)
+        for s in range(ctx.n_seqs):
+            prev = int(state[slots[s], 0])
+            for t in range(cu[s], cu[s + 1]):
+                rows[t] = buckets if pos[t] == 0 else (prev * mul_prev + ids[t] * mul_cur) % buckets
+                prev = ids[t]
+            state[slots[s], 0] = prev
+        return table[token_ids.long()].float() * scale + pair_table[rows].float()
+
     def cast(self, x, dtype):
         return x.to(dtype)
 
     # -- residual += rms norm of a sublayer's output ---------------------------
-    def norm_add(self, residual, y, weight, eps, out_dtype):
+    def norm_add(self, residual, y, weight, eps, out_dtype, bias=None):
         yf = y.float()
+        if bias is not None:
+            yf = yf + bias.float()
         residual.add_(yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * weight.float())
         return residual if out_dtype == torch.float32 else residual.to(out_dtype)
+
+    @staticmethod
+    def _normed_terms(terms):
+        total = 0.0
+        for y, factor, gain, eps in terms:
+            yf = y.float()
+            total = total + factor * (yf * torch.rsqrt(yf.pow(2).mean(-1, keepdim=True) + eps) * gain.float())
+        return total
+
+    def normed_sum(self, terms):
+        return self._normed_terms(terms).to(terms[0][0].dtype)
+
+    def norm_add_pair(self, residual, terms, weight, eps, out_dtype):
+        return self.norm_add(residual, self._normed_terms(terms), weight, eps, out_dtype)
 
     # -- residual add (of a result, or of its rms norm) + layer norm ------------
     def add_layernorm(self, residual, delta, post, weight, bias, eps, out_dtype, rows=None):
@@ -295,6 +324,110 @@ class TwinKernels:
         out = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps) * norm_weight.float()
         return out.view(n, H * Dv).to(proj.dtype)
 
+    # -- a state beside pages, recurrences with inputs of their own -------------------------
+    @staticmethod
+    def _ring_conv(u, weight, ctx, ring):
+        """Causal convolution of ``u [n, channels]`` (float) whose last inputs lie in ``ring [slots, taps, channels]``."""
+        channels, taps = weight.shape
+        out = torch.zeros_like(u)
+        cu, slots, pos = ctx.cu_q.tolist(), ctx.state_slots.tolist(), ctx.positions.tolist()
+        for s in range(ctx.n_seqs):
+            if cu[s] == cu[s + 1]:
+                continue
+            first, n = pos[cu[s]], cu[s + 1] - cu[s]
+            past = [ring[slots[s], (first - i) % taps].clone() if first - i >= 0 else torch.zeros(channels)
+                    for i in range(taps - 1, 0, -1)]
+            seq = torch.cat([torch.stack(past), u[cu[s]:cu[s + 1]]]) if past else u[cu[s]:cu[s + 1]]
+            out[cu[s]:cu[s + 1]] = sum(seq[j:j + n] * weight[:, j].float() for j in range(taps))
+            for i in range(max(0, n - taps + 1), n):
+                if taps > 1:
+                    ring[slots[s], (first + i) % taps] = u[cu[s] + i]
+        return out
+
+    def row_prepare(self, proj, columns, n_heads, n_kv, head_dim, value_dim, rotary_dim, cos, sin, pairing, bias, conv, norm,
+                    page_dim, ctx, cache):
+        n, dtype = proj.shape[0], proj.dtype
+        sizes = (n_heads * head_dim, n_kv * head_dim, n_kv * value_dim)
+        u = torch.cat([proj[:, c:c + size].float() for c, size in zip(columns, sizes)], dim=1)
+        if bias is not None:
+            u = u + bias.float()
+        if conv is not None:
+            ring = cache.state.view(cache.state.shape[0], conv.shape[1], -1) if conv.shape[1] > 1 else None
+            u = self._ring_conv(u, conv, ctx, ring)
+        q, k, v = u.split(sizes, dim=1)
+        rows = {"q": (q, n_heads), "k": (k, n_kv)}
+        for i, name in enumerate(rows):
+            x, heads = rows[name]
+            if norm is not None:
+                gain, eps, over = norm[i].float(), norm[2], norm[3]
+                x = x if over == "row" else x.reshape(n, heads, head_dim)
+                x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * gain
+            rows[name] = self._rotate_pairs(x.reshape(n, heads, head_dim), rotary_dim, cos, sin, ctx.positions, pairing).to(dtype)
+        pos = ctx.positions.long()
+        page = cache.block_table.long()[ctx.seq_of_token.long(), pos // cache.page_size]
+        off = pos % cache.page_size
+        cache.k_pages[page, :, off, :head_dim] = rows["k"]
+        cache.v_pages[page, :, :value_dim, off] = v.reshape(n, n_kv, value_dim).to(dtype)
+        wide = page_dim or head_dim
+        out = torch.zeros(n, n_heads, wide, dtype=dtype)
+        out[:, :, :head_dim] = rows["q"]
+        return out.view(n, n_heads * wide)
+
+    def linear_unit(self, proj, y_col, x_col, terms, blocks, ctx, state):
+        width, taps = terms["conv"].shape
+        bs, dtype = width // blocks, proj.dtype
+        x = proj[:, x_col:x_col + width].float() + terms["x_bias"]
+        ring = state[:, width:width * (1 + taps)].view(state.shape[0], taps, width) if taps > 1 else None
+        u = (self._ring_conv(x, terms["conv"], ctx, ring) + terms["conv_bias"]).to(dtype).float()
+        parts = u.view(-1, blocks, bs)
+        gate = lambda w, b: torch.sigmoid(torch.einsum("nbi,boi->nbo", parts, w.float()).reshape(u.shape) + b)
+        r, i = gate(terms["ra"], terms["ra_bias"]), gate(terms["ri"], terms["ri_bias"])
+        log_a = -r * terms["rate"]
+        a, b = torch.exp(log_a), torch.sqrt(-torch.expm1(2 * log_a)) * i * u
+        S_out = torch.zeros_like(u)
+        cu, slots = ctx.cu_q.tolist(), ctx.state_slots.tolist()
+        for s in range(ctx.n_seqs):
+            S = state[slots[s], :width]
+            for t in range(cu[s], cu[s + 1]):
+                S.copy_(a[t] * S + b[t])
+                S_out[t] = S
+        y = proj[:, y_col:y_col + width].float() + terms["y_bias"]
+        y = 0.5 * y * (1 + torch.tanh(0.7978845608028654 * (y + 0.044715 * y ** 3)))
+        return (S_out * y).to(dtype)
+
+    def token_shift(self, h, mu, ctx, state, state_offset):
+        hf = h.float()
+        before = torch.zeros_like(hf)
+        cu, slots = ctx.cu_q.tolist(), ctx.state_slots.tolist()
+        for s in range(ctx.n_seqs):
+            if cu[s] == cu[s + 1]:
+                continue
+            kept = state[slots[s], state_offset:state_offset + h.shape[1]]
+            before[cu[s]] = kept
+            before[cu[s] + 1:cu[s + 1]] = hf[cu[s]:cu[s + 1] - 1]
+            kept.copy_(hf[cu[s + 1] - 1])
+        return torch.stack([hf + (before - hf) * m.float() for m in mu]).to(h.dtype)
+
+    def grouped_linear(self, x, w, rows):
+        outs = [self.linear(x[g], w[g * rows:(g + 1) * rows] if g + 1 < x.shape[0] else w[g * rows:]) for g in range(x.shape[0])]
+        return torch.stack(outs[:-1]), outs[-1]
+
+    def bonus_recurrence(self, rkvg, low, w2, w0, u, norm_weight, n_heads, head_dim, eps, ctx, state):
+        n, H, D = low.shape[0], n_heads, head_dim
+        r, k, v = (rkvg[i].float().view(n, H, D) for i in range(3))
+        z = torch.tanh(low.float()) @ w2.float().T + w0
+        decay = torch.exp(-torch.exp(z)).view(n, H, D)
+        out = torch.zeros(n, H, D)
+        cu, slots = ctx.cu_q.tolist(), ctx.state_slots.tolist()
+        bonus = u.float().view(H, D)
+        for s in range(ctx.n_seqs):
+            S = state[slots[s], :H * D * D].view(H, D, D)
+            for t in range(cu[s], cu[s + 1]):
+                out[t] = torch.einsum("hd,hdv->hv", r[t], S) + (r[t] * bonus * k[t]).sum(-1, keepdim=True) * v[t]
+                S.mul_(decay[t][:, :, None]).add_(k[t][:, :, None] * v[t][:, None, :])
+        out = (out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps)).view(n, H * D) * norm_weight.float()
+        return (out * torch.nn.functional.silu(rkvg[3].float())).to(rkvg.dtype)
+
     # -- latent attention ------------------------------------------------------------------
     @staticmethod
     def _rotate_pairs(x, rotary_dim, cos, sin, pos, pairing="interleaved"):
@@ -349,8 +482,10 @@ class TwinKernels:
         return y.view(n, H * out_stride).to(x.dtype)
 
     # -- mixture of experts ---------------------------------------------------------
-    def moe_route(self, h, router, top, score="softmax", groups=None, scale=1.0, correction=None):
+    def moe_route(self, h, router, top, score="softmax", groups=None, scale=1.0, correction=None, bias=None):
         logits = h.float() @ router.float().T
+        if bias is not None:
+            logits = logits + bias.float()
         if score == "softmax_all":
             sc = torch.softmax(logits, -1)
             ranked = sc + correction.float() if correction is not None else sc
@@ -382,6 +517,8 @@ class TwinKernels:
         kind, limit = activation
         if kind == "relu":
             return torch.relu(g) * u
+        if kind == "gelu_tanh":
+            return 0.5 * g * (1 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g ** 3))) * u
         assert kind == "clamped"
         g, u = g.clamp(max=limit), u.clamp(-limit, limit)
         return g * torch.sigmoid(1.702 * g) * (u + 1.0)
@@ -389,7 +526,8 @@ class TwinKernels:
     def moe_experts(self, h, w_gate_up, w_down, ids, weights, shared=None, shared_gate=None, activation=None,
                     identity=0):
         n, top = ids.shape
-        ff = w_gate_up.shape[1] // 2
+        gated = not isinstance(activation, str)
+        ff = w_gate_up.shape[1] // (2 if gated else 1)
         real = w_gate_up.shape[0]
         x = h.float()
         y = torch.zeros(n, w_down.shape[1])
@@ -401,7 +539,8 @@ class TwinKernels:
                     y[t] += weights[t, k] * x[t]
                     continue
                 gu = w_gate_up[e].float() @ x[t]
-                a = self._glu(gu[:ff], gu[ff:], activation).to(h.dtype).float()
+                a = self._glu(gu[:ff], gu[ff:], activation) if gated else self._act(gu, activation)
+                a = a.to(h.dtype).float()
                 y[t] += weights[t, k] * (w_down[e].float() @ a)
         if shared is not None:
             s = shared.float()
@@ -417,9 +556,11 @@ class TwinKernels:
 
     pending_linear = linear   # computed at once: the twin's norm always has a kernel of its own
 
-    def gated_linear(self, x, w_gate_up, activation=None):
+    def gated_linear(self, x, w_gate_up, activation=None, bias=None):
         if activation is not None:
             gu = self.linear(x, w_gate_up).float()
+            if bias is not None:
+                gu = gu + bias.float()
             inter = gu.shape[-1] // 2
             return self._glu(gu[:, :inter], gu[:, inter:], activation).to(x.dtype)
         return self.swiglu(self.linear(x, w_gate_up))
@@ -431,7 +572,10 @@ class TwinKernels:
         return (g * torch.sigmoid(g) * u).to(gu.dtype)
 
     def activated_linear(self, x, w, activation):
-        z = self.linear(x, w).float()
+        return self._act(self.linear(x, w).float(), activation).to(x.dtype)
+
+    @staticmethod
+    def _act(z, activation):
         if activation == "relu2":
             a = torch.relu(z) ** 2
         elif activation == "gelu_tanh":
@@ -440,7 +584,7 @@ class TwinKernels:
             a = 0.5 * z * (1 + torch.erf(z * 0.7071067811865476))
         else:
             raise ValueError(activation)
-        return a.to(x.dtype)
+        return a
 
     def qkv_to_cache(self, x, w_qkv, n_heads, n_kv_written, head_dim, rotary_dim, cos, sin, ctx, cache,
                      value_dim=None, bias=None, qk_norm=None, q_temp=None, extra_columns=0, values_are_keys=False,
