@@ -47,8 +47,8 @@ __device__ __forceinline__ float activate(float z, int kind) {
 
 // Gated activations of a (gate, up) pair, in float.  SIA_GLU_SILU: silu(g) * u.  SIA_GLU_CLAMPED: with g = min(g, limit)
 // and u = clamp(u, -limit, limit):  g * sigmoid(1.702 g) * (u + 1).
-// SIA_GLU_RELU: max(g, 0) * u.
-enum SiaGlu { SIA_GLU_SILU = 0, SIA_GLU_CLAMPED = 1, SIA_GLU_RELU = 2 };
+// SIA_GLU_RELU: max(g, 0) * u.  SIA_GLU_GELU_TANH: gelu(g) * u in the tanh form.
+enum SiaGlu { SIA_GLU_SILU = 0, SIA_GLU_CLAMPED = 1, SIA_GLU_RELU = 2, SIA_GLU_GELU_TANH = 3 };
 
 __device__ __forceinline__ float gated_activation(float g, float u, int kind, float limit) {
     if (kind == SIA_GLU_CLAMPED) {
@@ -57,6 +57,7 @@ __device__ __forceinline__ float gated_activation(float g, float u, int kind, fl
         return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
     }
     if (kind == SIA_GLU_RELU) return fmaxf(g, 0.f) * u;
+    if (kind == SIA_GLU_GELU_TANH) return activate(g, SIA_GELU_TANH) * u;
     return g / (1.f + expf(-g)) * u;
 }
 

@@ -31,6 +31,55 @@ SIA_EXPORT int sia_embed(const int* ids, const void* table, float* out, int n_to
     return SIA_LAUNCH_CHECK();
 }
 
+// The same with a row of a second table added: token t behind token s takes row (s * mul_prev + t * mul_cur) mod buckets,
+// a sequence's first token row ``buckets``.  The token before a step's first one of a sequence is in the sequence's state
+// (one int); the workgroup of that first token reads it and then leaves the step's last token there, so nobody reads
+// what another has already replaced.
+template <typename T>
+__global__ void embed_pairs_kernel(const int* __restrict__ ids, const T* __restrict__ table, const T* __restrict__ pairs,
+                                   float* __restrict__ out, int hidden, float scale, int buckets, long long mul_prev,
+                                   long long mul_cur, const int* __restrict__ positions,
+                                   const int* __restrict__ seq_of_token, const int* __restrict__ cu_q,
+                                   const int* __restrict__ slots, int* __restrict__ last_token) {
+    const int n = blockIdx.x, seq = seq_of_token[n], first = cu_q[seq];
+    __shared__ int row_s;
+    if (threadIdx.x == 0) {
+        int prev = 0;
+        if (n == first) {
+            int* kept = last_token + slots[seq];
+            prev = *kept;
+            *kept = ids[cu_q[seq + 1] - 1];
+        } else {
+            prev = ids[n - 1];
+        }
+        row_s = positions[n] == 0 ? buckets
+                                  : (int)(((long long)prev * mul_prev + (long long)ids[n] * mul_cur) % buckets);
+    }
+    __syncthreads();
+    const T* src = table + (size_t)ids[n] * hidden;
+    const T* add = pairs + (size_t)min(max(row_s, 0), buckets) * hidden;
+    float* dst = out + (size_t)n * hidden;
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(src[i]) * scale + to_float(add[i]);
+}
+
+SIA_EXPORT int sia_embed_pairs(const int* ids, const void* table, const void* pairs, float* out, int n_tokens, int hidden,
+                               int table_dtype, float scale, int buckets, int mul_prev, int mul_cur,
+                               const int* positions, const int* seq_of_token, const int* cu_q, const int* slots,
+                               int* last_token, hipStream_t stream) {
+    if (n_tokens <= 0) return 0;
+    if (buckets <= 0 || mul_prev < 0 || mul_cur < 0 || !pairs || !last_token) return SIA_BAD_ARGUMENT;
+    dim3 grid(n_tokens), block(256);
+    if (table_dtype == SIA_F32)
+        hipLaunchKernelGGL(embed_pairs_kernel<float>, grid, block, 0, stream, ids, (const float*)table, (const float*)pairs,
+                           out, hidden, scale, buckets, mul_prev, mul_cur, positions, seq_of_token, cu_q, slots, last_token);
+    else if (table_dtype == SIA_BF16)
+        hipLaunchKernelGGL(embed_pairs_kernel<bf16_t>, grid, block, 0, stream, ids, (const bf16_t*)table, (const bf16_t*)pairs,
+                           out, hidden, scale, buckets, mul_prev, mul_cur, positions, seq_of_token, cu_q, slots, last_token);
+    else
+        return SIA_BAD_ARGUMENT;
+    return SIA_LAUNCH_CHECK();
+}
+
 // ---------------------------------------------------------------------------------------
 // Residual add + RMS norm  (reference: ops/rmsnorm.py:41-46, kernels/rmsnorm_kernel.py:105-113)
 //
@@ -176,7 +225,7 @@ SIA_EXPORT int sia_add_rmsnorm_scaled(float* residual, const void* delta, float 
 // ---------------------------------------------------------------------------------------
 // RMS norm of a sublayer's output, added into the residual:
 //
-//   residual[row] += y[row] * rsqrt(mean(y[row]^2) + eps) * w         (all float)
+//   residual[row] += y[row] * rsqrt(mean(y[row]^2) + eps) * w         (all float; y += bias first, if given)
 //   lowered[row]   = the new residual[row], rounded to T               (if lowered is given)
 //
 // for layers whose norm sits behind the sublayer and whose sublayers read the residual itself.  One workgroup a
@@ -184,18 +233,19 @@ SIA_EXPORT int sia_add_rmsnorm_scaled(float* residual, const void* delta, float 
 // ---------------------------------------------------------------------------------------
 template <typename T>
 __global__ void norm_add_kernel(float* __restrict__ residual, const T* __restrict__ y,
-                                const float* __restrict__ weight, T* __restrict__ lowered, int hidden, float eps) {
+                                const float* __restrict__ weight, T* __restrict__ lowered, int hidden, float eps,
+                                const float* __restrict__ bias) {
     __shared__ float scratch[16];
     const size_t base = (size_t)blockIdx.x * hidden;
     float ss = 0.f;
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
-        const float v = to_float(y[base + i]);
+        const float v = to_float(y[base + i]) + (bias ? bias[i] : 0.f);
         ss += v * v;
     }
     ss = block_sum(ss, scratch);
     const float inv = rsqrtf(ss / (float)hidden + eps);
     for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
-        const float x = residual[base + i] + to_float(y[base + i]) * inv * weight[i];
+        const float x = residual[base + i] + (to_float(y[base + i]) + (bias ? bias[i] : 0.f)) * inv * weight[i];
         residual[base + i] = x;
         if (lowered) lowered[base + i] = from_float<T>(x);
     }
@@ -205,21 +255,29 @@ __global__ void norm_add_kernel(float* __restrict__ residual, const T* __restric
 // elements a thread, every input read once, all loads issued before the first is used.
 template <typename T>
 __global__ void norm_add_row_kernel(float* __restrict__ residual, const T* __restrict__ y,
-                                    const float* __restrict__ weight, T* __restrict__ lowered, int hidden, float eps) {
+                                    const float* __restrict__ weight, T* __restrict__ lowered, int hidden, float eps,
+                                    const float* __restrict__ bias) {
     __shared__ float scratch[16];
     const size_t base = (size_t)blockIdx.x * hidden;
     const int i0 = threadIdx.x * 8;
     const bool live = i0 < hidden;
     float x[8], w[8], v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     if (live) {
-        Vec8<float> vr, vw;
+        Vec8<float> vr, vw, vb;
         Vec8<T> vy;
         vr.load(residual + base + i0);
         vw.load(weight + i0);
         vy.load(y + base + i0);
+        if (bias) vb.load(bias + i0);
         vr.get(x);
         vw.get(w);
         vy.get(v);
+        if (bias) {
+            float b[8];
+            vb.get(b);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v[i] += b[i];
+        }
     }
     float ss = 0.f;
 #pragma unroll
@@ -241,14 +299,14 @@ __global__ void norm_add_row_kernel(float* __restrict__ residual, const T* __res
 }
 
 SIA_EXPORT int sia_norm_add(float* residual, const void* y, const float* weight, void* lowered, int n_rows,
-                            int hidden, float eps, int dtype, hipStream_t stream) {
+                            int hidden, float eps, const float* bias, int dtype, hipStream_t stream) {
     if (n_rows <= 0) return 0;
     if ((dtype != SIA_F32 && dtype != SIA_BF16) || hidden <= 0 || !residual || !y || !weight) return SIA_BAD_ARGUMENT;
     dim3 grid(n_rows);
     const bool row = hidden % 8 == 0 && hidden <= 8 * 1024;
     dim3 block(row ? ((hidden / 8 + SIA_WAVE - 1) / SIA_WAVE) * SIA_WAVE : (hidden >= 2048 ? 512 : 256));
 #define LAUNCH(KERNEL, T)                                                                                         \
-    hipLaunchKernelGGL(KERNEL<T>, grid, block, 0, stream, residual, (const T*)y, weight, (T*)lowered, hidden, eps)
+    hipLaunchKernelGGL(KERNEL<T>, grid, block, 0, stream, residual, (const T*)y, weight, (T*)lowered, hidden, eps, bias)
     if (row) {
         if (dtype == SIA_F32) LAUNCH(norm_add_row_kernel, float);
         else LAUNCH(norm_add_row_kernel, bf16_t);
@@ -257,6 +315,128 @@ SIA_EXPORT int sia_norm_add(float* residual, const void* y, const float* weight,
         else LAUNCH(norm_add_kernel, bf16_t);
     }
 #undef LAUNCH
+    return SIA_LAUNCH_CHECK();
+}
+
+// ---------------------------------------------------------------------------------------
+// Two results, each behind an RMS norm of its own and with a constant factor, and the norm of their sum:
+//
+//   m = f1 * rms(y1) * g1 + f2 * rms(y2) * g2;   residual += rms(m) * w;   lowered = the new residual, rounded
+//
+// (without a residual only m is made, rounded, in ``lowered``).  A workgroup a row; eight elements a thread, held in
+// registers, where the row allows.
+// ---------------------------------------------------------------------------------------
+struct NormPair {
+    const void *y1, *y2;
+    const float *g1, *g2, *weight;
+    float f1, f2, eps1, eps2, eps;
+    float* residual;
+    void* lowered;
+    int hidden;
+};
+
+template <typename T, bool ROW>
+__global__ void norm_pair_kernel(const NormPair p) {
+    __shared__ float scratch[16];
+    const size_t base = (size_t)blockIdx.x * p.hidden;
+    const T *y1 = (const T*)p.y1 + base, *y2 = (const T*)p.y2 + base;
+    T* low = p.lowered ? (T*)p.lowered + base : nullptr;
+    if constexpr (ROW) {
+        const int i0 = threadIdx.x * 8;
+        const bool live = i0 < p.hidden;
+        float a[8] = {}, b[8] = {}, ga[8], gb[8], w[8], x[8];
+        if (live) {
+            Vec8<T> va, vb;
+            Vec8<float> vga, vgb, vw, vr;
+            va.load(y1 + i0);
+            vb.load(y2 + i0);
+            vga.load(p.g1 + i0);
+            vgb.load(p.g2 + i0);
+            if (p.residual) {
+                vw.load(p.weight + i0);
+                vr.load(p.residual + base + i0);
+                vw.get(w);
+                vr.get(x);
+            }
+            va.get(a);
+            vb.get(b);
+            vga.get(ga);
+            vgb.get(gb);
+        }
+        float sa = 0.f, sb = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            sa += a[i] * a[i];
+            sb += b[i] * b[i];
+        }
+        sa = block_sum(sa, scratch);
+        sb = block_sum(sb, scratch);
+        const float ia = p.f1 * rsqrtf(sa / (float)p.hidden + p.eps1), ib = p.f2 * rsqrtf(sb / (float)p.hidden + p.eps2);
+        float ss = 0.f;
+        if (live) {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                a[i] = ia * a[i] * ga[i] + ib * b[i] * gb[i];
+                ss += a[i] * a[i];
+            }
+        }
+        if (p.residual) {      // uniform
+            const float inv = rsqrtf(block_sum(ss, scratch) / (float)p.hidden + p.eps);
+            if (live) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) a[i] = x[i] + a[i] * inv * w[i];
+                Vec8<float> vr;
+                vr.set(a);
+                vr.store(p.residual + base + i0);
+            }
+        }
+        if (live && low) {
+            Vec8<T> vo;
+            vo.set(a);
+            vo.store(low + i0);
+        }
+    } else {
+        float sa = 0.f, sb = 0.f;
+        for (int i = threadIdx.x; i < p.hidden; i += blockDim.x) {
+            const float a = to_float(y1[i]), b = to_float(y2[i]);
+            sa += a * a;
+            sb += b * b;
+        }
+        sa = block_sum(sa, scratch);
+        sb = block_sum(sb, scratch);
+        const float ia = p.f1 * rsqrtf(sa / (float)p.hidden + p.eps1), ib = p.f2 * rsqrtf(sb / (float)p.hidden + p.eps2);
+        auto mixed = [&](int i) { return ia * to_float(y1[i]) * p.g1[i] + ib * to_float(y2[i]) * p.g2[i]; };
+        float inv = 0.f;
+        if (p.residual) {
+            float ss = 0.f;
+            for (int i = threadIdx.x; i < p.hidden; i += blockDim.x) ss += mixed(i) * mixed(i);
+            inv = rsqrtf(block_sum(ss, scratch) / (float)p.hidden + p.eps);
+        }
+        for (int i = threadIdx.x; i < p.hidden; i += blockDim.x) {
+            float x = mixed(i);
+            if (p.residual) {
+                x = p.residual[base + i] + x * inv * p.weight[i];
+                p.residual[base + i] = x;
+            }
+            if (low) low[i] = from_float<T>(x);
+        }
+    }
+}
+
+SIA_EXPORT int sia_norm_pair(float* residual, const void* y1, const float* g1, float f1, float eps1, const void* y2,
+                             const float* g2, float f2, float eps2, const float* weight, float eps, void* lowered,
+                             int n_rows, int hidden, int dtype, hipStream_t stream) {
+    if (n_rows <= 0) return 0;
+    if ((dtype != SIA_F32 && dtype != SIA_BF16) || hidden <= 0 || !y1 || !y2 || !g1 || !g2 || (residual && !weight) ||
+        (!residual && !lowered))
+        return SIA_BAD_ARGUMENT;
+    const NormPair p{y1, y2, g1, g2, weight, f1, f2, eps1, eps2, eps, residual, lowered, hidden};
+    const bool row = hidden % 8 == 0 && hidden <= 8 * 1024;
+    dim3 grid(n_rows), block(row ? ((hidden / 8 + SIA_WAVE - 1) / SIA_WAVE) * SIA_WAVE : (hidden >= 2048 ? 512 : 256));
+    if (dtype == SIA_F32 && row) hipLaunchKernelGGL((norm_pair_kernel<float, true>), grid, block, 0, stream, p);
+    else if (dtype == SIA_F32) hipLaunchKernelGGL((norm_pair_kernel<float, false>), grid, block, 0, stream, p);
+    else if (row) hipLaunchKernelGGL((norm_pair_kernel<bf16_t, true>), grid, block, 0, stream, p);
+    else hipLaunchKernelGGL((norm_pair_kernel<bf16_t, false>), grid, block, 0, stream, p);
     return SIA_LAUNCH_CHECK();
 }
 
@@ -300,17 +480,20 @@ SIA_EXPORT int sia_activation(const void* in, void* out, long long n, int kind, 
 // and the sum of up to two matrices with a constant factor each.
 // ---------------------------------------------------------------------------------------
 template <typename T>
-__global__ void glu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int kind, float limit) {
+__global__ void glu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int kind, float limit,
+                           const float* __restrict__ bias) {
     const int n = blockIdx.y;
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= inter) return;
     const T* row = gu + (size_t)n * 2 * inter;
-    out[(size_t)n * inter + i] = from_float<T>(gated_activation(to_float(row[i]), to_float(row[inter + i]), kind, limit));
+    const float g = to_float(row[i]) + (bias ? bias[i] : 0.f), u = to_float(row[inter + i]) + (bias ? bias[inter + i] : 0.f);
+    out[(size_t)n * inter + i] = from_float<T>(gated_activation(g, u, kind, limit));
 }
 
 // Eight elements a thread, 16- or 32-byte accesses (inter % 8 == 0).
 template <typename T>
-__global__ void glu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int kind, float limit) {
+__global__ void glu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int kind, float limit,
+                               const float* __restrict__ bias) {
     const int n = blockIdx.y;
     const int i = (blockIdx.x * blockDim.x + threadIdx.x) * 8;
     if (i >= inter) return;
@@ -321,33 +504,48 @@ __global__ void glu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, in
     float g[8], u[8];
     vg.get(g);
     vu.get(u);
+    if (bias) {      // uniform
+        Vec8<float> vb, vc;
+        float b[8], c[8];
+        vb.load(bias + i);
+        vc.load(bias + inter + i);
+        vb.get(b);
+        vc.get(c);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            g[j] += b[j];
+            u[j] += c[j];
+        }
+    }
 #pragma unroll
     for (int j = 0; j < 8; ++j) g[j] = gated_activation(g[j], u[j], kind, limit);
     vg.set(g);
     vg.store(out + (size_t)n * inter + i);
 }
 
-SIA_EXPORT int sia_glu(const void* gu, void* out, int n_tokens, int inter, int kind, float limit, int dtype,
-                       hipStream_t stream) {
+// bias: [2 * inter] floats added to gate and up first (null: none).
+SIA_EXPORT int sia_glu(const void* gu, void* out, int n_tokens, int inter, int kind, float limit, const float* bias,
+                       int dtype, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
-    if (n_tokens > 65535 || inter <= 0 || (dtype != SIA_F32 && dtype != SIA_BF16) ||
-        (kind != SIA_GLU_SILU && kind != SIA_GLU_CLAMPED && kind != SIA_GLU_RELU))
+    if (n_tokens > 65535 || inter <= 0 || (dtype != SIA_F32 && dtype != SIA_BF16) || kind < SIA_GLU_SILU ||
+        kind > SIA_GLU_GELU_TANH)
         return SIA_BAD_ARGUMENT;
     if (inter % 8 == 0) {
         dim3 block(256), grid((inter / 8 + 255) / 256, n_tokens);
         if (dtype == SIA_F32)
             hipLaunchKernelGGL(glu_vec_kernel<float>, grid, block, 0, stream, (const float*)gu, (float*)out, inter, kind,
-                               limit);
+                               limit, bias);
         else
             hipLaunchKernelGGL(glu_vec_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)gu, (bf16_t*)out, inter,
-                               kind, limit);
+                               kind, limit, bias);
         return SIA_LAUNCH_CHECK();
     }
     dim3 block(256), grid((inter + 255) / 256, n_tokens);
     if (dtype == SIA_F32)
-        hipLaunchKernelGGL(glu_kernel<float>, grid, block, 0, stream, (const float*)gu, (float*)out, inter, kind, limit);
+        hipLaunchKernelGGL(glu_kernel<float>, grid, block, 0, stream, (const float*)gu, (float*)out, inter, kind, limit, bias);
     else
-        hipLaunchKernelGGL(glu_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)gu, (bf16_t*)out, inter, kind, limit);
+        hipLaunchKernelGGL(glu_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)gu, (bf16_t*)out, inter, kind, limit,
+                           bias);
     return SIA_LAUNCH_CHECK();
 }
 

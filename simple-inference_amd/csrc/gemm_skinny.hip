@@ -38,7 +38,7 @@ __device__ __forceinline__ bf16x8 ld8(const bf16_t* p) {
     return __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(p));
 }
 
-enum SkinnyEpilogue { EPI_STORE = 0, EPI_SWIGLU = 1, EPI_ROPE = 2, EPI_RESIDUAL = 3, EPI_ACT = 4 };
+enum SkinnyEpilogue { EPI_STORE = 0, EPI_SWIGLU = 1, EPI_ROPE = 2, EPI_RESIDUAL = 3, EPI_ACT = 4, EPI_GROUPED = 5 };
 
 // What the q/k/v product needs to rotate its result and to put keys and values into the cache pages.
 struct RopeOut {
@@ -77,6 +77,8 @@ struct Epilogue {
     int table_width, table_dim;
     int glu;          // EPI_SWIGLU: which gated activation (SiaGlu; 0 is silu(gate) * up)
     float limit;      // EPI_SWIGLU: the clamp of the gated activations that have one
+    const float* glu_bias;   // EPI_SWIGLU: if given, [2 * N] floats added to gate and up in front of the activation
+    int groups, group_rows, last_rows, group_blocks;   // EPI_GROUPED: see below
 };
 
 // RB: blocks of bh rows of W per workgroup; WAVES: 8 or 16 waves that split K.
@@ -92,6 +94,10 @@ struct Epilogue {
 //                RMSNorm(x) W^T = rsqrt(mean x^2 + eps) * ((x * gain) W^T): the kernel leaves x * gain and the sums
 //                of squares of its own column blocks, and the product after it (SCALED) adds those up, in an
 //                order that depends on their number only, and scales its rows: no kernel of its own for the norm.
+//   EPI_GROUPED: as EPI_STORE, for W = groups of rows one behind the other that read inputs of their own: X is
+//                [groups][M][K], group g has group_rows rows of W (the last one last_rows) and gives the matrix
+//                Y + g * M * group_rows, [M][its rows]; a workgroup's blocks lie in one group (group_blocks workgroups
+//                each).
 // Output columns come in *units*: a column of Y (EPI_STORE, EPI_RESIDUAL, EPI_SWIGLU, where unit u needs row u of
 // the gate half and row u of the up half of W), or a pair of columns that the rotation mixes (EPI_ROPE: unit u is
 // column u % (head_dim / 2) of head u / (head_dim / 2) together with the column head_dim / 2 further).  A workgroup
@@ -112,11 +118,20 @@ __global__ __launch_bounds__(WAVES* SIA_WAVE) void gemm_skinny_kernel(const bf16
     __shared__ float part[WAVES][RB][16][17];
     __shared__ float squares[SK_SHARES][16];
     const RopeOut& rope = ep.rope;
+    int bx = blockIdx.x;
+    if (EPI == EPI_GROUPED) {
+        const int group = min(bx / ep.group_blocks, ep.groups - 1);
+        bx -= group * ep.group_blocks;
+        N = group + 1 < ep.groups ? ep.group_rows : ep.last_rows;
+        X += (size_t)group * M * K;
+        W += (size_t)group * ep.group_rows * K;
+        Y += (size_t)group * M * ep.group_rows;
+    }
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / SIA_WAVE);  // a scalar, and the compiler knows
     const int lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
     const int rope_half = EPI == EPI_ROPE ? rope.head_dim / 2 : 0;
     const int units = EPI == EPI_ROPE ? (rope.n_heads + 2 * rope.n_kv) * rope_half : N;
-    const int u0 = blockIdx.x * UNIT_BLOCKS * bh;
+    const int u0 = bx * UNIT_BLOCKS * bh;
     // the unit of place n of unit block jb; places beyond the block or beyond the last unit repeat a unit before
     auto unit_at = [&](int jb, int n) { return min(u0 + jb * bh + min(n, bh - 1), units - 1); };
     auto is_live = [&](int jb, int n) { return n < bh && u0 + jb * bh + n < units; };
@@ -311,6 +326,10 @@ __global__ __launch_bounds__(WAVES* SIA_WAVE) void gemm_skinny_kernel(const bf16
             float gate = total(j, m, n), up = total(UNIT_BLOCKS + j, m, n);
             gate *= rs;
             up *= rs;
+            if (ep.glu_bias) {
+                gate += ep.glu_bias[u0 + j * bh + n];
+                up += ep.glu_bias[N + u0 + j * bh + n];
+            }
             *y = from_float<TOut>(ep.glu == SIA_GLU_SILU ? gate / (1.f + expf(-gate)) * up
                                                          : gated_activation(gate, up, ep.glu, ep.limit));
         } else if (EPI == EPI_ACT) {
@@ -431,6 +450,44 @@ SIA_EXPORT int sia_gemm_skinny_embedding_gate(const void* X, const void* W, void
     return SIA_LAUNCH_CHECK();
 }
 
+// The products of groups of rows of W with inputs of their own (EPI_GROUPED): Y[g] = X[g] W[g]^T in bfloat16, group g's
+// matrix at Y + g * M * group_rows.  Needs M <= 16, K % 64 == 0.
+SIA_EXPORT int sia_gemm_skinny_grouped(const void* X, const void* W, void* Y, int M, int K, int groups, int group_rows,
+                                       int last_rows, hipStream_t stream) {
+    if (M <= 0) return 0;
+    if (M > 16 || K % 64 || K <= 0 || groups <= 0 || group_rows <= 0 || last_rows <= 0 || !X || !W || !Y) return SIA_BAD_ARGUMENT;
+    const int cus = compute_units();
+    Cut best{0, 0, 0, 0};
+    int best_blocks = 0;
+    for (int ub : {4, 2, 1})
+        for (int bh = 16; bh >= 8; --bh) {
+            const int a_group = (group_rows + ub * bh - 1) / (ub * bh), last = (last_rows + ub * bh - 1) / (ub * bh);
+            const int grid = (groups - 1) * a_group + last;
+            const Cut c{ub, bh, grid, (long long)((grid + cus - 1) / cus) * bh * ub};
+            if (!best.grid || c.cost < best.cost || (c.cost == best.cost && c.bh > best.bh)) {
+                best = c;
+                best_blocks = a_group;
+            }
+        }
+    Epilogue ep{};
+    ep.groups = groups;
+    ep.group_rows = group_rows;
+    ep.last_rows = last_rows;
+    ep.group_blocks = best_blocks;
+#define LAUNCH(RB, WAVES)                                                                                            \
+    hipLaunchKernelGGL((gemm_skinny_kernel<bf16_t, RB, WAVES, EPI_GROUPED, false>), dim3(best.grid),                  \
+                       dim3(WAVES * SIA_WAVE), 0, stream, (const bf16_t*)X, (const bf16_t*)W, (bf16_t*)Y, M, group_rows, \
+                       K, best.bh, ep)
+    if (best.unit_blocks == 4)
+        LAUNCH(4, 8);
+    else if (best.unit_blocks == 2)
+        LAUNCH(2, 16);
+    else
+        LAUNCH(1, 8);
+#undef LAUNCH
+    return SIA_LAUNCH_CHECK();
+}
+
 // Blocks of columns whose sums of squares sia_gemm_skinny_residual leaves for a result of N columns.
 SIA_EXPORT int sia_gemm_skinny_residual_blocks(int N) {
     if (N <= 0) return 0;
@@ -490,15 +547,16 @@ SIA_EXPORT int sia_gemm_skinny_tiled(const void* X, const void* W_tiled, void* Y
 // Y[M, I] = silu(X Wg^T) * (X Wu^T) for W = [Wg; Wu] of 2 I rows.  Needs M <= 16, K % 64 == 0.
 // With `partials` (else null) X is a `scaled` matrix of sia_gemm_skinny_residual and the rows are divided by their
 // root mean square first.
-// glu, limit: another gated activation than silu(gate) * up (SiaGlu of common.h).
+// glu, limit: another gated activation than silu(gate) * up (SiaGlu of common.h); bias: [2 I] floats or null.
 SIA_EXPORT int sia_gemm_skinny_glu(const void* X, const void* W, void* Y, int M, int inter, int K,
                                    const float* partials, int n_partials, float eps, int glu, float limit,
-                                   hipStream_t stream) {
+                                   const float* bias, hipStream_t stream) {
     if (M <= 0 || inter <= 0) return 0;
     if (M > 16 || K % 64 || K <= 0 || (partials && n_partials <= 0) ||
-        (glu != SIA_GLU_SILU && glu != SIA_GLU_CLAMPED && glu != SIA_GLU_RELU))
+        glu < SIA_GLU_SILU || glu > SIA_GLU_GELU_TANH)
         return SIA_BAD_ARGUMENT;
     Epilogue ep{};
+    ep.glu_bias = bias;
     ep.scale = RowScale{partials, n_partials, eps};
     ep.glu = glu;
     ep.limit = limit;
@@ -521,7 +579,7 @@ SIA_EXPORT int sia_gemm_skinny_glu(const void* X, const void* W, void* Y, int M,
 
 SIA_EXPORT int sia_gemm_skinny_swiglu(const void* X, const void* W, void* Y, int M, int inter, int K,
                                       const float* partials, int n_partials, float eps, hipStream_t stream) {
-    return sia_gemm_skinny_glu(X, W, Y, M, inter, K, partials, n_partials, eps, SIA_GLU_SILU, 0.f, stream);
+    return sia_gemm_skinny_glu(X, W, Y, M, inter, K, partials, n_partials, eps, SIA_GLU_SILU, 0.f, nullptr, stream);
 }
 
 // The q/k/v product of single-token steps with the rotation and the cache write in its epilogue:

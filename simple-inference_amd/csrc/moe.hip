@@ -18,14 +18,15 @@
 // score_mode 0: the softmax over the chosen logits alone.  score_mode 1: scores s = sigmoid(z); with n_groups > 0 the
 // experts form n_groups equal groups of neighbours, a group's score is the sum of its two largest s, and only
 // experts of the keep_groups best groups (ties: the lower group) can be chosen; the weights are the chosen s divided
-// by their sum (+ 1e-20), times weight_scale.  score_mode 2: scores s = softmax(z) over all experts; the choice goes by
+// by their sum (+ 1e-20), times weight_scale.  With logit_bias (score_mode 0) the logits are z + logit_bias.  score_mode 2: scores s = softmax(z) over all experts; the choice goes by
 // s + correction (a float per expert, if given), the weights are the chosen s divided by their sum (+ 1e-20).
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h, const float* __restrict__ router,
                                                          int* __restrict__ ids, float* __restrict__ weights, int width,
                                                          int n_experts, int top, int score_mode, int n_groups,
                                                          int keep_groups, float weight_scale,
-                                                         const float* __restrict__ correction) {
+                                                         const float* __restrict__ correction,
+                                                         const float* __restrict__ logit_bias) {
     __shared__ float logit_s[MOE_MAX_EXPERTS];
     __shared__ float group_s[MOE_MAX_EXPERTS];
     const int n = blockIdx.x, wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE;
@@ -40,7 +41,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
             for (int u = 0; u < 4; ++u) acc[u] += to_float(x[i + u * SIA_WAVE]) * w[i + u * SIA_WAVE];
         }
         for (; i < width; i += SIA_WAVE) acc[0] += to_float(x[i]) * w[i];
-        const float total = wave_sum((acc[0] + acc[1]) + (acc[2] + acc[3]));
+        float total = wave_sum((acc[0] + acc[1]) + (acc[2] + acc[3]));
+        if (logit_bias) total += logit_bias[e];
         if (lane == 0) logit_s[e] = score_mode == 1 ? 1.f / (1.f + expf(-total)) : total;
     }
     __syncthreads();
@@ -130,20 +132,22 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ h,
 
 static int route(const void* h, const float* router, int* ids, float* weights, int n_tokens, int width, int n_experts,
                  int top, int dtype, int score_mode, int n_groups, int keep_groups, float weight_scale,
-                 const float* correction, hipStream_t stream) {
+                 const float* correction, hipStream_t stream, const float* logit_bias = nullptr) {
     if (n_tokens <= 0) return 0;
     if (n_experts <= 0 || n_experts > MOE_MAX_EXPERTS || top <= 0 || top > n_experts || top > MOE_MAX_TOP ||
         (score_mode != 0 && score_mode != 1 && score_mode != 2) || n_groups < 0 || (correction && score_mode != 2) ||
+        (logit_bias && score_mode != 0) ||
         (n_groups > 0 && (score_mode != 1 || n_experts % n_groups || keep_groups <= 0 || keep_groups > n_groups ||
                           top > n_experts / n_groups * keep_groups)))
         return SIA_BAD_ARGUMENT;
     dim3 grid(n_tokens), block(256);
     if (dtype == SIA_F32)
         hipLaunchKernelGGL(moe_route_kernel<float>, grid, block, 0, stream, (const float*)h, router, ids, weights, width,
-                           n_experts, top, score_mode, n_groups, keep_groups, weight_scale, correction);
+                           n_experts, top, score_mode, n_groups, keep_groups, weight_scale, correction, logit_bias);
     else if (dtype == SIA_BF16)
         hipLaunchKernelGGL(moe_route_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)h, router, ids, weights,
-                           width, n_experts, top, score_mode, n_groups, keep_groups, weight_scale, correction);
+                           width, n_experts, top, score_mode, n_groups, keep_groups, weight_scale, correction,
+                           logit_bias);
     else
         return SIA_BAD_ARGUMENT;
     return SIA_LAUNCH_CHECK();
@@ -163,9 +167,22 @@ SIA_EXPORT int sia_moe_route_corrected(const void* h, const float* router, const
     return route(h, router, ids, weights, n_tokens, width, n_experts, top, dtype, 2, 0, 0, 1.f, correction, stream);
 }
 
+// the softmax over the chosen logits (score_mode 0) of logits with a bias
+SIA_EXPORT int sia_moe_route_biased(const void* h, const float* router, const float* bias, int* ids, float* weights,
+                                    int n_tokens, int width, int n_experts, int top, int dtype, hipStream_t stream) {
+    return route(h, router, ids, weights, n_tokens, width, n_experts, top, dtype, 0, 0, 0, 1.f, nullptr, stream, bias);
+}
+
 SIA_EXPORT int sia_moe_route(const void* h, const float* router, int* ids, float* weights, int n_tokens, int width,
                              int n_experts, int top, int dtype, hipStream_t stream) {
     return sia_moe_route_ex(h, router, ids, weights, n_tokens, width, n_experts, top, dtype, 0, 0, 0, 1.f, stream);
+}
+
+// Experts without a gate: ``glu`` is then MOE_UNGATED + the SiaActivation of W2 act(Wu h), and W1 is [E, ff, width].
+#define MOE_UNGATED 16
+
+static bool moe_known_activation(int glu) {
+    return glu == SIA_GLU_SILU || glu == SIA_GLU_CLAMPED || (glu >= MOE_UNGATED + SIA_RELU2 && glu <= MOE_UNGATED + SIA_GELU);
 }
 
 // dot product of two rows of K elements by one wave (every lane gets the sum)
@@ -200,12 +217,14 @@ __global__ __launch_bounds__(MOE_WAVES* SIA_WAVE) void moe_gate_up_kernel(
     const int e = ids[slot];
     if (e >= n_real) return;     // an expert without tensors: the down kernel hands the token's input on
     const T* x = h + (size_t)(slot / top) * width;
-    const T* w = w1 + (size_t)e * 2 * ff * width;
+    const bool gated = glu < MOE_UNGATED;
+    const T* w = w1 + (size_t)e * (gated ? 2 : 1) * ff * width;
     const int f0 = (blockIdx.y * MOE_WAVES + wave) * MOE_PER_WAVE;
     for (int f = f0; f < min(ff, f0 + MOE_PER_WAVE); ++f) {
         const float g = wave_dot<T>(x, w + (size_t)f * width, width, lane, vec);
-        const float u = wave_dot<T>(x, w + (size_t)(ff + f) * width, width, lane, vec);
-        if (lane == 0) act[(size_t)slot * ff + f] = from_float<T>(gated_activation(g, u, glu, limit));
+        const float u = gated ? wave_dot<T>(x, w + (size_t)(ff + f) * width, width, lane, vec) : 0.f;
+        if (lane == 0)
+            act[(size_t)slot * ff + f] = from_float<T>(gated ? gated_activation(g, u, glu, limit) : activate(g, glu - MOE_UNGATED));
     }
 }
 
@@ -242,7 +261,7 @@ SIA_EXPORT int sia_moe_gate_up_ex(const void* h, const void* w1, const int* ids,
                                   int ff, int top, int n_real, int glu, float limit, int dtype, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (width <= 0 || ff <= 0 || top <= 0 || (long long)n_tokens * top > 0x7fffffffLL || n_real <= 0 ||
-        (glu != SIA_GLU_SILU && glu != SIA_GLU_CLAMPED))
+        !moe_known_activation(glu))
         return SIA_BAD_ARGUMENT;
     const int per_block = MOE_WAVES * MOE_PER_WAVE;
     dim3 grid(n_tokens * top, (ff + per_block - 1) / per_block), block(MOE_WAVES * SIA_WAVE);
@@ -350,7 +369,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
 
 __device__ __forceinline__ moe_bf16x8 moe_ld8(const bf16_t* p) { return *reinterpret_cast<const moe_bf16x8*>(p); }
 
-// GATED: rows f and ff + f of W make silu(gate) * up; else a plain product.  Output row stride n_out.
+// GATED: rows f and ff + f of W make silu(gate) * up; else a plain product, or with ``glu`` at MOE_UNGATED and beyond the
+// activation of it.  Output row stride n_out.
 template <bool GATED>
 __global__ __launch_bounds__(256) void moe_tile_kernel(const bf16_t* __restrict__ x, int rows_per_slot,
                                                        const bf16_t* __restrict__ w, const int* __restrict__ place_slot,
@@ -417,6 +437,7 @@ __global__ __launch_bounds__(256) void moe_tile_kernel(const bf16_t* __restrict_
             for (int i = 0; i < 4; ++i) {
                 float y = acc[nb][mb][0][i];
                 if (GATED) y = gated_activation(y, acc[nb][mb][1][i], glu, limit);
+                else if (glu >= MOE_UNGATED) y = activate(y, glu - MOE_UNGATED);
                 v[i] = float_to_bf16(y);
             }
             bf16_t* dst = out + row * n_out + c;
@@ -470,7 +491,7 @@ SIA_EXPORT int sia_moe_tiled_ex(const void* h, const void* w1, const void* w2, c
                                 int glu, float limit, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
     if (sia_moe_tiled_workspace(n_tokens, top, n_experts, width, ff) == 0 || n_experts > MOE_MAX_EXPERTS ||
-        (shared_gate && !shared) || (glu != SIA_GLU_SILU && glu != SIA_GLU_CLAMPED))
+        (shared_gate && !shared) || !moe_known_activation(glu))
         return SIA_BAD_ARGUMENT;
     const int slots = n_tokens * top;
     const int max_tiles = (slots + MOE_TILE - 1) / MOE_TILE + n_experts;
@@ -479,9 +500,14 @@ SIA_EXPORT int sia_moe_tiled_ex(const void* h, const void* w1, const void* w2, c
     int* n_tiles = tile_expert + max_tiles;
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, ids, slots, n_experts, place_slot, tile_expert,
                        n_tiles, max_tiles);
-    hipLaunchKernelGGL(moe_tile_kernel<true>, dim3(max_tiles, (ff + 127) / 128), dim3(256), 0, stream,
-                       (const bf16_t*)h, top, (const bf16_t*)w1, place_slot, tile_expert, n_tiles, (bf16_t*)act, width, ff,
-                       glu, limit);
+    if (glu >= MOE_UNGATED)
+        hipLaunchKernelGGL(moe_tile_kernel<false>, dim3(max_tiles, (ff + 127) / 128), dim3(256), 0, stream,
+                           (const bf16_t*)h, top, (const bf16_t*)w1, place_slot, tile_expert, n_tiles, (bf16_t*)act, width,
+                           ff, glu, limit);
+    else
+        hipLaunchKernelGGL(moe_tile_kernel<true>, dim3(max_tiles, (ff + 127) / 128), dim3(256), 0, stream,
+                           (const bf16_t*)h, top, (const bf16_t*)w1, place_slot, tile_expert, n_tiles, (bf16_t*)act, width,
+                           ff, glu, limit);
     hipLaunchKernelGGL(moe_tile_kernel<false>, dim3(max_tiles, (width + 127) / 128), dim3(256), 0, stream,
                        (const bf16_t*)act, 1, (const bf16_t*)w2, place_slot, tile_expert, n_tiles, (bf16_t*)y, ff, width,
                        SIA_GLU_SILU, 0.f);

@@ -28,12 +28,16 @@
 
 __device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
 
-template <typename T, int ROWS>
+// BONUS: the query reads the state before this token's write, and the write itself weighed per key channel by ``bonus``
+// [heads, D] for this token only:  o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T q_t.  Where the outputs go to ``raw_out`` the
+// weighed write is left to the finishing kernel.  The norm's weights are then [heads, Dv], not shared.
+template <typename T, int ROWS, bool BONUS>
 __global__ __launch_bounds__(512) void gla_recurrent_kernel(
     const T* __restrict__ proj, int row_stride, int q_col, int k_col, int v_col, int g_col,
     const float* __restrict__ alpha, const float* __restrict__ norm_w, float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ slots, T* __restrict__ out,
     int n_heads, int D, int Dv, int R, int block_tokens, float q_scale, float eps, int slice,
-    float* __restrict__ raw_out, const float* __restrict__ k_f32, int q_share, long long state_stride) {
+    float* __restrict__ raw_out, const float* __restrict__ k_f32, int q_share, long long state_stride,
+    const float* __restrict__ bonus) {
     extern __shared__ float lds[];
     const int seq = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
     const int j0 = blockIdx.z * slice;     // this workgroup's columns: j0 .. j0 + slice - 1
@@ -46,6 +50,9 @@ __global__ __launch_bounds__(512) void gla_recurrent_kernel(
     float* v_s = al_s + TB * D;        // [TB][Dv]
     float* g_s = v_s + TB * Dv;        // [TB][Dv]
     float* o_s = g_s + TB * Dv;        // [TB][Dv]
+    float* u_s = o_s + TB * Dv;        // [D], BONUS only
+    if (BONUS)      // (read behind the first block's barrier)
+        for (int d = tid; d < D; d += blockDim.x) u_s[d] = raw_out ? 0.f : bonus[(size_t)head * D + d];
 
     const int j = j0 + tid / R, r = tid % R;
     const bool owns = tid / R < slice && j < Dv;
@@ -83,8 +90,10 @@ __global__ __launch_bounds__(512) void gla_recurrent_kernel(
             for (int i = 0; i < ROWS; ++i) {
                 const int d = i * R + r;
                 if (d < D) {
-                    S[i] = al_s[t * D + d] * S[i] + k_s[t * D + d] * v;
-                    acc += q_s[t * D + d] * S[i];
+                    const float write = k_s[t * D + d] * v;
+                    if (BONUS) acc += q_s[t * D + d] * (S[i] + u_s[d] * write);
+                    S[i] = al_s[t * D + d] * S[i] + write;
+                    if (!BONUS) acc += q_s[t * D + d] * S[i];
                 }
             }
             for (int o = R / 2; o > 0; o >>= 1) acc += __shfl_xor(acc, o, SIA_WAVE);
@@ -102,7 +111,7 @@ __global__ __launch_bounds__(512) void gla_recurrent_kernel(
             T* dst = out + ((size_t)(t0 + t) * n_heads + head) * Dv;
             for (int c = lane; c < Dv; c += SIA_WAVE) {
                 const float g = g_s[t * Dv + c];
-                dst[c] = from_float<T>(o_s[t * Dv + c] * inv * norm_w[c] * (g_col >= 0 ? g / (1.f + expf(-g)) : 1.f));
+                dst[c] = from_float<T>(o_s[t * Dv + c] * inv * norm_w[(BONUS ? head * Dv : 0) + c] * (g_col >= 0 ? g / (1.f + expf(-g)) : 1.f));
             }
         }
         __syncthreads();
@@ -137,7 +146,8 @@ __device__ __forceinline__ float row16_sum(float v) {
 // KF: what is written (k) comes as floats [tokens, heads, D] from ``k_f32``, as the decays do, not as columns of the
 // rows.  ``q_share`` neighbouring heads read the same q columns; a sequence's matrices begin ``state_stride`` floats
 // after the sequence before it.
-template <int ROWS, int GLA_WALK_COLS, bool KF>
+// BEFORE: the query reads the state before this token's write.
+template <int ROWS, int GLA_WALK_COLS, bool KF, bool BEFORE>
 __global__ __launch_bounds__(GLA_WALK_THREADS) void gla_walk_kernel(
     const bf16_t* __restrict__ proj, int row_stride, int q_col, int k_col, int v_col, const float* __restrict__ alpha,
     const float* __restrict__ k_f32, int q_share, float* __restrict__ state, long long state_stride,
@@ -288,14 +298,22 @@ __global__ __launch_bounds__(GLA_WALK_THREADS) void gla_walk_kernel(
                 float acc = 0.f;
 #pragma unroll
                 for (int i = 0; i < ROWS / 4; ++i) {
+                    if (BEFORE) {
+                        acc += qv[i].x * S[c][4 * i];
+                        acc += qv[i].y * S[c][4 * i + 1];
+                        acc += qv[i].z * S[c][4 * i + 2];
+                        acc += qv[i].w * S[c][4 * i + 3];
+                    }
                     S[c][4 * i] = av[i].x * S[c][4 * i] + kv[i].x * v;
                     S[c][4 * i + 1] = av[i].y * S[c][4 * i + 1] + kv[i].y * v;
                     S[c][4 * i + 2] = av[i].z * S[c][4 * i + 2] + kv[i].z * v;
                     S[c][4 * i + 3] = av[i].w * S[c][4 * i + 3] + kv[i].w * v;
-                    acc += qv[i].x * S[c][4 * i];
-                    acc += qv[i].y * S[c][4 * i + 1];
-                    acc += qv[i].z * S[c][4 * i + 2];
-                    acc += qv[i].w * S[c][4 * i + 3];
+                    if (!BEFORE) {
+                        acc += qv[i].x * S[c][4 * i];
+                        acc += qv[i].y * S[c][4 * i + 1];
+                        acc += qv[i].z * S[c][4 * i + 2];
+                        acc += qv[i].w * S[c][4 * i + 3];
+                    }
                 }
                 acc = row16_sum(acc);
                 if (r == 0) o_s[t * slice + jl + c] = acc;
@@ -398,12 +416,14 @@ SIA_EXPORT long long sia_gla_workspace(int n_tokens, int n_seqs, int max_q_len, 
 // slot's.  The outputs go to ``raw`` [tokens, heads, Dv] as floats if the caller wants them there (want_raw) or if a
 // head's columns are shared out between workgroups; otherwise they are normed over the head (norm_w, eps), gated by
 // silu of the columns at g_col (none if negative) and written to ``out``.  Returns through ``raw_used`` whether ``raw``
-// holds the outputs.
+// holds the outputs.  With ``bonus`` [heads, D] the query reads the state before the token's write and, unless the outputs are
+// raw, that write weighed by it; the norm's weights are then [heads, Dv].
 static int launch_recurrence(const void* proj, int row_stride, int q_col, int k_col, int v_col, int g_col,
                              const float* k_f32, int q_share, const float* alpha, const float* norm_w, float* state,
                              long long state_stride, const int* cu_q, const int* slots, void* out, int n_seqs,
                              int max_q_len, int n_heads, int D, int Dv, float q_scale, float eps, int dtype,
-                             float* raw_space, bool want_raw, bool* raw_used, hipStream_t stream) {
+                             float* raw_space, bool want_raw, bool* raw_used, hipStream_t stream,
+                             const float* bonus = nullptr) {
     // columns a workgroup: all of a head's, or with a workspace a slice of them, as narrow as it takes to fill the chip
     int slice = Dv;
     const bool prompt = gla_slices(n_seqs, max_q_len, n_heads);
@@ -423,7 +443,7 @@ static int launch_recurrence(const void* proj, int row_stride, int q_col, int k_
     const bool sliced = slice < Dv;
     const int threads = ((slice * R + SIA_WAVE - 1) / SIA_WAVE) * SIA_WAVE;
     int TB = max_q_len >= 16 ? 16 : (max_q_len >= 4 ? 4 : 1);
-    auto bytes = [&](int tb) { return (size_t)tb * (3 * D + 3 * Dv) * sizeof(float); };
+    auto bytes = [&](int tb) { return ((size_t)tb * (3 * D + 3 * Dv) + (bonus ? D : 0)) * sizeof(float); };
     while (TB > 1 && bytes(TB) > 60 * 1024) TB /= 2;
     if (bytes(TB) > 60 * 1024) return SIA_BAD_ARGUMENT;
     dim3 grid(n_seqs, n_heads, (Dv + slice - 1) / slice), block(threads);
@@ -443,14 +463,15 @@ static int launch_recurrence(const void* proj, int row_stride, int q_col, int k_
     if (raw_used) *raw_used = raw != nullptr;
     if (ahead) {
         dim3 wgrid(n_seqs, n_heads, (Dv + w_slice - 1) / w_slice), wblock(GLA_WALK_THREADS);
-#define WALK_AS(ROWS, COLS, KF)                                                                                      \
-    hipLaunchKernelGGL((gla_walk_kernel<ROWS, COLS, KF>), wgrid, wblock, w_lds, stream, (const bf16_t*)proj,         \
+#define WALK_AS(ROWS, COLS, KF, BEFORE)                                                                                      \
+    hipLaunchKernelGGL((gla_walk_kernel<ROWS, COLS, KF, BEFORE>), wgrid, wblock, w_lds, stream, (const bf16_t*)proj,         \
                        row_stride, q_col, k_col, v_col, alpha, k_f32, q_share, state, state_stride, cu_q, slots,     \
                        n_heads, D, Dv, q_scale, raw)
 #define WALK(ROWS, COLS)                                                                                             \
     do {                                                                                                             \
-        if (k_f32) WALK_AS(ROWS, COLS, true);                                                                        \
-        else WALK_AS(ROWS, COLS, false);                                                                             \
+        if (bonus) WALK_AS(ROWS, COLS, false, true);                                                                 \
+        else if (k_f32) WALK_AS(ROWS, COLS, true, false);                                                            \
+        else WALK_AS(ROWS, COLS, false, false);                                                                      \
     } while (0)
         if (w_rows_t == 4) WALK(4, 2);
         else if (w_rows_t == 8) WALK(8, 2);
@@ -458,10 +479,15 @@ static int launch_recurrence(const void* proj, int row_stride, int q_col, int k_
 #undef WALK
 #undef WALK_AS
     } else {
+#define LAUNCH_AS(T, ROWS, BONUS)                                                                                    \
+    hipLaunchKernelGGL((gla_recurrent_kernel<T, ROWS, BONUS>), grid, block, bytes(TB), stream, (const T*)proj,       \
+                       row_stride, q_col, k_col, v_col, g_col, alpha, norm_w, state, cu_q, slots, (T*)out, n_heads, D, \
+                       Dv, R, TB, q_scale, eps, slice, raw, k_f32, q_share, state_stride, bonus)
 #define LAUNCH(T, ROWS)                                                                                              \
-    hipLaunchKernelGGL((gla_recurrent_kernel<T, ROWS>), grid, block, bytes(TB), stream, (const T*)proj, row_stride,  \
-                       q_col, k_col, v_col, g_col, alpha, norm_w, state, cu_q, slots, (T*)out, n_heads, D, Dv, R, TB,   \
-                       q_scale, eps, slice, raw, k_f32, q_share, state_stride)
+    do {                                                                                                             \
+        if (bonus) LAUNCH_AS(T, ROWS, true);                                                                         \
+        else LAUNCH_AS(T, ROWS, false);                                                                              \
+    } while (0)
 #define PICK(T)                                                                                                      \
     do {                                                                                                             \
         if (rows <= 4) LAUNCH(T, 4);                                                                                 \
@@ -476,8 +502,72 @@ static int launch_recurrence(const void* proj, int row_stride, int q_col, int k_
     else return SIA_BAD_ARGUMENT;
 #undef PICK
 #undef LAUNCH
+#undef LAUNCH_AS
     }
     return 0;
+}
+
+// y = o * rsqrt(mean(o^2) + eps) * w * silu(g) with o = raw + (sum_d q_d bonus_d k_d) v: what the walk left in the float
+// workspace and the token's own weighed write.  A wave a (token, head); q, k, v and g are columns of rows row_stride apart,
+// weights and bonus a head's own.
+template <typename T>
+__global__ __launch_bounds__(SIA_WAVE) void bonus_finish_kernel(const float* __restrict__ raw, const T* __restrict__ proj,
+                                                                int row_stride, int q_col, int k_col, int v_col, int g_col,
+                                                                const float* __restrict__ bonus,
+                                                                const float* __restrict__ norm_w, T* __restrict__ out,
+                                                                int n_heads, int D, int Dv, float eps) {
+    const int n = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
+    const T* row = proj + (size_t)n * row_stride;
+    const T *q = row + q_col + head * D, *k = row + k_col + head * D, *v = row + v_col + head * Dv, *g = row + g_col + head * Dv;
+    float own = 0.f;
+    for (int d = lane; d < D; d += SIA_WAVE) own += to_float(q[d]) * bonus[(size_t)head * D + d] * to_float(k[d]);
+    own = wave_sum(own);
+    const float* o = raw + ((size_t)n * n_heads + head) * Dv;
+    float ss = 0.f;
+    for (int c = lane; c < Dv; c += SIA_WAVE) {
+        const float x = o[c] + own * to_float(v[c]);
+        ss += x * x;
+    }
+    const float inv = rsqrtf(wave_sum(ss) / (float)Dv + eps);
+    T* dst = out + ((size_t)n * n_heads + head) * Dv;
+    for (int c = lane; c < Dv; c += SIA_WAVE) {
+        const float x = o[c] + own * to_float(v[c]), z = to_float(g[c]);
+        dst[c] = from_float<T>(x * inv * norm_w[(size_t)head * Dv + c] * (z / (1.f + expf(-z))));
+    }
+}
+
+// floats of workspace behind the decays: the raw outputs [tokens, heads, D]
+SIA_EXPORT long long sia_bonus_recurrence_workspace(int n_tokens, int n_heads, int D) {
+    return (long long)n_tokens * n_heads * D;
+}
+
+// The recurrence with a bonus for the current token: rkvg is four matrices [tokens, heads * D] one behind the other (r, k, v
+// and the output gate), decays [tokens, heads, D] float, bonus and norm_w [heads, D].
+SIA_EXPORT int sia_bonus_recurrence(const void* rkvg, const float* decays, const float* bonus, const float* norm_w,
+                                    float* state, long long state_stride, const int* cu_q, const int* slots, void* out,
+                                    int n_tokens, int n_seqs, int max_q_len, int n_heads, int D, float eps, int dtype,
+                                    float* workspace, hipStream_t stream) {
+    if (n_seqs <= 0 || n_tokens <= 0) return 0;
+    const long long plane = (long long)n_tokens * n_heads * D;
+    if (D <= 0 || D > 512 || n_heads <= 0 || n_heads > 65535 || !rkvg || !decays || !bonus || !norm_w || !state || !out ||
+        !workspace || state_stride < (long long)n_heads * D * D || 4 * plane > 0x7fffffffLL)
+        return SIA_BAD_ARGUMENT;
+    const int width = n_heads * D, k_col = (int)plane, v_col = (int)(2 * plane), g_col = (int)(3 * plane);
+    bool raw = false;
+    const int code = launch_recurrence(rkvg, width, 0, k_col, v_col, g_col, nullptr, 1, decays, norm_w, state, state_stride,
+                                       cu_q, slots, out, n_seqs, max_q_len, n_heads, D, D, 1.f, eps, dtype, workspace,
+                                       false, &raw, stream, bonus);
+    if (code) return code;
+    if (raw) {
+        dim3 grid(n_tokens, n_heads), block(SIA_WAVE);
+        if (dtype == SIA_F32)
+            hipLaunchKernelGGL(bonus_finish_kernel<float>, grid, block, 0, stream, workspace, (const float*)rkvg, width, 0,
+                               k_col, v_col, g_col, bonus, norm_w, (float*)out, n_heads, D, D, eps);
+        else
+            hipLaunchKernelGGL(bonus_finish_kernel<bf16_t>, grid, block, 0, stream, workspace, (const bf16_t*)rkvg, width,
+                               0, k_col, v_col, g_col, bonus, norm_w, (bf16_t*)out, n_heads, D, D, eps);
+    }
+    return SIA_LAUNCH_CHECK();
 }
 
 SIA_EXPORT int sia_gla_recurrent(const void* proj, int row_stride, int q_col, int k_col, int v_col, int g_col, int a_col,

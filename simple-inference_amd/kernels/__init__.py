@@ -23,13 +23,36 @@ from . import build
 
 _DT = {torch.float32: 0, torch.bfloat16: 1}
 _ACTIVATIONS = {"relu2": 0, "gelu_tanh": 1, "gelu": 2}   # ``SiaActivation`` of csrc/common.h
-_GLUS = {"silu": 0, "clamped": 1, "relu": 2}             # ``SiaGlu`` of csrc/common.h
+_GLUS = {"silu": 0, "clamped": 1, "relu": 2, "gelu_tanh": 3}   # ``SiaGlu`` of csrc/common.h
+_UNGATED = 16                                            # ``MOE_UNGATED`` of csrc/moe.hip
 
 _c_int, _c_float, _c_ptr, _c_ll = ctypes.c_int, ctypes.c_float, ctypes.c_void_p, ctypes.c_longlong
 
 _SIGNATURES = {
     "sia_embed": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr],
-    "sia_norm_add": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
+    "sia_norm_add": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_ptr, _c_int, _c_ptr],
+    "sia_norm_pair": [_c_ptr, _c_ptr, _c_ptr, _c_float, _c_float, _c_ptr, _c_ptr, _c_float, _c_float, _c_ptr, _c_float, _c_ptr,
+                      _c_int, _c_int, _c_int, _c_ptr],
+    "sia_embed_pairs": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr,
+                        _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr],
+    "sia_row_prepare_max_elements": [],
+    "sia_row_prepare": [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int,
+                        _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ll,
+                        _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                        _c_int, _c_int, _c_int, _c_ptr],
+    "sia_linear_unit_max_taps": [],
+    "sia_linear_unit_workspace": [_c_int, _c_int, _c_int],
+    "sia_linear_unit": [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                        _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int,
+                        _c_int, _c_int, _c_int, _c_ptr, _c_ptr],
+    "sia_token_shift": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ll, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
+                        _c_int, _c_ptr],
+    "sia_gemm_skinny_grouped": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+    "sia_low_rank_decay": [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
+    "sia_bonus_recurrence_workspace": [_c_int, _c_int, _c_int],
+    "sia_bonus_recurrence": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
+                             _c_int, _c_int, _c_float, _c_int, _c_ptr, _c_ptr],
+    "sia_moe_route_biased": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "sia_activation": [_c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_ptr],
     "sia_qk_prepare": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int,
                        _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr,
@@ -105,8 +128,9 @@ _SIGNATURES = {
     "sia_add_rmsnorm_scaled": [_c_ptr, _c_ptr, _c_float, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float,
                                _c_int, _c_ptr],
     "sia_scaled_sum": [_c_ptr, _c_float, _c_ptr, _c_float, _c_ptr, _c_ll, _c_int, _c_ptr],
-    "sia_gemm_skinny_glu": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_float, _c_int, _c_float, _c_ptr],
-    "sia_glu": [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr],
+    "sia_gemm_skinny_glu": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_float, _c_int, _c_float, _c_ptr,
+                            _c_ptr],
+    "sia_glu": [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_int, _c_ptr],
     "sia_qk_prepare_ex": [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int,
                           _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr,
                           _c_int, _c_int, _c_float, _c_int, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr],
@@ -252,6 +276,8 @@ class HipKernels:
         self.core.sia_hgrn2_workspace.restype = ctypes.c_longlong
         self.core.sia_ssd_workspace.restype = ctypes.c_longlong
         self.core.sia_delta_rule_workspace.restype = ctypes.c_longlong
+        self.core.sia_linear_unit_workspace.restype = ctypes.c_longlong
+        self.core.sia_bonus_recurrence_workspace.restype = ctypes.c_longlong
         self.tiled_experts = True        # many slots in bfloat16: experts' products on the matrix cores, slots sorted by expert
         self._attn_libs = {}
         # the short way to the current stream's handle, where this torch has it (a few microseconds less a launch)
@@ -391,19 +417,77 @@ class HipKernels:
                                         float(scale), self._stream()), "embed")
         return out
 
+    def embed_pairs(self, token_ids, table, pair_table, pairs, ctx, state, scale=1.0):
+        """``table[t] * scale + pair_table[row]`` (float) for every token ``t`` of the step: ``pairs = (buckets, mul_prev,
+        mul_cur)``, ``row = (s * mul_prev + t * mul_cur) mod buckets`` with ``s`` the token before it in its sequence, and row
+        ``buckets`` at position 0.  ``state [slots, 1]`` (int32) holds every sequence's last token and is left holding the
+        step's last ones."""
+        self._want(token_ids, "token_ids", torch.int32, (ctx.n_tokens,))
+        self._want(table, "embedding table")
+        if table.dtype not in _DT or table.dim() != 2:
+            raise KernelError(f"embedding table must be a float32 or bfloat16 matrix, is {table.dtype} {tuple(table.shape)}")
+        buckets, mul_prev, mul_cur = (int(p) for p in pairs)
+        hidden = table.shape[1]
+        self._want(pair_table, "table of pairs", table.dtype, (buckets + 1, hidden))
+        if state is None or state.dim() != 2 or state.shape[1] != 1:
+            raise KernelError("the embedding of pairs keeps one token a sequence")
+        self._want(state, "last tokens", torch.int32)
+        out = torch.empty((ctx.n_tokens, hidden), dtype=torch.float32, device=table.device)
+        self._check(self.core.sia_embed_pairs(
+            _ptr(token_ids), _ptr(table), _ptr(pair_table), _ptr(out), ctx.n_tokens, hidden, _DT[table.dtype], float(scale),
+            buckets, mul_prev, mul_cur, _ptr(ctx.positions), _ptr(ctx.seq_of_token), _ptr(ctx.cu_q), _ptr(ctx.state_slots),
+            _ptr(state), self._stream()), "embed_pairs")
+        return out
+
     # -- rms norm of a sublayer's output, added into the residual -------------------
-    def norm_add(self, residual, y, weight, eps, out_dtype):
-        """``residual += y * rsqrt(mean(y^2) + eps) * weight`` (float); returns the new residual in ``out_dtype``
-        (the residual itself if that is float32)."""
+    def norm_add_pair(self, residual, terms, weight, eps, out_dtype):
+        """``m = sum_i factor_i * rms(y_i) * gain_i`` over the two ``terms`` ``(y, factor, gain, eps)`` and ``residual += rms(m) *
+        weight`` (float); returns the new residual in ``out_dtype`` (the residual itself if that is float32)."""
+        n, hidden = residual.shape
+        self._want(residual, "residual", torch.float32)
+        self._want(weight, "norm weight", torch.float32, (hidden,))
+        lowered = None if out_dtype == torch.float32 else torch.empty((n, hidden), dtype=out_dtype, device=residual.device)
+        self._norm_pair(residual, terms, weight, eps, lowered, n, hidden, out_dtype)
+        return residual if lowered is None else lowered
+
+    def _norm_pair(self, residual, terms, weight, eps, lowered, n, hidden, dtype):
+        if dtype not in _DT or len(terms) != 2:
+            raise KernelError(f"two normed results of float32 or bfloat16 are summed, got {len(terms)} of {dtype}")
+        for y, _, gain, _ in terms:
+            self._want(y, "result", dtype, (n, hidden))
+            self._want(gain, "result's norm weight", torch.float32, (hidden,))
+        (y1, f1, g1, e1), (y2, f2, g2, e2) = terms
+        self._check(self.core.sia_norm_pair(
+            _ptr(residual), _ptr(y1), _ptr(g1), float(f1), float(e1), _ptr(y2), _ptr(g2), float(f2), float(e2), _ptr(weight),
+            float(eps), _ptr(lowered), n, hidden, _DT[dtype], self._stream()), "norm_pair")
+
+    def normed_sum(self, terms):
+        """``sum_i factor_i * rms(y_i) * gain_i`` over ``(y, factor, gain, eps)`` terms, rounded to the results' type."""
+        terms = list(terms)
+        y0 = terms[0][0]
+        if len(terms) % 2:      # two at a time: a lone term has itself with a factor of zero beside it
+            terms.append((terms[-1][0], 0.0, terms[-1][2], terms[-1][3]))
+        outs = []
+        for i in range(0, len(terms), 2):
+            out = torch.empty_like(y0)
+            self._norm_pair(None, terms[i:i + 2], None, 0.0, out, y0.shape[0], y0.shape[1], y0.dtype)
+            outs.append((out, 1.0))
+        return outs[0][0] if len(outs) == 1 else self.scaled_sum(outs)
+
+    def norm_add(self, residual, y, weight, eps, out_dtype, bias=None):
+        """``residual += y * rsqrt(mean(y^2) + eps) * weight`` (float, ``y + bias`` for ``y`` if a bias is given); returns
+        the new residual in ``out_dtype`` (the residual itself if that is float32)."""
         n, hidden = residual.shape
         self._want(residual, "residual", torch.float32)
         self._want(weight, "norm weight", torch.float32, (hidden,))
         if out_dtype not in _DT:
             raise KernelError(f"norm output dtype {out_dtype} is not float32 or bfloat16")
         self._want(y, "sublayer output", out_dtype, (n, hidden))
+        if bias is not None:
+            self._want(bias, "sublayer bias", torch.float32, (hidden,))
         lowered = None if out_dtype == torch.float32 else torch.empty((n, hidden), dtype=out_dtype, device=residual.device)
         self._check(self.core.sia_norm_add(_ptr(residual), _ptr(y), _ptr(weight), _ptr(lowered), n, hidden, float(eps),
-                                           _DT[out_dtype], self._stream()), "norm_add")
+                                           _ptr(bias), _DT[out_dtype], self._stream()), "norm_add")
         return residual if lowered is None else lowered
 
     # -- residual add (of a result, or of its rms norm) + layer norm -----------------
@@ -698,12 +782,13 @@ class HipKernels:
             raise KernelError(f"head sizes {key_dim} x {value_dim} are outside what the recurrent kernel takes (up to {limit})")
 
     # -- mixture of experts ------------------------------------------------------------
-    def moe_route(self, h, router, top, score="softmax", groups=None, scale=1.0, correction=None):
+    def moe_route(self, h, router, top, score="softmax", groups=None, scale=1.0, correction=None, bias=None):
         """The ``top`` experts of every row with the largest router logits ``h @ router^T`` (float; ties go to the
         lower index) and the softmax over their logits alone: ``(ids [n, top] int32, weights [n, top] float32)``.
         ``score="sigmoid"``: the scores are the logits' sigmoids; with ``groups = (count, keep)`` only experts of the
         ``keep`` groups (of ``count`` equal groups of neighbours) whose two largest scores sum highest can be chosen;
-        the weights are the chosen scores over their sum, times ``scale``."""
+        the weights are the chosen scores over their sum, times ``scale``.  ``bias`` (softmax scores): a float per expert
+        added to the logits."""
         if score not in ("softmax", "sigmoid", "softmax_all"):
             raise KernelError(f"score must be 'softmax', 'sigmoid' or 'softmax_all', got {score!r}")
         if correction is not None and score != "softmax_all":
@@ -723,6 +808,13 @@ class HipKernels:
             raise KernelError(f"{experts} experts in {count} groups of which {keep} are kept cannot give {top}")
         if not 0 < top <= experts:
             raise KernelError(f"top {top} is not between 1 and the number of experts {experts}")
+        if bias is not None:
+            if score != "softmax":
+                raise KernelError("a bias of the logits comes with softmax scores over the chosen")
+            self._want(bias, "router bias", torch.float32, (experts,))
+            self._check(self.core.sia_moe_route_biased(_ptr(h), _ptr(router), _ptr(bias), _ptr(ids), _ptr(weights), n, width,
+                                                       experts, int(top), _DT[h.dtype], self._stream()), "moe_route")
+            return ids, weights
         if score == "softmax_all":
             # scores: the softmax over all experts; the choice goes by score + correction, the weights by the scores
             if correction is not None:
@@ -774,13 +866,127 @@ class HipKernels:
 
     # -- short convolution and recurrences with a state --------------------------------------
     def _state_rows(self, state, ctx, least):
+        """Floats from one slot's row to the next.  The rows may be a run of columns of wider ones (a mixer that shares
+        its row with another)."""
         if state is None:
             raise KernelError("a mixer with a state needs its state rows")
-        self._want(state, "state", torch.float32)
-        stride = state[0].numel()
-        if stride < least:
-            raise KernelError(f"a state row of {stride} floats does not hold {least}")
-        return stride
+        if state.device.type != "cuda" or state.dtype != torch.float32:
+            raise KernelError(f"state must be float32 on the GPU, is {state.dtype} on {state.device}")
+        row = state[0]
+        if not row.is_contiguous():
+            raise KernelError("a state row must be contiguous")
+        if row.numel() < least:
+            raise KernelError(f"a state row of {row.numel()} floats does not hold {least}")
+        return max(state.stride(0), row.numel())
+
+    def check_linear_unit(self, block: int, taps: int) -> None:
+        limit = self.core.sia_linear_unit_max_taps()
+        if not (block > 0 and 0 < taps <= limit):
+            raise KernelError(f"blocks of {block} behind a convolution of {taps} taps are outside what the kernel takes "
+                              f"(up to {limit} taps)")
+
+    def linear_unit(self, proj, y_col, x_col, terms, blocks, ctx, state):
+        """The linear recurrent unit between its products, over the step's runs of tokens.  ``proj`` (perhaps columns of a
+        wider matrix) holds the two branches at ``y_col`` and ``x_col``; ``terms``: y_bias, x_bias, conv ``[taps, width]``,
+        conv_bias, ra, ri ``[blocks, size, size]``, ra_bias, ri_bias, rate ``[width]``.  The state rows hold the unit's
+        ``width`` floats and behind them the convolution's ring of ``taps`` rows.  Returns ``[tokens, width]``."""
+        conv = terms["conv"]
+        taps, width = conv.shape
+        n = proj.shape[0]
+        stride = self._columns(proj, "projected rows", proj.dtype, tuple(proj.shape))
+        if proj.dtype not in _DT or n != ctx.n_tokens or min(y_col, x_col) < 0 or max(y_col, x_col) + width > proj.shape[1]:
+            raise KernelError(f"projected rows {proj.dtype} {tuple(proj.shape)} do not hold two branches of {width} at {y_col} "
+                              f"and {x_col} for {ctx.n_tokens} tokens")
+        size = width // blocks
+        for name in ("y_bias", "x_bias", "conv_bias", "ra_bias", "ri_bias", "rate"):
+            self._want(terms[name], name, torch.float32, (width,))
+        self._want(conv, "convolution weight", torch.float32)
+        for name in ("ra", "ri"):
+            self._want(terms[name], name, proj.dtype, (blocks, size, size))
+        self.check_linear_unit(size, taps)
+        row = self._state_rows(state, ctx, width * (1 + (taps if taps > 1 else 0)))
+        out = torch.empty((n, width), dtype=proj.dtype, device=proj.device)
+        workspace = self._float_workspace(ctx, self.core.sia_linear_unit_workspace(n, ctx.n_seqs, width), proj.device)
+        self._check(self.core.sia_linear_unit(
+            _ptr(proj), stride, int(y_col), int(x_col), _ptr(terms["y_bias"]), _ptr(terms["x_bias"]), _ptr(conv),
+            _ptr(terms["conv_bias"]), _ptr(terms["ra"]), _ptr(terms["ra_bias"]), _ptr(terms["ri"]), _ptr(terms["ri_bias"]),
+            _ptr(terms["rate"]), _ptr(state), row, _ptr(ctx.positions), _ptr(ctx.seq_of_token), _ptr(ctx.cu_q),
+            _ptr(ctx.state_slots), _ptr(out), n, ctx.n_seqs, ctx.max_q_len, width, blocks, taps, _DT[proj.dtype],
+            _ptr(workspace), self._stream()), "linear_unit")
+        return out
+
+    # -- a matrix state with a bonus for the current token ---------------------------------
+    def token_shift(self, h, mu, ctx, state, state_offset):
+        """``out[s, n] = h[n] + (h[n - 1] - h[n]) * mu[s]``, the row before a sequence's first token of the step taken from
+        its state row at ``state_offset`` (and the step's last row left there)."""
+        self._want(h, "rows")
+        n, width = h.shape
+        if h.dtype not in _DT or n != ctx.n_tokens:
+            raise KernelError(f"rows {h.dtype} {tuple(h.shape)} do not fit a step of {ctx.n_tokens} tokens")
+        self._want(mu, "mixture weights", torch.float32, (mu.shape[0], width))
+        stride = self._state_rows(state, ctx, state_offset + width)
+        out = torch.empty((mu.shape[0], n, width), dtype=h.dtype, device=h.device)
+        self._check(self.core.sia_token_shift(
+            _ptr(h), _ptr(mu), mu.shape[0], _ptr(state), stride, int(state_offset), _ptr(ctx.cu_q), _ptr(ctx.seq_of_token),
+            _ptr(ctx.state_slots), _ptr(out), n, width, _DT[h.dtype], self._stream()), "token_shift")
+        return out
+
+    def grouped_linear(self, x, w, rows):
+        """Products of groups of rows of ``w`` with inputs of their own: ``x [G, M, K]``, every group but the last ``rows``
+        rows tall.  Returns ``([G - 1, M, rows], [M, last])``; for few rows in bfloat16 one launch makes them all."""
+        self._want(x, "grouped inputs")
+        groups, M, K = x.shape
+        last = w.shape[0] - (groups - 1) * rows
+        self._want(w, "grouped weights", x.dtype, (w.shape[0], K))
+        if groups < 2 or rows <= 0 or last <= 0 or x.dtype not in _DT:
+            raise KernelError(f"{w.shape[0]} rows do not make {groups} groups of {rows} rows (the last one what is left)")
+        flat = torch.empty(((groups - 1) * M * rows + M * last,), dtype=x.dtype, device=x.device)
+        most = (groups - 1) * M * rows
+        main, low = flat[:most].view(groups - 1, M, rows), flat[most:].view(M, last)
+        if self.use_skinny_gemm and x.dtype == torch.bfloat16 and M <= self._skinny_rows and K % 64 == 0:
+            self._check(self.core.sia_gemm_skinny_grouped(_ptr(x), _ptr(w), _ptr(flat), M, K, groups, rows, last,
+                                                          self._stream()), "gemm_skinny_grouped")
+            return main, low
+        for g in range(groups):
+            wg = w[g * rows:(g + 1) * rows] if g + 1 < groups else w[g * rows:]
+            self._product_into(x[g], wg, main[g] if g + 1 < groups else low)
+        return main, low
+
+    def _product_into(self, x, w, y):
+        M, K = x.shape
+        N = w.shape[0]
+        if x.dtype == torch.float32:
+            self._check(self.core.sia_gemm_generic(_ptr(x), _ptr(w), _ptr(y), M, N, K, 0, 1, self._stream()), "gemm_generic")
+        elif self.blas is None or self.blas.sia_blas_mm(_ptr(x), _ptr(w), _ptr(y), M, N, K, 0, self._stream()) != 0:
+            torch.mm(x, w.t(), out=y)
+
+    def bonus_recurrence(self, rkvg, low, w2, w0, u, norm_weight, n_heads, head_dim, eps, ctx, state):
+        """``rkvg [4, tokens, heads * head_dim]``: r, k, v and the output gate; ``low [tokens, rank]``.  Decays ``exp(-exp(w2
+        tanh(low) + w0))`` in float; per head ``o = (S + diag(u) k v^T)^T r``, then ``S <- diag(decay) S + k v^T``; every head's
+        ``o`` is divided by its root mean square, multiplied by ``norm_weight [heads * head_dim]`` and by ``silu(gate)``.  The
+        matrices ``[heads, head_dim, head_dim]`` are the first floats of a sequence's state row."""
+        self._want(rkvg, "projected rows")
+        n, inner = ctx.n_tokens, n_heads * head_dim
+        if rkvg.dtype not in _DT or tuple(rkvg.shape) != (4, n, inner):
+            raise KernelError(f"projected rows {rkvg.dtype} {tuple(rkvg.shape)} are not [4, {n}, {inner}]")
+        rank = w2.shape[1]
+        self._want(low, "low-rank rows", rkvg.dtype, (n, rank))
+        self._want(w2, "decay matrix", rkvg.dtype, (inner, rank))
+        for t, what in ((w0, "decay bias"), (u, "bonus"), (norm_weight, "output norm weight")):
+            self._want(t, what, torch.float32, (inner,))
+        self.check_recurrent_geometry(head_dim, head_dim)
+        stride = self._state_rows(state, ctx, inner * head_dim)
+        out = torch.empty((n, inner), dtype=rkvg.dtype, device=rkvg.device)
+        decays = n * inner + (-n * inner) % 4
+        workspace = self._float_workspace(ctx, decays + self.core.sia_bonus_recurrence_workspace(n, n_heads, head_dim), rkvg.device)
+        raw = workspace[decays:]
+        self._check(self.core.sia_low_rank_decay(_ptr(low), rank, rank, _ptr(w2), _ptr(w0), inner, _ptr(workspace), n,
+                                                 _DT[rkvg.dtype], self._stream()), "low_rank_decay")
+        self._check(self.core.sia_bonus_recurrence(
+            _ptr(rkvg), _ptr(workspace), _ptr(u), _ptr(norm_weight), _ptr(state), stride, _ptr(ctx.cu_q),
+            _ptr(ctx.state_slots), _ptr(out), n, ctx.n_seqs, ctx.max_q_len, n_heads, head_dim, float(eps), _DT[rkvg.dtype],
+            _ptr(raw), self._stream()), "bonus_recurrence")
+        return out
 
     def _float_workspace(self, ctx, floats, device):
         workspace = getattr(ctx, "recurrent_workspace", None)
@@ -1067,13 +1273,13 @@ class HipKernels:
     def _glu(activation):
         """(kind, limit) of a gated activation as the kernels take it: None is ``silu(g) * u``, ``("clamped", limit)`` is
         ``g * sigmoid(1.702 g) * (u + 1)`` with ``g = min(g, limit)`` and ``u = clamp(u, -limit, limit)``, ``("relu",
-        None)`` is ``max(g, 0) * u``."""
+        None)`` is ``max(g, 0) * u``, ``("gelu_tanh", None)`` is ``gelu(g) * u`` in the tanh form."""
         if activation is None:
             return _GLUS["silu"], 0.0
         kind, limit = activation
-        if kind == "relu" and limit is None:
-            return _GLUS["relu"], 0.0
-        if kind not in _GLUS or not float(limit) > 0:
+        if kind in ("relu", "gelu_tanh") and limit is None:
+            return _GLUS[kind], 0.0
+        if kind not in _GLUS or limit is None or not float(limit) > 0:
             raise KernelError(f"gated activation {activation!r} is not one of {', '.join(_GLUS)} with a positive limit")
         return _GLUS[kind], float(limit)
 
@@ -1082,14 +1288,18 @@ class HipKernels:
         """``sum_k weights[n, k] * expert_{ids[n, k]}(h[n])`` with ``expert_e(x) = W2_e (silu(Wg_e x) * (Wu_e x))``,
         ``w_gate_up [E, 2 ff, width]`` (gate rows first), ``w_down [E, width, ff]``; plus ``shared`` ``[n, width]``
         (times ``sigmoid(shared_gate [n, 1])`` if given), the sum rounded once.  ``activation``: another gated
-        activation than ``silu(g) * u`` (see ``_glu``); ``identity``: ids ``E .. E + identity - 1`` name experts
+        activation than ``silu(g) * u`` (see ``_glu``), or the name of an activation without a gate (``w_gate_up`` is then ``[E, ff,
+        width]`` and an expert ``W2 act(Wu x)``); ``identity``: ids ``E .. E + identity - 1`` name experts
         without tensors, which return their input."""
-        glu, limit = self._glu(activation)
+        gated = not isinstance(activation, str)
+        if not gated and activation not in _ACTIVATIONS:
+            raise KernelError(f"activation {activation!r} is not one of {', '.join(_ACTIVATIONS)}")
+        glu, limit = self._glu(activation) if gated else (_UNGATED + _ACTIVATIONS[activation], 0.0)
         self._want(h, "expert input")
         n, width = h.shape
         experts, two_ff, _ = w_gate_up.shape
-        ff, top = two_ff // 2, ids.shape[1]
-        self._want(w_gate_up, "expert gate/up weights", h.dtype, (experts, 2 * ff, width))
+        ff, top = two_ff // (2 if gated else 1), ids.shape[1]
+        self._want(w_gate_up, "expert gate/up weights", h.dtype, (experts, (2 if gated else 1) * ff, width))
         self._want(w_down, "expert down weights", h.dtype, (experts, width, ff))
         self._want(ids, "expert ids", torch.int32, (n, top))
         self._want(weights, "expert weights", torch.float32, (n, top))
@@ -1160,12 +1370,17 @@ class HipKernels:
             y = self.cast(y, back)
         return y
 
-    def gated_linear(self, x, w_gate_up, activation=None):
+    def gated_linear(self, x, w_gate_up, activation=None, bias=None):
         """``silu(x Wg^T) * (x Wu^T)`` for ``w_gate_up = [Wg; Wu]``: one kernel for few rows, else product + SwiGLU.
-        ``activation``: another gated activation (see ``_glu``), by the product and a kernel of its own."""
+        ``activation``: another gated activation (see ``_glu``), by the product and a kernel of its own; ``bias`` (with such
+        an activation): float, one per row of ``w_gate_up``, added to the product in front of the activation."""
         self._want(w_gate_up, "gate/up weight")
         M, K = x.shape
         two_i = w_gate_up.shape[0]
+        if bias is not None:
+            self._want(bias, "gate/up bias", torch.float32, (two_i,))
+            if activation is None:
+                raise KernelError("the silu gate has no biases")
         if activation is not None:
             glu, limit = self._glu(activation)
             if (self.use_skinny_gemm and x.dtype == torch.bfloat16 and w_gate_up.dtype == torch.bfloat16
@@ -1174,7 +1389,7 @@ class HipKernels:
                 self._want(rows, "gated linear input")
                 y = torch.empty((M, two_i // 2), dtype=torch.bfloat16, device=rows.device)
                 self._check(self.core.sia_gemm_skinny_glu(_ptr(rows), _ptr(w_gate_up), _ptr(y), M, two_i // 2, K,
-                                                          _ptr(partials), n_partials, eps, glu, limit, self._stream()),
+                                                          _ptr(partials), n_partials, eps, glu, limit, _ptr(bias), self._stream()),
                             "gemm_skinny_glu")
                 return y
             gu = self.linear(x, w_gate_up)
@@ -1184,7 +1399,7 @@ class HipKernels:
             for n0 in range(0, M, 65535):
                 n1 = min(M, n0 + 65535)
                 self._check(self.core.sia_glu(_ptr(gu[n0:n1]), _ptr(out[n0:n1]), n1 - n0, two_i // 2, glu, limit,
-                                              _DT[gu.dtype], self._stream()), "glu")
+                                              _ptr(bias), _DT[gu.dtype], self._stream()), "glu")
             return out
         if (self.use_skinny_gemm and x.dtype == torch.bfloat16 and w_gate_up.dtype == torch.bfloat16
                 and M <= self._skinny_rows and two_i % 2 == 0 and K % 64 == 0 and w_gate_up.shape[1] == K):
@@ -1520,6 +1735,64 @@ class HipKernels:
             _ptr(v_pages), n, n_heads, n_kv_written, head_dim, value_dim, rotary_dim, page_size, k_row, v_rows,
             _ptr(q_out), n_heads * page_dim if page_dim else 0, page_dim or 0, temp_coef, temp_every,
             int(bool(values_are_keys)), _ptr(given), given_stride, _ptr(mix), _DT[qkv.dtype], self._stream()), "qk_prepare")
+
+    def check_row_prepare(self, n_heads, n_kv_heads, head_dim, taps) -> None:
+        """Raises for rows that ``row_prepare`` does not take (q and k of a token meet in LDS)."""
+        limit, taps_limit = self.core.sia_row_prepare_max_elements(), self.core.sia_linear_unit_max_taps()
+        if (n_heads + n_kv_heads) * head_dim > limit or not 0 < taps <= taps_limit:
+            raise KernelError(f"{n_heads} + {n_kv_heads} heads of {head_dim} behind {taps} taps are outside what the kernel "
+                              f"takes (up to {limit} elements and {taps_limit} taps)")
+
+    def row_prepare(self, proj, columns, n_heads, n_kv, head_dim, value_dim, rotary_dim, cos, sin, pairing, bias, conv, norm,
+                    page_dim, ctx, cache):
+        """What lies between the q/k/v product and attention where a token's whole row is needed at once: bias, a causal
+        convolution per channel (``conv [taps, channels]``, its last inputs in ``cache.state`` as a ring of ``taps`` rows), an
+        RMS norm of q and k over the row or per head (``norm = (q_gain, k_gain, eps, "row" or "head")``), the rotation with
+        neighbours or halves paired, and the write of k and v into the pages.  ``proj`` (perhaps columns of a wider matrix)
+        holds q, k and v at ``columns``.  Returns ``[tokens, n_heads * (page_dim or head_dim)]``: the queries, zeros behind
+        every head where the pages are wider."""
+        n = proj.shape[0]
+        stride = self._columns(proj, "projected rows", proj.dtype, tuple(proj.shape))
+        if proj.dtype not in _DT or n != ctx.n_tokens:
+            raise KernelError(f"projected rows {proj.dtype} {tuple(proj.shape)} do not fit a step of {ctx.n_tokens} tokens")
+        sizes = (n_heads * head_dim, n_kv * head_dim, n_kv * value_dim)
+        for col, size in zip(columns, sizes):
+            if col < 0 or col + size > proj.shape[1]:
+                raise KernelError(f"columns {col} .. {col + size} lie outside a row of {proj.shape[1]}")
+        channels, taps = sum(sizes), 1
+        if bias is not None:
+            self._want(bias, "q/k/v bias", torch.float32, (channels,))
+        if conv is not None:
+            taps = conv.shape[0]
+            self._want(conv, "convolution weight", torch.float32, (taps, channels))
+        self.check_row_prepare(n_heads, n_kv, head_dim, taps)
+        state, row = None, 0
+        if taps > 1:
+            state = cache.state
+            row = self._state_rows(state, ctx, taps * channels)
+        q_gain = k_gain = None
+        eps, over = 0.0, "row"
+        if norm is not None:
+            q_gain, k_gain, eps, over = norm
+            want = sizes[:2] if over == "row" else (head_dim, head_dim)
+            self._want(q_gain, "q norm gain", torch.float32, (want[0],))
+            self._want(k_gain, "k norm gain", torch.float32, (want[1],))
+        if rotary_dim:
+            self._rotation_tables(rotary_dim, cos, sin, ctx.max_kv_len)
+        if pairing not in ("interleaved", "half"):
+            raise KernelError(f"pairing must be 'half' or 'interleaved', got {pairing!r}")
+        wide = page_dim or head_dim
+        v_rows = page_dim or value_dim
+        self._check_pages(cache.k_pages, cache.v_pages, cache.block_table, cache.page_size, n_kv, wide, proj.dtype, ctx, v_rows)
+        q = torch.empty((n, n_heads * wide), dtype=proj.dtype, device=proj.device)
+        self._check(self.core.sia_row_prepare(
+            _ptr(proj), stride, *(int(c) for c in columns), _ptr(bias), _ptr(conv), taps, _ptr(q_gain), _ptr(k_gain),
+            float(eps), int(over == "row"), _ptr(cos) if rotary_dim else None, _ptr(sin) if rotary_dim else None, rotary_dim,
+            int(pairing == "interleaved"), _ptr(ctx.positions), _ptr(ctx.seq_of_token), _ptr(ctx.cu_q), _ptr(ctx.state_slots),
+            _ptr(cache.block_table), cache.block_table.shape[1], _ptr(state), row, _ptr(cache.k_pages), _ptr(cache.v_pages),
+            _ptr(q), n, ctx.n_seqs, ctx.max_q_len, n_heads, n_kv, head_dim, value_dim, cache.page_size, wide, v_rows, wide,
+            _DT[proj.dtype], self._stream()), "row_prepare")
+        return q
 
     def _check_pages(self, k_pages, v_pages, table, page_size, n_kv, head_dim, dtype, ctx, value_dim=None):
         value_dim = value_dim or head_dim

@@ -42,7 +42,7 @@ HIPCC_FLAGS = [
 LIBRARIES: Dict[str, Sequence[str]] = {
     "core": ("elementwise.hip", "rope_cache.hip", "qk_prepare.hip", "attention_generic.hip", "gemm_generic.hip", "gemm_skinny.hip",
              "sampling.hip", "bandwidth.hip", "block.hip", "gated.hip", "recurrent.hip", "moe.hip", "dyt.hip", "conv.hip", "latent.hip",
-             "layernorm.hip", "lowrank.hip", "token_input.hip"),
+             "layernorm.hip", "lowrank.hip", "token_input.hip", "row_prepare.hip", "rglru.hip", "token_shift.hip"),
     # the vendor's BLAS library called directly (the products of steps of many tokens); optional: without it those
     # products go through torch
     "blas": ("library_product.hip",),

@@ -146,6 +146,9 @@ class Attention:
         check = getattr(env.kernels, "check_attention_geometry", None)
         if check is not None:     # sizes the kernels refuse are refused here, when the model is built
             check(self.num_heads, self.num_kv_heads, max(self.head_dim, self.value_dim))
+        check = getattr(env.kernels, "check_row_prepare", None)
+        if check is not None and self.row_form:
+            check(self.num_heads, self.num_kv_heads, self.head_dim, self.conv_taps or 1)
         # kernels that want keys and values of one width say at which width this mixer should keep its pages
         page_dim = getattr(env.kernels, "attention_page_dim", None)
         self.page_dim = page_dim(self.head_dim, self.value_dim, env.dtype) if page_dim is not None and self._options() else None
@@ -232,7 +235,7 @@ class Attention:
             self.row_columns, stacked = tuple(columns), parts
         self.w_qkv = torch.cat(stacked, dim=0).contiguous()
         if self.conv_taps is not None:
-            self.conv_w = torch.cat([tensors[n] for n in ("q_conv", "k_conv", "v_conv")], dim=0).float().contiguous()
+            self.conv_w = torch.cat([tensors[n] for n in ("q_conv", "k_conv", "v_conv")], dim=0).float().t().contiguous()   # [taps, channels]
         self.w_o = tensors["o"].contiguous()
         if self.page_dim is not None and not self.element_gate:
             # the attention's rows come with page_dim elements a head: zero columns for the rest (the elements' gate

@@ -62,7 +62,7 @@ class LinearRecurrentUnit:
         self.w_o = tensors["o"].contiguous()
         f32 = lambda n: tensors[n].float().reshape(-1).contiguous()
         self.terms = {
-            "y_bias": f32("y_bias"), "x_bias": f32("x_bias"), "conv": tensors["conv"].float().contiguous(),
+            "y_bias": f32("y_bias"), "x_bias": f32("x_bias"), "conv": tensors["conv"].float().t().contiguous(),
             "conv_bias": f32("conv_bias"), "ra": tensors["ra"].contiguous(), "ri": tensors["ri"].contiguous(),
             "ra_bias": f32("ra_bias"), "ri_bias": f32("ri_bias"),
             "rate": RATE * torch.nn.functional.softplus(tensors["lam"].double(), threshold=1e9).float().contiguous(),

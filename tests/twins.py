@@ -327,8 +327,9 @@ class TwinKernels:
     # -- a state beside pages, recurrences with inputs of their own -------------------------
     @staticmethod
     def _ring_conv(u, weight, ctx, ring):
-        """Causal convolution of ``u [n, channels]`` (float) whose last inputs lie in ``ring [slots, taps, channels]``."""
-        channels, taps = weight.shape
+        """Causal convolution of ``u [n, channels]`` (float) whose last inputs lie in ``ring [slots, taps, channels]``;
+        ``weight [taps, channels]``."""
+        taps, channels = weight.shape
         out = torch.zeros_like(u)
         cu, slots, pos = ctx.cu_q.tolist(), ctx.state_slots.tolist(), ctx.positions.tolist()
         for s in range(ctx.n_seqs):
@@ -338,7 +339,7 @@ class TwinKernels:
             past = [ring[slots[s], (first - i) % taps].clone() if first - i >= 0 else torch.zeros(channels)
                     for i in range(taps - 1, 0, -1)]
             seq = torch.cat([torch.stack(past), u[cu[s]:cu[s + 1]]]) if past else u[cu[s]:cu[s + 1]]
-            out[cu[s]:cu[s + 1]] = sum(seq[j:j + n] * weight[:, j].float() for j in range(taps))
+            out[cu[s]:cu[s + 1]] = sum(seq[j:j + n] * weight[j].float() for j in range(taps))
             for i in range(max(0, n - taps + 1), n):
                 if taps > 1:
                     ring[slots[s], (first + i) % taps] = u[cu[s] + i]
@@ -352,7 +353,7 @@ class TwinKernels:
         if bias is not None:
             u = u + bias.float()
         if conv is not None:
-            ring = cache.state.view(cache.state.shape[0], conv.shape[1], -1) if conv.shape[1] > 1 else None
+            ring = cache.state.unflatten(1, (conv.shape[0], -1)) if conv.shape[0] > 1 else None
             u = self._ring_conv(u, conv, ctx, ring)
         q, k, v = u.split(sizes, dim=1)
         rows = {"q": (q, n_heads), "k": (k, n_kv)}
@@ -374,10 +375,10 @@ class TwinKernels:
         return out.view(n, n_heads * wide)
 
     def linear_unit(self, proj, y_col, x_col, terms, blocks, ctx, state):
-        width, taps = terms["conv"].shape
+        taps, width = terms["conv"].shape
         bs, dtype = width // blocks, proj.dtype
         x = proj[:, x_col:x_col + width].float() + terms["x_bias"]
-        ring = state[:, width:width * (1 + taps)].view(state.shape[0], taps, width) if taps > 1 else None
+        ring = state[:, width:width * (1 + taps)].unflatten(1, (taps, width)) if taps > 1 else None
         u = (self._ring_conv(x, terms["conv"], ctx, ring) + terms["conv_bias"]).to(dtype).float()
         parts = u.view(-1, blocks, bs)
         gate = lambda w, b: torch.sigmoid(torch.einsum("nbi,boi->nbo", parts, w.float()).reshape(u.shape) + b)
