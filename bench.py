@@ -33,6 +33,8 @@ layers with routed experts and the Llama model.
 windowed attention beside a decaying linear attention, both with clamped experts, beside the same two models.
 ``--workload lunerax`` does the same for the Lunerax design: a model of each of its three mixers and one of its attention
 with a short window, with dense feed-forwards, beside the Tadinex delta rule, the Famepel latent attention and the Llama model.
+``--workload melerax`` does the same for the Melerax design: a model of each of its three mixers beside the Tadinex model of
+layers with two mixers side by side, the Mogisun model of linear-attention layers, the Lunerax attention and the Llama model.
 
 The engine runs on one GPU; asked for more it says so and exits with 2.
 """
@@ -85,12 +87,13 @@ def parse_args(argv=None):
     ap.add_argument("--temperature", type=float, default=0.0, help="sampling of the decode measurement (0: greedy)")
     ap.add_argument("--top-k", type=int, default=0)
     ap.add_argument("--top-p", type=float, default=1.0)
-    ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "shared-prefix", "feduzen", "mogisun", "famepel", "tadinex", "lunerax"])
+    ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "shared-prefix", "feduzen", "mogisun", "famepel", "tadinex", "lunerax", "melerax"])
     ap.add_argument("--shapes", default="1b,3b,8b", help="--workload feduzen: which layer sizes, comma separated")
-    ap.add_argument("--models", default=None, help="--workload feduzen, mogisun, famepel, tadinex or lunerax: which of the models to run "
+    ap.add_argument("--models", default=None, help="--workload feduzen, mogisun, famepel, tadinex, lunerax or melerax: which of the models to run "
                     "(feduzen,llama; mogisun-attention,mogisun-linear,llama; famepel-ssm,famepel-hgrn,famepel-latent,"
                     "mogisun-linear,llama; tadinex-delta,tadinex-parallel,mogisun-linear,llama; "
-                    "lunerax-delta,lunerax-latent,lunerax-attention,lunerax-window,tadinex-delta,famepel-latent,llama)")
+                    "lunerax-delta,lunerax-latent,lunerax-attention,lunerax-window,tadinex-delta,famepel-latent,llama; "
+                    "melerax-parallel,melerax-wkv,melerax-rglru,tadinex-parallel,mogisun-linear,lunerax-attention,llama)")
     ap.add_argument("--max-running", type=int, default=64, help="request slots of the stream workloads")
     return ap.parse_args(argv)
 
@@ -656,6 +659,67 @@ def lunerax_workload(args):
     return 0
 
 
+def melerax_config_like(llama_cfg, layers, kind):
+    """A Melerax config.json with the width, head count, head width and feed-forward size of a Llama one.  ``parallel``: the
+    Llama model's attention heads behind convolutions of four taps, capped scores, a block of positions wider than the
+    measured context (so that the attention does the other models' work), beside a linear unit of the model's width in
+    as many parts as there are heads, and a dense gated feed-forward of the Llama size.  ``wkv``: heads of 64 that fill the
+    width, a decay pair of rank 64; ``rglru``: the linear unit alone; both with eight experts of a quarter of the
+    feed-forward size, two a token, and a shared expert of half of it, none of them gated."""
+    dim, heads, width = llama_cfg["head_dim"], llama_cfg["num_attention_heads"], llama_cfg["hidden_size"]
+    ff = llama_cfg["intermediate_size"]
+    unit = {"width": width, "blocks": heads, "conv": 4}
+    mlp = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 2}}
+    if kind == "parallel":
+        mixer = {"type": "parallel", "mixer": {"right": unit, "left": {
+            "conv": 4, "dim": dim, "heads": heads, "kv_heads": llama_cfg["num_key_value_heads"], "vdim": dim, "scale": dim ** -0.5,
+            "softcap": 30.0, "mask": {"size": 1 << 20}, "rot": {"base": llama_cfg["rope_theta"], "dims": dim}}}}
+        mlp = {"kind": "dense", "ff": ff}
+    elif kind == "wkv":
+        mixer = {"type": "wkv", "mixer": {"dim": 64, "heads": width // 64, "decay_rank": 64}}
+    else:
+        mixer = {"type": "rglru", "mixer": unit}
+    return {"architecture": "Melerax", "vocab": llama_cfg["vocab_size"], "width": width,
+            "norm": {"eps": llama_cfg["rms_norm_eps"]},
+            "embedding": {"bigram": {"buckets": 65521, "mul_cur": 31, "mul_prev": 1009}},
+            "layers": [json.loads(json.dumps(dict(mixer, mlp=mlp))) for _ in range(layers)]}
+
+
+def melerax_workload(args):
+    """Decode and prefill of the Melerax design (each of its three mixers alone) beside the closest models' layers at equal
+    sizes: the Tadinex layer of two mixers side by side, the Mogisun linear attention (both with routed experts), the
+    Lunerax attention with capped scores and the Llama model."""
+    layers = args.layers or 8
+    dt_name = "bf16" if args.dtype == "bfloat16" else "fp32"
+    names = "melerax-parallel,melerax-wkv,melerax-rglru,tadinex-parallel,mogisun-linear,lunerax-attention,llama"
+    out = measure_beside(args, lambda llama, n: (("melerax-parallel", melerax_config_like(llama, n, "parallel")),
+                                                 ("melerax-wkv", melerax_config_like(llama, n, "wkv")),
+                                                 ("melerax-rglru", melerax_config_like(llama, n, "rglru")),
+                                                 ("tadinex-parallel", tadinex_config_like(llama, n, "parallel")),
+                                                 ("mogisun-linear", mogisun_config_like(llama, n, "linear")),
+                                                 ("lunerax-attention", lunerax_config_like(llama, n, "attention")),
+                                                 ("llama", llama)), (args.models or names).split(","))
+    line = {"metric": "Melerax beside Tadinex, Mogisun, Lunerax and Llama at equal layer sizes: decode tok/s (batch 8, 1) and "
+                      "prefill tok/s",
+            "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "dtype": dt_name,
+            "data": "synthetic (seeded random weights and uniform-random token ids)",
+            "config": {"layers": layers, "context": args.context, "prefill_tokens": args.prefill_tokens,
+                       "shapes": FEDUZEN_SHAPES,
+                       "melerax-*": "norms behind the sublayers, layer scales, an embedding of token pairs",
+                       "melerax-parallel": "the Llama model's attention heads (4 taps, row norms, capped scores, block beyond "
+                                           "the context) beside a linear unit of the width, dense gated feed-forward",
+                       "melerax-wkv": "matrix state of heads of 64 with a bonus, 8 ungated experts of ff/4, 2 a token, a shared "
+                                      "one of ff/2",
+                       "melerax-rglru": "linear unit of the width, the same experts",
+                       "tadinex-parallel": "windowed attention beside a decaying linear attention, 8 clamped experts of ff/4 "
+                                           "and 2 identity experts, 2 a token, a shared one of ff/2",
+                       "mogisun-linear": "gated linear attention, 8 experts of ff/4 (2 a token) and a shared one of ff/2",
+                       "lunerax-attention": "the Llama model's heads without rotation, capped scores, gate per element, dense"},
+            "shapes": out}
+    print(json.dumps(line), flush=True)
+    return 0
+
+
 def further_points(args, pts, config, layer_w, head_w, el):
     """What the headline leaves out, at sizes a server meets: the same model with contexts of 8,192 and 32,768 tokens
     and a prompt of 8,192 (an engine of its own with a context limit of 33,792), and the two request streams of the
@@ -732,6 +796,8 @@ def main(argv=None):
         return tadinex_workload(args)
     if args.workload == "lunerax":
         return lunerax_workload(args)
+    if args.workload == "melerax":
+        return melerax_workload(args)
     if args.workload != "decode":
         return stream_workload(args)
     points = [int(p) for p in args.points.split(",") if p]

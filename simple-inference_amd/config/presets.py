@@ -72,6 +72,17 @@ def _lunerax_layer(kind):
     return {"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": 1536}}
 
 
+def _melerax_layer(kind, mlp):
+    mixer = {"parallel": {"left": {"conv": 4, "dim": 64, "heads": 8, "kv_heads": 2, "vdim": 64, "scale": 0.125, "softcap": 20.0,
+                                   "mask": {"size": 256}, "rot": {"base": 100000.0, "dims": 32}},
+                          "right": {"width": 512, "blocks": 8, "conv": 4}},
+             "wkv": {"dim": 64, "heads": 8, "decay_rank": 32},
+             "rglru": {"width": 512, "blocks": 8, "conv": 4}}[kind]
+    return {"type": kind, "mixer": mixer, "mlp": mlp}
+
+
+_MELERAX_EXPERTS = {"kind": "moe", "router": {"experts": 16, "top": 2}, "expert": {"ff": 512}, "shared": {"ff": 768}}
+
 PRESETS = {
     "llama-3.2-3b": {
         "architectures": ["LlamaForCausalLM"], "model_type": "llama",
@@ -139,6 +150,14 @@ PRESETS = {
         "token_side": {"dim": 64}, "logit_softcap": 25.0,
         "layers": [_lunerax_layer(kind) for kind in ("attention", "channel_delta", "channel_delta", "latent_attention",
                                                      "channel_delta", "channel_delta", "attention")],
+    },
+    # a small model of the Melerax design: a layer of attention beside a linear unit with a dense feed-forward, then two
+    # recurrent layers with routed experts, twice
+    "melerax-small": {
+        "architecture": "Melerax", "vocab": 4096, "width": 512, "norm": {"eps": 1e-6},
+        "embedding": {"bigram": {"buckets": 2048, "mul_cur": 31, "mul_prev": 1009}},
+        "layers": [_melerax_layer("parallel", {"kind": "dense", "ff": 1536}), _melerax_layer("wkv", _MELERAX_EXPERTS),
+                   _melerax_layer("rglru", _MELERAX_EXPERTS)] * 2,
     },
     "tiny-a": {
         "architectures": ["LlamaForCausalLM"], "model_type": "llama",

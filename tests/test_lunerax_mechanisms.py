@@ -29,7 +29,7 @@ def bind_part(part, g, dev, dtype, names, std=0.3, **fixed):
         given = fixed.get(name)
         shape = given if isinstance(given, (list, tuple)) else spec.shape
         t = given.double() if isinstance(given, torch.Tensor) else rnd(g, *shape, std=std) + (1.0 if name.endswith(("norm", "weight")) and spec.role == "vector" else 0.0)
-        bound[name], T[names.get(name, "m." + name)] = lowered(t, torch.float32 if spec.role == "vector" else dtype, dev)
+        bound[name], T[names.get(name, "m." + name)] = lowered(t, torch.float32 if spec.role in ("vector", "float_matrix") else dtype, dev)
     part.bind(bound)
     return T
 
