@@ -460,6 +460,7 @@ SIA_EXPORT int sia_gemm_skinny_grouped(const void* X, const void* W, void* Y, in
     Cut best{0, 0, 0, 0};
     int best_blocks = 0;
     for (int ub : {4, 2, 1})
+        // (where the workgroups are many, full blocks: lower ones would fetch X more often for the same rows)
         for (int bh = 16; bh >= 8; --bh) {
             const int a_group = (group_rows + ub * bh - 1) / (ub * bh), last = (last_rows + ub * bh - 1) / (ub * bh);
             const int grid = (groups - 1) * a_group + last;
@@ -468,6 +469,7 @@ SIA_EXPORT int sia_gemm_skinny_grouped(const void* X, const void* W, void* Y, in
                 best = c;
                 best_blocks = a_group;
             }
+            if (bh == 16 && grid > 2 * cus) break;
         }
     Epilogue ep{};
     ep.groups = groups;

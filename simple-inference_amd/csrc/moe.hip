@@ -371,7 +371,8 @@ __device__ __forceinline__ moe_bf16x8 moe_ld8(const bf16_t* p) { return *reinter
 
 // GATED: rows f and ff + f of W make silu(gate) * up; else a plain product, or with ``glu`` at MOE_UNGATED and beyond the
 // activation of it.  Output row stride n_out.
-template <bool GATED>
+// NB: blocks of 16 columns a wave takes.
+template <bool GATED, int NB>
 __global__ __launch_bounds__(256) void moe_tile_kernel(const bf16_t* __restrict__ x, int rows_per_slot,
                                                        const bf16_t* __restrict__ w, const int* __restrict__ place_slot,
                                                        const int* __restrict__ tile_expert,
@@ -381,42 +382,42 @@ __global__ __launch_bounds__(256) void moe_tile_kernel(const bf16_t* __restrict_
     if (tile >= *n_tiles) return;
     const int wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE, r = lane & 15, g = lane >> 4;
     const int e = tile_expert[tile];
-    const int c0 = blockIdx.y * 128 + wave * 32;          // this wave's 32 output columns
+    const int c0 = (blockIdx.y * 4 + wave) * NB * 16;     // this wave's output columns
     if (c0 >= n_out) return;
     const size_t expert_rows = GATED ? 2 * (size_t)n_out : (size_t)n_out;
     const bf16_t* we = w + (size_t)e * expert_rows * K;
     int slot[2];
     const bf16_t* xp[2];
-    const bf16_t* wp[2][2];
+    const bf16_t* wp[NB][2];
 #pragma unroll
     for (int mb = 0; mb < 2; ++mb) {
         slot[mb] = place_slot[tile * MOE_TILE + mb * 16 + r];
         xp[mb] = x + (size_t)(max(slot[mb], 0) / rows_per_slot) * K + g * 8;
     }
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb) {
+    for (int nb = 0; nb < NB; ++nb) {
         const int c = min(c0 + nb * 16 + r, n_out - 1);
         wp[nb][0] = we + (size_t)c * K + g * 8;
         wp[nb][1] = we + (size_t)(n_out + c) * K + g * 8;     // the up rows (GATED only)
     }
-    moe_floatx4 acc[2][2][2];
+    moe_floatx4 acc[NB][2][2];
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb)
+    for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
         for (int mb = 0; mb < 2; ++mb)
 #pragma unroll
             for (int h = 0; h < 2; ++h) acc[nb][mb][h] = moe_floatx4{0.f, 0.f, 0.f, 0.f};
     for (int k = 0; k < K; k += 32) {
-        moe_bf16x8 a[2][2], b[2];
+        moe_bf16x8 a[NB][2], b[2];
 #pragma unroll
         for (int mb = 0; mb < 2; ++mb) b[mb] = moe_ld8(xp[mb] + k);
 #pragma unroll
-        for (int nb = 0; nb < 2; ++nb) {
+        for (int nb = 0; nb < NB; ++nb) {
             a[nb][0] = moe_ld8(wp[nb][0] + k);
             if (GATED) a[nb][1] = moe_ld8(wp[nb][1] + k);
         }
 #pragma unroll
-        for (int nb = 0; nb < 2; ++nb)
+        for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
             for (int mb = 0; mb < 2; ++mb) {
                 acc[nb][mb][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[nb][0], b[mb], acc[nb][mb][0], 0, 0, 0);
@@ -430,7 +431,7 @@ __global__ __launch_bounds__(256) void moe_tile_kernel(const bf16_t* __restrict_
         if (slot[mb] < 0) continue;
         const size_t row = GATED ? (size_t)slot[mb] : (size_t)slot[mb];
 #pragma unroll
-        for (int nb = 0; nb < 2; ++nb) {
+        for (int nb = 0; nb < NB; ++nb) {
             const int c = c0 + nb * 16 + 4 * g;
             bf16_t v[4];
 #pragma unroll
@@ -500,15 +501,16 @@ SIA_EXPORT int sia_moe_tiled_ex(const void* h, const void* w1, const void* w2, c
     int* n_tiles = tile_expert + max_tiles;
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, ids, slots, n_experts, place_slot, tile_expert,
                        n_tiles, max_tiles);
+    // products without a gate: four blocks of columns a wave, as many products a load of the slots' rows as with one
     if (glu >= MOE_UNGATED)
-        hipLaunchKernelGGL(moe_tile_kernel<false>, dim3(max_tiles, (ff + 127) / 128), dim3(256), 0, stream,
+        hipLaunchKernelGGL((moe_tile_kernel<false, 4>), dim3(max_tiles, (ff + 255) / 256), dim3(256), 0, stream,
                            (const bf16_t*)h, top, (const bf16_t*)w1, place_slot, tile_expert, n_tiles, (bf16_t*)act, width,
                            ff, glu, limit);
     else
-        hipLaunchKernelGGL(moe_tile_kernel<true>, dim3(max_tiles, (ff + 127) / 128), dim3(256), 0, stream,
+        hipLaunchKernelGGL((moe_tile_kernel<true, 2>), dim3(max_tiles, (ff + 127) / 128), dim3(256), 0, stream,
                            (const bf16_t*)h, top, (const bf16_t*)w1, place_slot, tile_expert, n_tiles, (bf16_t*)act, width,
                            ff, glu, limit);
-    hipLaunchKernelGGL(moe_tile_kernel<false>, dim3(max_tiles, (width + 127) / 128), dim3(256), 0, stream,
+    hipLaunchKernelGGL((moe_tile_kernel<false, 4>), dim3(max_tiles, (width + 255) / 256), dim3(256), 0, stream,
                        (const bf16_t*)act, 1, (const bf16_t*)w2, place_slot, tile_expert, n_tiles, (bf16_t*)y, ff, width,
                        SIA_GLU_SILU, 0.f);
     hipLaunchKernelGGL(moe_combine_kernel, dim3(n_tokens), dim3(256), 0, stream, (const bf16_t*)y, weights,

@@ -511,12 +511,13 @@ static int launch_recurrence(const void* proj, int row_stride, int q_col, int k_
 // workspace and the token's own weighed write.  A wave a (token, head); q, k, v and g are columns of rows row_stride apart,
 // weights and bonus a head's own.
 template <typename T>
-__global__ __launch_bounds__(SIA_WAVE) void bonus_finish_kernel(const float* __restrict__ raw, const T* __restrict__ proj,
+__global__ __launch_bounds__(4 * SIA_WAVE) void bonus_finish_kernel(const float* __restrict__ raw, const T* __restrict__ proj,
                                                                 int row_stride, int q_col, int k_col, int v_col, int g_col,
                                                                 const float* __restrict__ bonus,
                                                                 const float* __restrict__ norm_w, T* __restrict__ out,
                                                                 int n_heads, int D, int Dv, float eps) {
-    const int n = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
+    const int n = blockIdx.x, head = blockIdx.y * 4 + threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE;
+    if (head >= n_heads) return;      // a wave leaves as a whole
     const T* row = proj + (size_t)n * row_stride;
     const T *q = row + q_col + head * D, *k = row + k_col + head * D, *v = row + v_col + head * Dv, *g = row + g_col + head * Dv;
     float own = 0.f;
@@ -559,7 +560,7 @@ SIA_EXPORT int sia_bonus_recurrence(const void* rkvg, const float* decays, const
                                        false, &raw, stream, bonus);
     if (code) return code;
     if (raw) {
-        dim3 grid(n_tokens, n_heads), block(SIA_WAVE);
+        dim3 grid(n_tokens, (n_heads + 3) / 4), block(4 * SIA_WAVE);
         if (dtype == SIA_F32)
             hipLaunchKernelGGL(bonus_finish_kernel<float>, grid, block, 0, stream, workspace, (const float*)rkvg, width, 0,
                                k_col, v_col, g_col, bonus, norm_w, (float*)out, n_heads, D, D, eps);

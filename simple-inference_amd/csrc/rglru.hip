@@ -52,27 +52,18 @@ __device__ __forceinline__ void rg_terms(float zr, float zi, float rate, float u
 // (begin + n) / 64 - begin / 64 + 1 chunks).
 __device__ __forceinline__ int rg_chunk_id(int run_begin, int seq, int chunk) { return run_begin / RG_CHUNK + seq + chunk; }
 
-// ---------------------------------------------------------------------------------------------------------------
-template <typename T, int V>
-__global__ __launch_bounds__(256) void rg_conv_kernel(const LinearUnit p, T* __restrict__ u) {
-    const int n = blockIdx.x, c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
-    if (c >= p.width) return;
-    const int seq = p.seq_of_token[n];
-    float acc[V], own[V];
-    ring_conv<T, V>((const T*)p.proj, p.row_stride, p.x_col + c, c, p.width, p.x_bias, p.conv, p.taps,
-                    p.state + (size_t)p.slots[seq] * p.state_stride + p.width, n, p.cu_q[seq], p.positions[n], acc, own);
-#pragma unroll
-    for (int e = 0; e < V; ++e) acc[e] += p.conv_bias[c + e];
-    T* dst = u + (size_t)n * p.width + c;
-    if constexpr (V == 8) {
-        Vec8<T> v;
-        v.set(acc);
-        v.store(dst);
-    } else {
-        dst[0] = from_float<T>(acc[0]);
+// The run that chunk ``id`` belongs to: the last one whose range starts at or before it (the ranges' starts grow strictly).
+__device__ __forceinline__ int rg_run_of(int id, const int* __restrict__ cu_q, int n_seqs) {
+    int lo = 0, hi = n_seqs - 1;
+    while (lo < hi) {
+        const int mid = (lo + hi + 1) / 2;
+        if (cu_q[mid] / RG_CHUNK + mid <= id) lo = mid;
+        else hi = mid - 1;
     }
+    return lo;
 }
 
+// ---------------------------------------------------------------------------------------------------------------
 // A thread a channel, eight tokens a workgroup.
 #define RG_TOKENS 8
 template <typename T>
@@ -107,10 +98,10 @@ __global__ __launch_bounds__(256) void rg_gates_kernel(const LinearUnit p, const
 
 // In place: decays become their running product from the chunk's start, what is written the chunk's own recurrence.
 __global__ __launch_bounds__(256) void rg_scan_kernel(const LinearUnit p, float* __restrict__ prod, float* __restrict__ local,
-                                                      float* __restrict__ end_prod, float* __restrict__ end_local,
-                                                      int max_chunks) {
-    const int seq = blockIdx.x / max_chunks, chunk = blockIdx.x % max_chunks, c = blockIdx.y * blockDim.x + threadIdx.x;
-    const int begin = p.cu_q[seq], t0 = begin + chunk * RG_CHUNK, t1 = min(t0 + RG_CHUNK, p.cu_q[seq + 1]);
+                                                      float* __restrict__ end_prod, float* __restrict__ end_local) {
+    const int c = blockIdx.y * blockDim.x + threadIdx.x;
+    const int seq = rg_run_of(blockIdx.x, p.cu_q, p.n_seqs), begin = p.cu_q[seq], chunk = blockIdx.x - rg_chunk_id(begin, seq, 0);
+    const int t0 = begin + chunk * RG_CHUNK, t1 = min(t0 + RG_CHUNK, p.cu_q[seq + 1]);
     if (c >= p.width || t0 >= t1) return;
     float A = 1.f, S = 0.f;
     for (int t = t0; t < t1; ++t) {
@@ -130,12 +121,12 @@ __global__ __launch_bounds__(256) void rg_scan_kernel(const LinearUnit p, float*
 __global__ __launch_bounds__(256) void rg_gates_mfma_kernel(const LinearUnit p, const bf16_t* __restrict__ u,
                                                             float* __restrict__ prod, float* __restrict__ local,
                                                             float* __restrict__ end_prod, float* __restrict__ end_local,
-                                                            int max_chunks, int tiles) {
+                                                            int tiles) {
     __shared__ __attribute__((aligned(16))) float a_s[RG_CHUNK][RG_PAD];
     __shared__ __attribute__((aligned(16))) float b_s[RG_CHUNK][RG_PAD];
     __shared__ float seg_a[4][64], seg_b[4][64];
-    const int seq = blockIdx.x / max_chunks, chunk = blockIdx.x % max_chunks;
-    const int begin = p.cu_q[seq], t0 = begin + chunk * RG_CHUNK, nt = min(RG_CHUNK, p.cu_q[seq + 1] - t0);
+    const int seq = rg_run_of(blockIdx.x, p.cu_q, p.n_seqs), begin = p.cu_q[seq], chunk = blockIdx.x - rg_chunk_id(begin, seq, 0);
+    const int t0 = begin + chunk * RG_CHUNK, nt = min(RG_CHUNK, p.cu_q[seq + 1] - t0);
     if (nt <= 0) return;      // uniform
     const int block = blockIdx.y / tiles, j0 = (blockIdx.y % tiles) * 64;      // channels j0 .. of the block
     const int wave = threadIdx.x / SIA_WAVE, lane = threadIdx.x % SIA_WAVE, r = lane & 15, g = lane >> 4;
@@ -299,6 +290,7 @@ __global__ __launch_bounds__(256) void rg_finish_kernel(const LinearUnit p, cons
 }
 
 // A step of single tokens, bfloat16: 16 channels of a block for up to 16 tokens.
+template <int TAPS>      // 0: any number
 __global__ __launch_bounds__(256) void rg_decode_kernel(const LinearUnit p, int tiles) {
     extern __shared__ __attribute__((aligned(16))) bf16_t u_s[];      // [16][bs + 8]
     __shared__ float part[4][16][17];
@@ -311,7 +303,10 @@ __global__ __launch_bounds__(256) void rg_decode_kernel(const LinearUnit p, int 
         if (m < M) {
             const int n = m0 + m, pos = p.positions[n];
             float* ring = p.state + (size_t)p.slots[p.seq_of_token[n]] * p.state_stride + p.width;
-            ring_conv<bf16_t, 8>(proj, p.row_stride, p.x_col + c, c, p.width, p.x_bias, p.conv, p.taps, ring, n, n, pos, acc, own);
+            if constexpr (TAPS > 0)
+                ring_conv_single<bf16_t, 8, TAPS>(proj, p.row_stride, p.x_col + c, c, p.width, p.x_bias, p.conv, ring, n, pos, acc, own);
+            else
+                ring_conv<bf16_t, 8>(proj, p.row_stride, p.x_col + c, c, p.width, p.x_bias, p.conv, p.taps, ring, n, n, pos, acc, own);
 #pragma unroll
             for (int e = 0; e < 8; ++e) acc[e] += p.conv_bias[c + e];
             // this workgroup's own channels: the input goes into the ring row that no token of the step reads
@@ -382,7 +377,13 @@ SIA_EXPORT int sia_linear_unit(const void* proj, int row_stride, int y_col, int 
     if (cores && max_q_len <= 1 && bs <= RG_MAX_BLOCK) {
         const int tiles = (bs + 15) / 16;
         dim3 grid(blocks * tiles, (n_tokens + 15) / 16), block(256);
-        hipLaunchKernelGGL(rg_decode_kernel, grid, block, (size_t)16 * (bs + 8) * sizeof(bf16_t), stream, p, tiles);
+        const size_t lds = (size_t)16 * (bs + 8) * sizeof(bf16_t);
+        const bool wide = state_stride % 4 == 0 && ((uintptr_t)state % 16) == 0;      // rows in 16-byte pieces
+        if (taps == 1) hipLaunchKernelGGL(rg_decode_kernel<1>, grid, block, lds, stream, p, tiles);
+        else if (taps == 2 && wide) hipLaunchKernelGGL(rg_decode_kernel<2>, grid, block, lds, stream, p, tiles);
+        else if (taps == 3 && wide) hipLaunchKernelGGL(rg_decode_kernel<3>, grid, block, lds, stream, p, tiles);
+        else if (taps == 4 && wide) hipLaunchKernelGGL(rg_decode_kernel<4>, grid, block, lds, stream, p, tiles);
+        else hipLaunchKernelGGL(rg_decode_kernel<0>, grid, block, lds, stream, p, tiles);
         return SIA_LAUNCH_CHECK();
     }
     const size_t w8 = (width + 7) / 8 * 8, chunks = (size_t)n_tokens / RG_CHUNK + n_seqs + 1;
@@ -391,25 +392,23 @@ SIA_EXPORT int sia_linear_unit(const void* proj, int row_stride, int y_col, int 
     float* local = prod + w8 * n_tokens;
     float* end_prod = local + w8 * n_tokens;
     float* end_local = end_prod + w8 * chunks;
-    const int max_chunks = (max_q_len + RG_CHUNK - 1) / RG_CHUNK;
-    if ((long long)n_seqs * max_chunks > 0x7fffffffLL) return SIA_BAD_ARGUMENT;
     const dim3 block(256), by8(n_tokens, (width / 8 + 255) / 256), by1(n_tokens, (width + 255) / 256);
     const RingColumns cols{{x_col, 0, 0}, {width, 0, 0}};
 #define RUN(T)                                                                                                       \
     do {                                                                                                             \
-        if (rows8) hipLaunchKernelGGL((rg_conv_kernel<T, 8>), by8, block, 0, stream, p, (T*)u);                      \
-        else hipLaunchKernelGGL((rg_conv_kernel<T, 1>), by1, block, 0, stream, p, (T*)u);                            \
+        launch_ring_conv<T>((const T*)proj, row_stride, cols, x_bias, conv, conv_bias, state, state_stride, width, taps, \
+                            cu_q, seq_of_token, positions, slots, (T*)u, width, n_tokens, rows8, stream);            \
         launch_ring_keep<T>((const T*)proj, row_stride, cols, x_bias, state, state_stride, width, taps, cu_q,        \
                             positions, slots, n_seqs, stream);                                                       \
         if (cores) {                                                                                                 \
             const int tiles = (bs + 63) / 64;                                                                        \
-            hipLaunchKernelGGL(rg_gates_mfma_kernel, dim3(n_seqs * max_chunks, blocks * tiles), block, 0, stream, p, \
-                               (const bf16_t*)u, prod, local, end_prod, end_local, max_chunks, tiles);               \
+            hipLaunchKernelGGL(rg_gates_mfma_kernel, dim3((unsigned)chunks, blocks * tiles), block, 0, stream, p,    \
+                               (const bf16_t*)u, prod, local, end_prod, end_local, tiles);                           \
         } else {                                                                                                     \
             hipLaunchKernelGGL(rg_gates_kernel<T>, dim3((n_tokens + RG_TOKENS - 1) / RG_TOKENS, (width + 255) / 256), \
                                block, 0, stream, p, (const T*)u, prod, local);                                       \
-            hipLaunchKernelGGL(rg_scan_kernel, dim3(n_seqs * max_chunks, (width + 255) / 256), block, 0, stream, p,  \
-                               prod, local, end_prod, end_local, max_chunks);                                        \
+            hipLaunchKernelGGL(rg_scan_kernel, dim3((unsigned)chunks, (width + 255) / 256), block, 0, stream, p,     \
+                               prod, local, end_prod, end_local);                                                    \
         }                                                                                                            \
         hipLaunchKernelGGL(rg_carry_kernel, dim3(n_seqs, (width + 63) / 64), dim3(64), 0, stream, p, end_prod, end_local); \
         if (rows8) hipLaunchKernelGGL((rg_finish_kernel<T, 8>), by8, block, 0, stream, p, prod, local, end_local);   \

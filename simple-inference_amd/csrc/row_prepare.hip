@@ -11,13 +11,17 @@
 // the token's place in its page (layout as in qk_prepare.hip).  q, k and v are runs of columns of the projected rows that
 // start anywhere; the channels of bias, convolution and ring are [q | k | v] without gaps.
 //
-// A workgroup takes a token's q and k: their convolved elements meet in LDS as floats, where norm and rotation find their
-// partners.  A second workgroup a token takes the values: where 8 or 16 consecutive tokens of a sequence fill an aligned run of a page, the
-// run's workgroups share its channels and each walks its channels over all the run's tokens, a window of inputs in
-// registers, and writes the run's positions (innermost in a page) at once.
+// In a step of single tokens the convolution is part of this kernel (the ring holds what it needs); a step of runs of tokens
+// is convolved first, by ring_conv.h's kernel into rows of their own (rounded once more, as a convolution's result may be).
+//
+// A workgroup takes a token's q and k.  Where neighbours turn together, a piece of eight elements is a thread's and the norm is
+// over the row (or absent), everything stays in registers and all loads are issued before the row's sums are taken
+// (``row_pieces_kernel``); else the elements meet in LDS as floats, where norm and rotation find their
+// partners.  The values are further workgroups' (16 tokens each, or one in a step of single tokens): where 8 or 16 consecutive
+// tokens of a sequence fill an aligned run of a page, the run's positions of a channel (innermost in a page) are written at
+// once.
 #include "ring_conv.h"
 
-#define ROWP_THREADS 256
 #define ROWP_MAX_ELEMENTS 15000       // q and k elements of a token (LDS)
 
 struct RowPrepare {
@@ -37,91 +41,192 @@ struct RowPrepare {
     long long state_stride;
     void *k_pages, *v_pages, *q_out;
     int n_tokens, n_heads, n_kv, head_dim, value_dim, page_size, k_row, v_rows, q_head_stride;
-    int v_group, single;
+    int v_group, v_tile, single;
 };
 
-// the run's values of one channel, position by position
-template <typename T>
-__device__ __forceinline__ void prepare_values(const RowPrepare& p, int n) {
+// TAPS: 0 the rows are convolved already (or there is no convolution); 1 to 4, or -1 for any number, the convolution of a
+// step of single tokens.
+template <typename T, int V, int TAPS>
+__device__ __forceinline__ void elements(const RowPrepare& p, int n, int pos, int at, int c, float* ring, float (&x)[V]) {
     const T* proj = (const T*)p.proj;
-    T* pages = (T*)p.v_pages;
-    const int pos = p.positions[n], seq = p.seq_of_token[n], first = p.cu_q[seq];
-    const int page = p.block_table[(size_t)seq * p.table_width + pos / p.page_size], off = pos % p.page_size;
-    if (page < 0) return;
-    const int channels = p.cols.channels(), c0 = p.cols.size[0] + p.cols.size[1], rows = p.cols.size[2];
-    float* ring = p.taps > 1 ? p.state + (size_t)p.slots[seq] * p.state_stride : nullptr;
-    auto at_page = [&](int i) {
-        return pages + (((size_t)page * p.n_kv + i / p.value_dim) * p.v_rows + i % p.value_dim) * p.page_size;
-    };
-    int place = 0, begin = n;
-    bool whole = false;
-    if (p.v_group > 0) {
-        place = off % p.v_group;
-        begin = n - place;
-        whole = begin >= first && begin + p.v_group <= p.cu_q[seq + 1];
-    }
-    if (!whole) {
-        for (int i = threadIdx.x; i < rows; i += ROWP_THREADS) {
-            float acc[1], own[1];
-            ring_conv<T, 1>(proj, p.row_stride, p.cols.col[2] + i, c0 + i, channels, p.bias, p.conv, p.taps, ring, n, first, pos, acc, own);
-            at_page(i)[off] = from_float<T>(acc[0]);
-            if (p.single && ring) ring[(size_t)(pos % p.taps) * channels + c0 + i] = own[0];
+    if constexpr (TAPS == 0) {
+        if constexpr (V == 8) {
+            Vec8<T> v;
+            v.load(proj + (size_t)n * p.row_stride + at);
+            v.get(x);
+        } else {
+            x[0] = to_float(proj[(size_t)n * p.row_stride + at]);
         }
-        return;
-    }
-    constexpr int MAX = 16, PER = 16 / sizeof(T);
-    const int slice = (rows + p.v_group - 1) / p.v_group;
-    for (int i = place * slice + threadIdx.x; i < min(rows, (place + 1) * slice); i += ROWP_THREADS) {
-        const int c = c0 + i;
-        const float add = p.bias ? p.bias[c] : 0.f;
-        float acc[MAX];
+        if (p.bias) {
 #pragma unroll
-        for (int m = 0; m < MAX; ++m) acc[m] = 0.f;
-        for (int j = 0; j < p.taps; ++j) {
-            const int back = p.taps - 1 - j;
-            const float w = p.conv ? p.conv[(size_t)j * channels + c] : 1.f;
-#pragma unroll
-            for (int m = 0; m < MAX; ++m) {
-                if (m >= p.v_group) continue;
-                const int src = begin + m - back, at = pos - place + m - back;
-                if (src >= first) acc[m] += w * (to_float(proj[(size_t)src * p.row_stride + p.cols.col[2] + i]) + add);
-                else if (at >= 0) acc[m] += w * ring[(size_t)(at % p.taps) * channels + c];
-            }
+            for (int e = 0; e < V; ++e) x[e] += p.bias[c + e];
         }
-        __attribute__((aligned(16))) T vals[MAX];
+    } else {
+        float own[V];
+        const int channels = p.cols.channels();
+        if constexpr (TAPS > 0)
+            ring_conv_single<T, V, TAPS>(proj, p.row_stride, at, c, channels, p.bias, p.conv, ring, n, pos, x, own);
+        else
+            ring_conv<T, V>(proj, p.row_stride, at, c, channels, p.bias, p.conv, p.taps, ring, n, n, pos, x, own);
+        if (p.taps > 1) {
+            float* row = ring + (size_t)(pos % p.taps) * channels + c;      // nobody reads this row in this step
 #pragma unroll
-        for (int m = 0; m < MAX; ++m) vals[m] = from_float<T>(acc[m]);
-        T* dst = at_page(i) + (off - place);
-#pragma unroll
-        for (int m = 0; m < MAX; m += PER)
-            if (m < p.v_group) *reinterpret_cast<uint4*>(dst + m) = *reinterpret_cast<const uint4*>(vals + m);
+            for (int e = 0; e < V; ++e) row[e] = own[e];
+        }
     }
 }
 
-template <typename T, int V>
-__global__ __launch_bounds__(ROWP_THREADS) void row_prepare_kernel(const RowPrepare p) {
-    extern __shared__ float row_s[];      // q and k elements; behind them a factor per head
-    __shared__ float scratch[16];
+template <typename T, int V, int TAPS>
+__device__ __forceinline__ void prepare_values(const RowPrepare& p, int n) {
+    const T* proj = (const T*)p.proj;
+    T* pages = (T*)p.v_pages;
+    const int pos = p.positions[n], seq = p.seq_of_token[n];
+    const int page = p.block_table[(size_t)seq * p.table_width + pos / p.page_size], off = pos % p.page_size;
+    if (page < 0) return;
+    const int c0 = p.cols.size[0] + p.cols.size[1], rows = p.cols.size[2];
+    auto at_page = [&](int i) {
+        return pages + (((size_t)page * p.n_kv + i / p.value_dim) * p.v_rows + i % p.value_dim) * p.page_size;
+    };
+    if (TAPS == 0 && p.v_group > 0) {
+        const int place = off % p.v_group, begin = n - place;
+        if (begin >= p.cu_q[seq] && begin + p.v_group <= p.cu_q[seq + 1]) {      // a whole run: its first token writes it
+            if (place != 0) return;
+            constexpr int MAX = 16, PER = 16 / sizeof(T);
+            for (int i = threadIdx.x; i < rows; i += blockDim.x) {
+                const float add = p.bias ? p.bias[c0 + i] : 0.f;
+                __attribute__((aligned(16))) T vals[MAX];
+#pragma unroll
+                for (int m = 0; m < MAX; ++m)
+                    vals[m] = m < p.v_group ? from_float<T>(to_float(proj[(size_t)(n + m) * p.row_stride + p.cols.col[2] + i]) + add) : T(0);
+                T* dst = at_page(i) + off;
+#pragma unroll
+                for (int m = 0; m < MAX; m += PER)
+                    if (m < p.v_group) *reinterpret_cast<uint4*>(dst + m) = *reinterpret_cast<const uint4*>(vals + m);
+            }
+            return;
+        }
+    }
+    float* ring = p.taps > 1 ? p.state + (size_t)p.slots[seq] * p.state_stride : nullptr;
+    for (int i = threadIdx.x * V; i < rows; i += blockDim.x * V) {
+        float x[V];
+        elements<T, V, TAPS>(p, n, pos, p.cols.col[2] + i, c0 + i, ring, x);
+#pragma unroll
+        for (int e = 0; e < V; ++e) at_page(i + e)[off] = from_float<T>(x[e]);
+    }
+}
+
+// The values of the tokens of value workgroup ``g``.
+template <typename T, int V, int TAPS>
+__device__ __forceinline__ void values_of(const RowPrepare& p, int g) {
+    for (int n = g * p.v_tile; n < min(p.n_tokens, (g + 1) * p.v_tile); ++n) prepare_values<T, V, TAPS>(p, n);
+}
+
+// Sums of two values over a workgroup, in one pass (``scratch``: 32 floats).
+__device__ __forceinline__ void block_sums(float& a, float& b, float* scratch) {
+    a = wave_sum(a);
+    b = wave_sum(b);
+    const int wave = threadIdx.x / SIA_WAVE, n_waves = blockDim.x / SIA_WAVE;
+    if (threadIdx.x % SIA_WAVE == 0) {
+        scratch[wave] = a;
+        scratch[16 + wave] = b;
+    }
+    __syncthreads();
+    a = b = 0.f;
+    for (int w = 0; w < n_waves; ++w) {
+        a += scratch[w];
+        b += scratch[16 + w];
+    }
+}
+
+// A thread a piece of eight q or k elements (at most 1,024 pieces): neighbours turn together, rotary_dim % 8 == 0.
+template <typename T, int TAPS>
+__global__ __launch_bounds__(1024) void row_pieces_kernel(const RowPrepare p) {
+    __shared__ float scratch[32];
     const int n = blockIdx.x, tid = threadIdx.x;
-    if (blockIdx.y == 1) {
-        prepare_values<T>(p, n);
+    if (n >= p.n_tokens) {
+        values_of<T, 8, TAPS>(p, n - p.n_tokens);
         return;
     }
-    const T* proj = (const T*)p.proj;
-    const int pos = p.positions[n], seq = p.seq_of_token[n], first = p.cu_q[seq];
-    const int channels = p.cols.channels(), nq = p.cols.size[0], nqk = nq + p.cols.size[1], D = p.head_dim;
+    const int nq = p.cols.size[0], nqk = nq + p.cols.size[1], D = p.head_dim, c = tid * 8;
+    const bool live = c < nqk, is_q = c < nq;
+    const int h = c / D, d0 = c % D;
+    const int pos = p.positions[n], seq = p.seq_of_token[n];
+    float* ring = p.taps > 1 ? p.state + (size_t)p.slots[seq] * p.state_stride : nullptr;
+    float x[8] = {};
+    Vec8<float> vg;
+    float4 vc, vs;
+    const bool turns = live && d0 < p.rotary_dim;
+    if (live) {
+        if (p.q_gain) vg.load(is_q ? p.q_gain + c : p.k_gain + c - nq);
+        if (turns) {
+            const size_t at = (size_t)pos * (p.rotary_dim / 2) + d0 / 2;
+            vc = *reinterpret_cast<const float4*>(p.cos_table + at);
+            vs = *reinterpret_cast<const float4*>(p.sin_table + at);
+        }
+        elements<T, 8, TAPS>(p, n, pos, is_q ? p.cols.col[0] + c : p.cols.col[1] + c - nq, c, ring, x);
+    }
+    if (p.q_gain) {      // uniform
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+        float sq = is_q ? ss : 0.f, sk = is_q ? 0.f : ss;
+        block_sums(sq, sk, scratch);
+        if (live) {
+            const float inv = is_q ? rsqrtf(sq / (float)nq + p.eps) : rsqrtf(sk / (float)(nqk - nq) + p.eps);
+            float gain[8];
+            vg.get(gain);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] *= inv * gain[e];
+        }
+    }
+    if (!live) return;
+    if (turns) {
+        const float co[4] = {vc.x, vc.y, vc.z, vc.w}, si[4] = {vs.x, vs.y, vs.z, vs.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const float a = x[2 * i], b = x[2 * i + 1];
+            x[2 * i] = a * co[i] - b * si[i];
+            x[2 * i + 1] = b * co[i] + a * si[i];
+        }
+    }
+    Vec8<T> v;
+    v.set(x);
+    if (is_q) {
+        T* head = (T*)p.q_out + ((size_t)n * p.n_heads + h) * p.q_head_stride;
+        v.store(head + d0);
+        if (d0 + 8 == D) {      // zeros between the heads
+            const float zero[8] = {};
+            v.set(zero);
+            for (int d = D; d < p.q_head_stride; d += 8) v.store(head + d);
+        }
+    } else {
+        const int page = p.block_table[(size_t)seq * p.table_width + pos / p.page_size];
+        if (page >= 0)
+            v.store((T*)p.k_pages + (((size_t)page * p.n_kv + h - p.n_heads) * p.page_size + pos % p.page_size) * p.k_row + d0);
+    }
+}
+
+template <typename T, int V, int TAPS>
+__global__ __launch_bounds__(1024) void row_prepare_kernel(const RowPrepare p) {
+    extern __shared__ float row_s[];      // q and k elements
+    __shared__ float scratch[16];
+    const int n = blockIdx.x, tid = threadIdx.x, threads = blockDim.x;
+    if (n >= p.n_tokens) {
+        values_of<T, V, TAPS>(p, n - p.n_tokens);
+        return;
+    }
+    const int pos = p.positions[n], seq = p.seq_of_token[n];
+    const int nq = p.cols.size[0], nqk = nq + p.cols.size[1], D = p.head_dim;
     float* ring = p.taps > 1 ? p.state + (size_t)p.slots[seq] * p.state_stride : nullptr;
     float ss_q = 0.f, ss_k = 0.f;
-    for (int c = tid * V; c < nqk; c += ROWP_THREADS * V) {
-        float acc[V], own[V];
-        const int at = c < nq ? p.cols.col[0] + c : p.cols.col[1] + c - nq;
-        ring_conv<T, V>(proj, p.row_stride, at, c, channels, p.bias, p.conv, p.taps, ring, n, first, pos, acc, own);
+    for (int c = tid * V; c < nqk; c += threads * V) {
+        float x[V];
+        elements<T, V, TAPS>(p, n, pos, c < nq ? p.cols.col[0] + c : p.cols.col[1] + c - nq, c, ring, x);
         float ss = 0.f;
 #pragma unroll
         for (int e = 0; e < V; ++e) {
-            row_s[c + e] = acc[e];
-            ss += acc[e] * acc[e];
-            if (p.single && ring) ring[(size_t)(pos % p.taps) * channels + c + e] = own[e];
+            row_s[c + e] = x[e];
+            ss += x[e] * x[e];
         }
         if (c < nq) ss_q += ss;
         else ss_k += ss;
@@ -130,13 +235,13 @@ __global__ __launch_bounds__(ROWP_THREADS) void row_prepare_kernel(const RowPrep
         ss_q = block_sum(ss_q, scratch);
         ss_k = block_sum(ss_k, scratch);
         const float iq = rsqrtf(ss_q / (float)nq + p.eps), ik = rsqrtf(ss_k / (float)(nqk - nq) + p.eps);
-        for (int c = tid * V; c < nqk; c += ROWP_THREADS * V)      // a thread's own elements
+        for (int c = tid * V; c < nqk; c += threads * V)      // a thread's own elements
 #pragma unroll
             for (int e = 0; e < V; ++e) row_s[c + e] *= c < nq ? iq * p.q_gain[c + e] : ik * p.k_gain[c + e - nq];
     } else if (p.q_gain) {
         __syncthreads();
         const int wave = tid / SIA_WAVE, lane = tid % SIA_WAVE;
-        for (int h = wave; h < p.n_heads + p.n_kv; h += ROWP_THREADS / SIA_WAVE) {
+        for (int h = wave; h < p.n_heads + p.n_kv; h += threads / SIA_WAVE) {
             float ss = 0.f;
             for (int d = lane; d < D; d += SIA_WAVE) ss += row_s[h * D + d] * row_s[h * D + d];
             const float inv = rsqrtf(wave_sum(ss) / (float)D + p.eps);
@@ -148,7 +253,7 @@ __global__ __launch_bounds__(ROWP_THREADS) void row_prepare_kernel(const RowPrep
     const int page = p.block_table[(size_t)seq * p.table_width + pos / p.page_size], off = pos % p.page_size;
     const int half = p.rotary_dim / 2;
     const float *cs = p.cos_table + (size_t)pos * half, *sn = p.sin_table + (size_t)pos * half;
-    for (int c = tid * V; c < nqk; c += ROWP_THREADS * V) {
+    for (int c = tid * V; c < nqk; c += threads * V) {
         const int h = c / D, d0 = c % D;      // V divides D: a piece lies in one head
         float x[V];
 #pragma unroll
@@ -181,14 +286,15 @@ __global__ __launch_bounds__(ROWP_THREADS) void row_prepare_kernel(const RowPrep
     }
     const int gap = p.q_head_stride - D;      // zeros between the heads of q
     if (gap > 0)
-        for (int i = tid; i < p.n_heads * gap; i += ROWP_THREADS)
+        for (int i = tid; i < p.n_heads * gap; i += threads)
             ((T*)p.q_out)[((size_t)n * p.n_heads + i / gap) * p.q_head_stride + D + i % gap] = from_float<T>(0.f);
 }
 
 SIA_EXPORT int sia_row_prepare_max_elements() { return ROWP_MAX_ELEMENTS; }
 
 // q_col, k_col, v_col: where the three runs of columns start; state: ring of taps rows of [q | k | v] channels (null with
-// one tap); conv [taps][channels] or null (taps must then be 1); neighbours: which elements the rotation pairs.
+// one tap); conv [taps][channels] or null (taps must then be 1), bias must come with it; neighbours: which elements the
+// rotation pairs; convolved: room for the convolved rows of a step of runs of tokens, [tokens][channels, rounded up to 8].
 SIA_EXPORT int sia_row_prepare(const void* proj, int row_stride, int q_col, int k_col, int v_col, const float* bias,
                                const float* conv, int taps, const float* q_gain, const float* k_gain, float eps,
                                int over_row, const float* cos_table, const float* sin_table, int rotary_dim,
@@ -196,13 +302,14 @@ SIA_EXPORT int sia_row_prepare(const void* proj, int row_stride, int q_col, int 
                                const int* slots, const int* block_table, int table_width, float* state,
                                long long state_stride, void* k_pages, void* v_pages, void* q_out, int n_tokens,
                                int n_seqs, int max_q_len, int n_heads, int n_kv, int head_dim, int value_dim,
-                               int page_size, int k_row, int v_rows, int q_head_stride, int dtype, hipStream_t stream) {
+                               int page_size, int k_row, int v_rows, int q_head_stride, void* convolved, int dtype,
+                               hipStream_t stream) {
     if (n_tokens <= 0 || n_seqs <= 0) return 0;
     RowPrepare p{};
     p.cols = RingColumns{{q_col, k_col, v_col}, {n_heads * head_dim, n_kv * head_dim, n_kv * value_dim}};
     const int nqk = p.cols.size[0] + p.cols.size[1];
     if (n_heads <= 0 || n_kv <= 0 || head_dim <= 0 || value_dim <= 0 || nqk > ROWP_MAX_ELEMENTS || taps < 1 ||
-        taps > RING_MAX_TAPS || (taps > 1 && (!conv || !state || state_stride < (long long)taps * p.cols.channels())) ||
+        taps > RING_MAX_TAPS || (conv && (!bias || (max_q_len > 1 && !convolved))) || (taps > 1 && (!conv || !state || state_stride < (long long)taps * p.cols.channels())) ||
         rotary_dim < 0 || rotary_dim > head_dim || (rotary_dim & 1) || (rotary_dim > 0 && (!cos_table || !sin_table)) ||
         (q_gain == nullptr) != (k_gain == nullptr) || !k_pages || !v_pages || !q_out || !block_table || page_size <= 0 ||
         k_row < head_dim || v_rows < value_dim || q_head_stride < head_dim || (dtype != SIA_F32 && dtype != SIA_BF16))
@@ -244,20 +351,60 @@ SIA_EXPORT int sia_row_prepare(const void* proj, int row_stride, int q_col, int 
     p.q_head_stride = q_head_stride;
     p.single = max_q_len <= 1;
     p.v_group = p.single ? 0 : page_size % 16 == 0 ? 16 : page_size % 8 == 0 ? 8 : 0;
-    const bool vec = head_dim % 8 == 0 && row_stride % 8 == 0 && q_col % 8 == 0 && k_col % 8 == 0 && k_row % 8 == 0 &&
-                     q_head_stride % 8 == 0 && ((uintptr_t)proj % 16) == 0;
-    dim3 grid(n_tokens, 2), block(ROWP_THREADS);
+    bool vec = head_dim % 8 == 0 && value_dim % 8 == 0 && row_stride % 8 == 0 && q_col % 8 == 0 && k_col % 8 == 0 &&
+               v_col % 8 == 0 && k_row % 8 == 0 && q_head_stride % 8 == 0 && ((uintptr_t)proj % 16) == 0;
+    if (conv && !p.single) {      // convolved first, the projection's bias included
+        const int channels = p.cols.channels(), wide = (channels + 7) / 8 * 8;
+#define CONVOLVE(T)                                                                                                  \
+    do {                                                                                                             \
+        launch_ring_conv<T>((const T*)proj, row_stride, p.cols, bias, conv, nullptr, state, state_stride, 0, taps, cu_q, \
+                            seq_of_token, positions, slots, (T*)convolved, wide, n_tokens, vec, stream);             \
+        launch_ring_keep<T>((const T*)proj, row_stride, p.cols, bias, state, state_stride, 0, taps, cu_q, positions, \
+                            slots, n_seqs, stream);                                                                  \
+    } while (0)
+        if (dtype == SIA_F32) CONVOLVE(float);
+        else CONVOLVE(bf16_t);
+#undef CONVOLVE
+        p.proj = convolved;
+        p.row_stride = wide;
+        p.cols.col[0] = 0;
+        p.cols.col[1] = p.cols.size[0];
+        p.cols.col[2] = nqk;
+        p.bias = nullptr;
+        p.conv = nullptr;
+        p.taps = 1;
+    } else if (conv && taps > 1 && (state_stride % 4 != 0 || ((uintptr_t)state % 16) != 0)) {
+        vec = false;      // the ring's rows are read in 16-byte pieces
+    }
+    const int pieces = vec ? nqk / 8 : nqk;
+    int threads = (pieces + SIA_WAVE - 1) / SIA_WAVE * SIA_WAVE;
+    threads = threads > 1024 ? 1024 : threads;
+    if (!p.single && threads > 512) threads = 512;
+    // the form that stays in registers
+    const bool pieces_fit = vec && pieces <= 1024 && (rotary_dim == 0 || neighbours) && rotary_dim % 8 == 0 && (!q_gain || over_row) &&
+                            (rotary_dim == 0 || (((uintptr_t)cos_table % 16) == 0 && ((uintptr_t)sin_table % 16) == 0));
+    if (pieces_fit) threads = (pieces + SIA_WAVE - 1) / SIA_WAVE * SIA_WAVE;
+    p.v_tile = p.single ? 1 : 16;
+    dim3 grid(n_tokens + (n_tokens + p.v_tile - 1) / p.v_tile), block(threads);
     const size_t lds = (size_t)nqk * sizeof(float);
+#define LAUNCH_AS(T, TAPS)                                                                             \
+    do {                                                                                               \
+        if (pieces_fit) hipLaunchKernelGGL((row_pieces_kernel<T, TAPS>), grid, block, 0, stream, p);   \
+        else if (vec) hipLaunchKernelGGL((row_prepare_kernel<T, 8, TAPS>), grid, block, lds, stream, p); \
+        else hipLaunchKernelGGL((row_prepare_kernel<T, 1, TAPS>), grid, block, lds, stream, p);        \
+    } while (0)
 #define LAUNCH(T)                                                                                      \
     do {                                                                                               \
-        if (vec) hipLaunchKernelGGL((row_prepare_kernel<T, 8>), grid, block, lds, stream, p);          \
-        else hipLaunchKernelGGL((row_prepare_kernel<T, 1>), grid, block, lds, stream, p);              \
-        if (!p.single)                                                                                 \
-            launch_ring_keep<T>((const T*)proj, row_stride, p.cols, bias, state, state_stride, 0, taps, cu_q, positions, \
-                                slots, n_seqs, stream);                                                \
+        if (!p.conv) LAUNCH_AS(T, 0);                                                                  \
+        else if (taps == 1) LAUNCH_AS(T, 1);                                                           \
+        else if (taps == 2) LAUNCH_AS(T, 2);                                                           \
+        else if (taps == 3) LAUNCH_AS(T, 3);                                                           \
+        else if (taps == 4) LAUNCH_AS(T, 4);                                                           \
+        else LAUNCH_AS(T, -1);                                                                         \
     } while (0)
     if (dtype == SIA_F32) LAUNCH(float);
     else LAUNCH(bf16_t);
 #undef LAUNCH
+#undef LAUNCH_AS
     return SIA_LAUNCH_CHECK();
 }

@@ -39,7 +39,7 @@ _SIGNATURES = {
     "sia_row_prepare": [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float, _c_int,
                         _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ll,
                         _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                        _c_int, _c_int, _c_int, _c_ptr],
+                        _c_int, _c_int, _c_ptr, _c_int, _c_ptr],
     "sia_linear_unit_max_taps": [],
     "sia_linear_unit_workspace": [_c_int, _c_int, _c_int],
     "sia_linear_unit": [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
@@ -1785,13 +1785,19 @@ class HipKernels:
         v_rows = page_dim or value_dim
         self._check_pages(cache.k_pages, cache.v_pages, cache.block_table, cache.page_size, n_kv, wide, proj.dtype, ctx, v_rows)
         q = torch.empty((n, n_heads * wide), dtype=proj.dtype, device=proj.device)
+        convolved = None
+        if conv is not None:
+            if bias is None:
+                bias = torch.zeros(channels, dtype=torch.float32, device=proj.device)
+            if ctx.max_q_len > 1:      # a step of runs of tokens is convolved by a kernel of its own
+                convolved = torch.empty((n, channels + (-channels) % 8), dtype=proj.dtype, device=proj.device)
         self._check(self.core.sia_row_prepare(
             _ptr(proj), stride, *(int(c) for c in columns), _ptr(bias), _ptr(conv), taps, _ptr(q_gain), _ptr(k_gain),
             float(eps), int(over == "row"), _ptr(cos) if rotary_dim else None, _ptr(sin) if rotary_dim else None, rotary_dim,
             int(pairing == "interleaved"), _ptr(ctx.positions), _ptr(ctx.seq_of_token), _ptr(ctx.cu_q), _ptr(ctx.state_slots),
             _ptr(cache.block_table), cache.block_table.shape[1], _ptr(state), row, _ptr(cache.k_pages), _ptr(cache.v_pages),
             _ptr(q), n, ctx.n_seqs, ctx.max_q_len, n_heads, n_kv, head_dim, value_dim, cache.page_size, wide, v_rows, wide,
-            _DT[proj.dtype], self._stream()), "row_prepare")
+            _ptr(convolved), _DT[proj.dtype], self._stream()), "row_prepare")
         return q
 
     def _check_pages(self, k_pages, v_pages, table, page_size, n_kv, head_dim, dtype, ctx, value_dim=None):
